@@ -46,6 +46,17 @@ def add_rms_norm(stream, rows, gain_post, eps_post, gain_next, eps_next, out_dty
     return _norm(stream, gain_next, eps_next, groups).to(out_dtype)
 
 
+def join_rms_norm(stream, a, b, gain, eps, out_dtype, vec=None, origin=None):
+    for r in (a, b):
+        if r is not None:
+            stream += r.slices.sum(0) if hasattr(r, "slices") else r.float()
+    if origin is not None:
+        stream += origin
+    if vec is not None:
+        stream += vec
+    return None if gain is None else _norm(stream, gain, eps).to(out_dtype)
+
+
 def scale_rows(x, scale):
     x *= scale
 
@@ -100,27 +111,35 @@ def head_linear(x, w, out=None):
     return out
 
 
-def route_top(logits, top, renormalize=False, score="softmax"):
+def route_top(logits, top, renormalize=False, score="softmax", correction=None, scale=1.0):
     s = torch.softmax(logits.float(), dim=-1) if score == "softmax" else torch.sigmoid(logits.float())
-    order = torch.argsort(-s, dim=-1, stable=True)[:, :top]
+    order = torch.argsort(-(s if correction is None else s + correction), dim=-1, stable=True)[:, :top]
     w = torch.gather(s, 1, order)
     if renormalize:
-        w = w / w.sum(-1, keepdim=True)
-    return order.to(torch.int32), w
+        w = w / (w.sum(-1, keepdim=True) + 1e-20)
+    return order.to(torch.int32), w * scale
 
 
-def expert_ffn(x, chosen, weights, w_gate_up, w_down, limit, alpha, shift, weight_input=False, out=None):
+def expert_ffn(x, chosen, weights, w_gate_up, w_down, limit, alpha, shift, weight_input=False, out=None, kind="gated"):
     """fp32 [M, D]: sum over a token's chosen experts, in the order they were chosen, of weight * expert(x), or
-    (weight_input) of expert(weight * x): gate and up sums times the weight, before the clamps."""
+    (weight_input) of expert(weight * x): gate and up sums times the weight, before the clamps.  kind "relu2":
+    max(W_up x, 0)^2 in the gated unit's place.  A choice beyond the matrices is the row itself."""
     m, ff = x.shape[0], w_gate_up.shape[1] // 2
     limit = float("inf") if limit is None else limit
     res = torch.zeros((m, w_down.shape[1]), dtype=torch.float32, device=x.device)
     for k in range(chosen.shape[1]):
         for r in range(m):
             e = int(chosen[r, k])
+            if e >= w_gate_up.shape[0]:
+                res[r] += weights[r, k] * x[r].float()
+                continue
             gu = w_gate_up[e].float() @ x[r].float()
             if weight_input:
                 gu = gu * weights[r, k]
+            if kind == "relu2":
+                y = (torch.clamp(gu, min=0.0) ** 2).to(x.dtype).float()
+                res[r] += (1.0 if weight_input else weights[r, k]) * (w_down[e].float() @ y)
+                continue
             g, u = torch.clamp(gu[:ff], max=limit), torch.clamp(gu[ff:], -limit, limit)
             y = (g * torch.sigmoid(alpha * g) * (u + shift)).to(x.dtype).float()
             res[r] += (1.0 if weight_input else weights[r, k]) * (w_down[e].float() @ y)
@@ -128,6 +147,11 @@ def expert_ffn(x, chosen, weights, w_gate_up, w_down, limit, alpha, shift, weigh
         return res
     out.copy_(res)
     return out
+
+
+def linear_act(x, w, out_dtype, activation):
+    assert activation == "relu2"
+    return (torch.clamp(x.float() @ w.float().T, min=0.0) ** 2).to(out_dtype)
 
 
 def linear(x, w, out_dtype, softcap=None, defer=False, bias=None, out=None):
@@ -173,15 +197,22 @@ def _rotate(x, pos, inv_freq, rotary_dim, pairing="halves"):
     return torch.cat([x0 * c - x1 * s, x1 * c + x0 * s, x[..., rotary_dim:]], dim=-1)
 
 
-def _cache_rows(k, v, row_seq, row_pos, new_len, table, k_pool, v_pool, rows_cap):
+def _row_of(p, rows_cap, pin):
+    """The cache row of position p: the first `pin` stay, the others take the rest of the ring's rows in turn."""
+    return p if not rows_cap or p < pin else pin + (p - pin) % (rows_cap - pin)
+
+
+def _rows_of(pos, rows_cap, pin):
+    return torch.tensor([_row_of(int(p), rows_cap, pin) for p in pos], dtype=torch.long)
+
+
+def _cache_rows(k, v, row_seq, row_pos, new_len, table, k_pool, v_pool, rows_cap, pin=0):
     KV, page, hd = k_pool.shape[1], k_pool.shape[2], k_pool.shape[3]
     for r in range(k.shape[0]):
         s, p = int(row_seq[r]), int(row_pos[r])
-        row = p
-        if rows_cap:
-            if p + rows_cap < int(new_len[s]):
-                continue                                  # a later row of this step lands on the same ring row
-            row = p % rows_cap
+        if rows_cap and p >= pin and p + rows_cap - pin < int(new_len[s]):
+            continue                                      # a later row of this step lands on the same ring row
+        row = _row_of(p, rows_cap, pin)
         pg = int(table[s, row // page])
         assert pg >= 0
         k_pool[pg, :, row % page, :] = k[r].reshape(KV, hd)
@@ -189,18 +220,18 @@ def _cache_rows(k, v, row_seq, row_pos, new_len, table, k_pool, v_pool, rows_cap
 
 
 def rope_kv_write(q, k, v, H, KV, hd, inv_freq, rotary_dim, row_seq, row_pos, new_len, table,
-                  k_pool, v_pool, rows_cap, pairing="halves", write=True):
+                  k_pool, v_pool, rows_cap, pairing="halves", write=True, pin=0):
     m = q.shape[0]
     q.copy_(_rotate(q.float().reshape(m, H, hd), row_pos, inv_freq, rotary_dim, pairing).reshape(m, H * hd).to(q.dtype))
     if k is None:
         return
     k.copy_(_rotate(k.float().reshape(m, KV, hd), row_pos, inv_freq, rotary_dim, pairing).reshape(m, KV * hd).to(k.dtype))
     if write:
-        _cache_rows(k, v, row_seq, row_pos, new_len, table, k_pool, v_pool, rows_cap)
+        _cache_rows(k, v, row_seq, row_pos, new_len, table, k_pool, v_pool, rows_cap, pin)
 
 
-def kv_write(k, v, KV, hd, row_seq, row_pos, new_len, table, k_pool, v_pool, rows_cap):
-    _cache_rows(k, v, row_seq, row_pos, new_len, table, k_pool, v_pool, rows_cap)
+def kv_write(k, v, KV, hd, row_seq, row_pos, new_len, table, k_pool, v_pool, rows_cap, pin=0):
+    _cache_rows(k, v, row_seq, row_pos, new_len, table, k_pool, v_pool, rows_cap, pin)
 
 
 def _attend(qrow, keys, vals, scale, softcap, sink=None):
@@ -214,13 +245,19 @@ def _attend(qrow, keys, vals, scale, softcap, sink=None):
     return p @ vals
 
 
+def _positions_seen(p, window, chunk, keep):
+    """The positions a query at p sees: its window's (or chunk's), and the first `keep`."""
+    lo = _first_seen(p, window, chunk)
+    return torch.cat([torch.arange(0, min(keep, lo)), torch.arange(lo, p + 1)])
+
+
 def _first_seen(p, window, chunk):
     lo = 0 if not window else max(0, p - window + 1)
     return max(lo, (p // chunk) * chunk) if chunk else lo
 
 
 def attention_prefill(q, k, v, H, KV, hd, cu_rows, max_count, scale, softcap, window, out_dtype, row_seq=None, row_pos=None,
-                      cached=None, shape=0, wide_weights=False, chunk=0, head_scale=None, sink=None):
+                      cached=None, shape=0, wide_weights=False, chunk=0, head_scale=None, sink=None, keep=0, pin=0):
     """k, v: the step's own rows.  cached None: every sequence starts at position 0.  Else cached = (new_len, table,
     k_pool, v_pool, rows_cap): sequence i's first row stands at new_len[i] - its count, and the positions before it are
     read from the cache as it is."""
@@ -236,17 +273,19 @@ def attention_prefill(q, k, v, H, KV, hd, cu_rows, max_count, scale, softcap, wi
             page = k_pool.shape[2]
             start = int(new_len[i]) - (b - a)
             first = _first_seen(start, window, chunk)                    # the earliest position any query of the step sees
-            pos = torch.arange(first, start)
-            rows = pos % rows_cap if rows_cap else pos
-            pages = table[i].long()[rows // page]
+            pos = torch.cat([torch.arange(0, min(keep, first, start)), torch.arange(first, start)])
+            rows = _rows_of(pos, rows_cap, pin)
+            pages = table[i].long().cpu()[rows // page]
             assert (pages >= 0).all()
-            keys = torch.cat([torch.zeros(first, KV, hd), k_pool[pages, :, rows % page, :].float().cpu(), kf[a:b].cpu()]).to(q.device)
-            vals = torch.cat([torch.zeros(first, KV, hd), v_pool[pages, :, rows % page, :].float().cpu(), vf[a:b].cpu()]).to(q.device)
+            past = torch.zeros((2, start, KV, hd))
+            past[0, pos], past[1, pos] = k_pool.cpu()[pages, :, rows % page, :].float(), v_pool.cpu()[pages, :, rows % page, :].float()
+            keys = torch.cat([past[0], kf[a:b].cpu()]).to(q.device)
+            vals = torch.cat([past[1], vf[a:b].cpu()]).to(q.device)
         for r in range(a, b):
             p = start + r - a
-            lo = _first_seen(p, window, chunk)
+            see = _positions_seen(p, window, chunk, keep).to(q.device)
             for h in range(H):
-                out[r, h * hd:(h + 1) * hd] = _attend(qf[r, h], keys[lo:p + 1, h // g], vals[lo:p + 1, h // g],
+                out[r, h * hd:(h + 1) * hd] = _attend(qf[r, h], keys[see, h // g], vals[see, h // g],
                                                       scale * (float(head_scale[h]) if head_scale is not None else 1.0), softcap,
                                                       None if sink is None else sink[h])
     return out.to(out_dtype)
@@ -257,7 +296,7 @@ def decode_splits(n, KV, hd, keys):
 
 
 def attention_decode(q, H, KV, hd, new_len, table, k_pool, v_pool, rows_cap, scale, softcap, window, out_dtype, max_keys=None, splits=None, head_groups=None,
-                     chunk=0, head_scale=None, sink=None):
+                     chunk=0, head_scale=None, sink=None, keep=0, pin=0):
     n = q.shape[0]
     page = k_pool.shape[2]
     out = torch.zeros((n, H * hd), dtype=torch.float32, device=q.device)
@@ -265,9 +304,7 @@ def attention_decode(q, H, KV, hd, new_len, table, k_pool, v_pool, rows_cap, sca
     g = H // KV
     for i in range(n):
         p = int(new_len[i]) - 1
-        lo = _first_seen(p, window, chunk)
-        pos = torch.arange(lo, p + 1)
-        rows = pos % rows_cap if rows_cap else pos
+        rows = _rows_of(_positions_seen(p, window, chunk, keep), rows_cap, pin).to(q.device)
         pages = table[i].long()[rows // page]
         assert (pages >= 0).all()
         keys = k_pool[pages, :, rows % page, :].float()          # [n_keys, KV, hd]
@@ -284,7 +321,7 @@ def fuses_decode_step(dtype, H, KV, hd, k_pool):
 
 
 def attention_decode_step(qkv, H, KV, hd, inv_freq, rotary_dim, new_len, table, k_pool, v_pool, rows_cap, scale, softcap,
-                          window, out_dtype, max_keys=None, write_kv=True, splits=None):
+                          window, out_dtype, max_keys=None, write_kv=True, splits=None, sink=None, keep=0, pin=0):
     """The fused decode step as its three parts: qkv float32 [n, (H + 2 KV) hd] (already summed over K slices),
     rotated in float32 and rounded once to the cache's dtype."""
     n = qkv.shape[0]
@@ -295,12 +332,12 @@ def attention_decode_step(qkv, H, KV, hd, inv_freq, rotary_dim, new_len, table, 
         v = qkv[:, (H + KV) * hd:].reshape(n, KV, hd).to(k_pool.dtype)
         page = k_pool.shape[2]
         for i in range(n):
-            row = int(pos[i]) % rows_cap if rows_cap else int(pos[i])
+            row = _row_of(int(pos[i]), rows_cap, pin)
             pg = int(table[i, row // page])
             assert pg >= 0
             k_pool[pg, :, row % page, :] = k[i]
             v_pool[pg, :, row % page, :] = v[i]
-    return attention_decode(q, H, KV, hd, new_len, table, k_pool, v_pool, rows_cap, scale, softcap, window, out_dtype)
+    return attention_decode(q, H, KV, hd, new_len, table, k_pool, v_pool, rows_cap, scale, softcap, window, out_dtype, sink=sink, keep=keep, pin=pin)
 
 
 class SplitRows:
@@ -421,6 +458,32 @@ def matrix_memory_scan(q, k, v, gates, cap, q_scale, memory, normalizer, maximum
             den = torch.maximum((n * qf[t]).sum(-1).abs(), torch.exp(-mx)) + 1e-6
             y[t] = torch.einsum("hkv,hk->hv", S, qf[t]) / den[:, None]
         memory[slot], normalizer[slot], maximum[slot] = S, n, mx
+    return y.reshape(M, heads * dv).float()
+
+
+def delta_scan(q, k, v, b, a, a_log, dt_bias, state, slot_ids, cu_rows, max_count, heads, kv_heads, dk, dv, q_scale, chunks=None):
+    """S <- g S, u = beta (v - S^T k), S <- S + k u^T, o = S^T q, row after row of every sequence from state[slot] [heads, dk,
+    dv], which is left updated; k and q unit vectors, q times q_scale, beta = sigmoid(b), g = exp(-exp(a_log) softplus(a + dt_bias))."""
+    M = q.shape[0]
+    wide = state.dtype                                   # float64 states: the whole recurrence in float64
+    per = heads // kv_heads
+
+    def unit(x):
+        x = x.to(wide).reshape(M, kv_heads, dk)
+        return (x / torch.sqrt((x * x).sum(-1, keepdim=True) + 1e-6)).repeat_interleave(per, dim=1)
+    qf, kf, vf = unit(q) * q_scale, unit(k), v.to(wide).reshape(M, heads, dv)
+    beta = torch.sigmoid(b.to(wide))
+    decay = torch.exp(-torch.exp(a_log.to(wide)) * torch.nn.functional.softplus(a.to(wide) + dt_bias.to(wide), threshold=1e9))
+    y = torch.empty((M, heads, dv), dtype=wide, device=q.device)
+    for s in range(len(cu_rows) - 1):
+        slot = int(slot_ids[s])
+        S = state[slot].clone()
+        for t in range(int(cu_rows[s]), int(cu_rows[s + 1])):
+            S = decay[t][:, None, None] * S
+            u = beta[t][:, None] * (vf[t] - (S * kf[t][:, :, None]).sum(1))
+            S = S + kf[t][:, :, None] * u[:, None, :]
+            y[t] = (S * qf[t][:, :, None]).sum(1)
+        state[slot] = S
     return y.reshape(M, heads * dv).float()
 
 

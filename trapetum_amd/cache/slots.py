@@ -49,9 +49,12 @@ class GroupPages:
     """Pages of one group of layers: a pool and each slot's page list.
 
     `rows_cap`: None if a sequence keeps every row, else the number of rows of its
-    ring (position p lives in ring row p % rows_cap).  `every`: tokens per row (a row exists once its last token does)."""
+    ring (position p lives in ring row p % rows_cap).  `pinned`: of these, the rows in front of the ring that
+    keep a sequence's first tokens (position p >= pinned then lives in row pinned + (p - pinned) % (rows_cap - pinned)).
+    `every`: tokens per row (a row exists once its last token does)."""
 
-    def __init__(self, n_pages, page_size, rows_cap, name, every=1):
+    def __init__(self, n_pages, page_size, rows_cap, name, every=1, pinned=0):
+        self.pinned = pinned
         self.page_size = page_size
         self.rows_cap = rows_cap
         self.every = every

@@ -10,6 +10,9 @@ its own:
                stand before the last dimension, so that a row of d elements is
                contiguous); a sequence's rows are found through its page list.  A
                window group keeps a ring: position p lives in ring row p % rows_cap.
+               (A window that keeps a sequence's first tokens as well has whole pages of
+               `pinned` rows for them in front of the ring: positions below `pinned` stay
+               in their rows, the others take the rows behind them in turn.)
                (Attention declares keys and values, each (kv_heads, head_dim); a
                mixer that keeps one tensor per token declares one.)
   state        [entries, slots, *shape], zeroed when a slot is taken.
@@ -38,16 +41,19 @@ class TokenSpec:
     window: Optional[int] = None        # None: every token is kept
     every: int = 1                      # one row per `every` tokens: row b belongs to the positions b * every .. b * every + every - 1
                                         # and exists once the last of them does (a summary of a block of tokens)
+    keep_first: int = 0                 # beside the window, the first `keep_first` tokens of a sequence are kept for good
 
     @staticmethod
-    def of(window=None, every=1, **tensors):
+    def of(window=None, every=1, keep_first=0, **tensors):
         """TokenSpec.of(window, k=(kv_heads, head_dim), v=(kv_heads, head_dim))"""
         for name, shape in tensors.items():
             if not shape or any(int(n) <= 0 for n in shape):
                 raise CacheError(f"per-token tensor '{name}' needs a shape of positive sizes, found {shape!r}")
         if int(every) < 1 or (int(every) > 1 and window is not None):
             raise CacheError(f"a row per {every} tokens: the number must be positive, and such rows are kept of all tokens, not of a window")
-        return TokenSpec(tuple((name, tuple(int(n) for n in shape)) for name, shape in tensors.items()), window, int(every))
+        if int(keep_first) < 0 or (int(keep_first) > 0 and window is None):
+            raise CacheError(f"{keep_first} first tokens are kept beside a window: the number must not be negative, and there must be a window")
+        return TokenSpec(tuple((name, tuple(int(n) for n in shape)) for name, shape in tensors.items()), window, int(every), int(keep_first))
 
     def shape_of(self, name):
         for n, shape in self.tensors:
@@ -85,6 +91,11 @@ class CacheSite:
         return self._group.pages.rows_cap
 
     @property
+    def pinned(self):
+        """Rows in front of the ring that keep a sequence's first tokens (0 without a ring)."""
+        return self._group.pages.pinned
+
+    @property
     def state(self):
         return self._group.tensor[self.index_in_group]
 
@@ -93,13 +104,14 @@ class _TokenGroup:
     def __init__(self, spec, entries, n_pages, max_slots, page_size, max_context, dtype, device, name):
         self.spec = spec
         self.entries = entries
-        rows_cap = None
+        rows_cap, pinned = None, 0
         if spec.window is not None and spec.window < max_context:
-            rows_cap = -(-spec.window // page_size) * page_size
+            pinned = -(-spec.keep_first // page_size) * page_size            # whole pages, so that a page is of one kind
+            rows_cap = pinned + -(-spec.window // page_size) * page_size
             n_pages = min(n_pages, max_slots * (rows_cap // page_size))      # a ring never grows beyond its rows
         if spec.every > 1:                                                   # whole pages of rows, and a last page per sequence
             n_pages = min(n_pages, -(-n_pages // spec.every) + max_slots)
-        self.pages = GroupPages(n_pages, page_size, rows_cap, name, every=spec.every)
+        self.pages = GroupPages(n_pages, page_size, rows_cap, name, every=spec.every, pinned=pinned)
         self.spare_page = n_pages                                          # the pool's last page, never handed out
         self.pools = {}
         for tname, shape in spec.tensors:
@@ -144,6 +156,7 @@ class ModelCache:
                 keyed.setdefault(spec, []).append(entry)
         def token_group(spec, entries):
             name = f"tokens{len(self.token_groups)}:" + ("all" if spec.window is None else f"window{spec.window}") + \
+                (f"+{spec.keep_first}" if spec.keep_first else "") + \
                 (f"/{spec.every}" if spec.every > 1 else "")
             g = _TokenGroup(spec, entries, n_pages, max_slots, page_size, max_context, dtype, device, name)
             self.token_groups.append(g)

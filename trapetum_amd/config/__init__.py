@@ -4,3 +4,4 @@ from .golepel import GolepelConfig   # noqa: F401
 from .lutovik import LutovikConfig   # noqa: F401
 from .besulix import BesulixConfig   # noqa: F401
 from .vogunex import VogunexConfig   # noqa: F401
+from .solulix import SolulixConfig   # noqa: F401

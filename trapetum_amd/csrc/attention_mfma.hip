@@ -76,6 +76,8 @@ struct DecodeArgs {
     // chunk C > 0: the query sees keys from floor(p / C) C on only.  head_scale, sink ([H] or null): a factor on every
     // head's scores; a score without key or value that joins every head's softmax sum once
     int chunk; const float* head_scale; const float* sink;
+    // the first `keep` positions stay visible behind the window; in a ring they live in the `pin` rows in front of it
+    int keep, pin;
 };
 
 namespace {
@@ -104,11 +106,17 @@ attn_decode_k(DecodeArgs a) {
     int lo = a.window > 0 ? max(0, p - a.window + 1) : 0;
     if (a.chunk > 0) lo = max(lo, p / a.chunk * a.chunk);
     const int lo_al = lo & ~15;
-    int chunk = (p + 1 - lo_al + a.nsplit - 1) / a.nsplit;
+    // The positions a block walks are counted without the gap between the kept ones (rounded up to a tile) and the
+    // window: place u stands for position u below kept_al and for u + gap from there on.  Without kept positions (or where
+    // the window reaches them) there is no gap.
+    const int kept_al = (a.keep + 15) & ~15;
+    const int first = a.keep > 0 ? 0 : lo_al, gap = a.keep > 0 && lo_al > kept_al ? lo_al - kept_al : 0;
+    const int places = p + 1 - gap;
+    int chunk = (places - first + a.nsplit - 1) / a.nsplit;
     chunk = (chunk + ROUND - 1) / ROUND * ROUND;
-    const int t_begin = lo_al + split * chunk;
-    const int t_end = min(p + 1, t_begin + chunk);
-    if (t_begin > p) {                               // this slice has no keys (only when there are several)
+    const int t_begin = first + split * chunk;           // in places
+    const int t_end = min(places, t_begin + chunk);
+    if (t_begin >= places) {                               // this slice has no keys (only when there are several)
         if (tid < G) {
             float* ml = a.ws_ml + (((size_t)seq * a.H + kvh * G + tid) * a.nsplit + split) * 2;
             ml[0] = -INFINITY;
@@ -121,12 +129,13 @@ attn_decode_k(DecodeArgs a) {
     // t % rows_cap of a ring (rows_cap a multiple of the page size, the page size a power of two >= 16), so a tile
     // lies in one page, in 16 consecutive rows: one page-table entry per tile, looked up once for the wave.
     const int page_shift = __ffs(a.page) - 1, page_mask = a.page - 1;
-    const int ring_lo = a.rows_cap > 0 ? lo_al % a.rows_cap : 0;
+    // (pin rows, whole pages, stand before the ring and keep the first positions)
+    const int ring = a.rows_cap - a.pin, ring_from = max(lo_al, a.pin), ring_lo = a.rows_cap > 0 ? (ring_from - a.pin) % ring : 0;
     auto tile_offset = [&](int tb) -> size_t {                     // element offset of the tile's first row in a pool
         int row = tb;
-        if (a.rows_cap > 0) {
-            row = ring_lo + (tb - lo_al);
-            row = row >= a.rows_cap ? row - a.rows_cap : row;
+        if (a.rows_cap > 0 && tb >= a.pin) {
+            row = ring_lo + (tb - ring_from);
+            row = a.pin + (row >= ring ? row - ring : row);
         }
         const int pg = table[row >> page_shift];
         return (((size_t)pg * a.pool_kv + (a.pool_kv == a.KV ? kvh : kvh % a.pool_kv)) * a.page + (row & page_mask)) * HD;
@@ -137,10 +146,13 @@ attn_decode_k(DecodeArgs a) {
     const bool pv_lane = kgw < KGW;
     // ---- loads of a round: the key row of lane c for the scores, value chunks for the sum.  Unconditional loads of
     // rows that exist: a hidden or surplus key gets probability 0 (or is skipped) in the sum ---------------------
-    auto load_round = [&](int tb, bf16x8 (&kf)[DSTEPS], Frag (&vf)[VPT]) {
+    auto row_in_tile = [&](int tb, int t) {                        // a row of the tile that exists, for position t of it
+        return t > p ? p : (t < lo && t >= a.keep ? (lo < tb + 15 ? lo : tb + 15) : t);
+    };
+    auto load_round = [&](int ub, bf16x8 (&kf)[DSTEPS], Frag (&vf)[VPT]) {
+        const int tb = ub < kept_al ? ub : ub + gap;
         const size_t tile = tile_offset(__builtin_amdgcn_readfirstlane(tb));
-        int tk = tb + c;
-        tk = tk < lo ? lo : (tk > p ? p : tk);
+        const int tk = row_in_tile(tb, tb + c);
         const bf16_t* kp = a.k_pool + tile + (size_t)(tk - tb) * HD;
 #pragma unroll
         for (int ks = 0; ks < DSTEPS; ks++) {
@@ -151,8 +163,7 @@ attn_decode_k(DecodeArgs a) {
         for (int j = 0; j < VPT; j++) {
             int kk = kgw + j * KGW;
             kk = kk > 15 ? 15 : kk;
-            int tv = tb + kk;
-            tv = tv < lo ? lo : (tv > p ? p : tv);
+            const int tv = row_in_tile(tb, tb + kk);
             vf[j].u = *reinterpret_cast<const uint4*>(a.v_pool + tile + (size_t)(tv - tb) * HD + ch * 8);
         }
     };
@@ -161,7 +172,7 @@ attn_decode_k(DecodeArgs a) {
     bf16x8 kf[DSTEPS];
     Frag vf[VPT];
     const int tb0 = t_begin + wave * 16;
-    const bool late = a.qkv && a.write_kv && tb0 <= p && p < tb0 + 16;
+    const bool late = a.qkv && a.write_kv && tb0 < places && places - 1 < tb0 + 16;
     if (tb0 < t_end && !late) load_round(tb0, kf, vf);
 
     // ---- the group's queries into LDS; in the fused form from the step's projections: K slices added, queries and
@@ -195,13 +206,13 @@ attn_decode_k(DecodeArgs a) {
                 for (int c = 0; c < NC; c++) out[c] = bf16_to_f32(src[cols[c]]);
             }
         };
-        // the slice that holds position p (t_begin <= p holds here) also rotates the new key and writes it and the value
+        // the slice that holds position p (t_begin < places holds here) also rotates the new key and writes it and the value
         // into the cache: thread f < rot/2 does that beside its pair of the first query head, whose angle is the same
-        const bool writer = a.write_kv && p < t_begin + chunk;
+        const bool writer = a.write_kv && places - 1 < t_begin + chunk;
         bf16_t* kdst = nullptr;
         bf16_t* vdst = nullptr;
         if (writer) {
-            int row = a.rows_cap > 0 ? p % a.rows_cap : p;
+            const int row = a.rows_cap > 0 && p >= a.pin ? a.pin + (p - a.pin) % ring : p;
             const int pg = table[row >> page_shift];
             const size_t at = (((size_t)pg * a.KV + kvh) * a.page + (row & page_mask)) * HD;
             kdst = a.k_pool + at;
@@ -276,8 +287,8 @@ attn_decode_k(DecodeArgs a) {
         float mx = -INFINITY;
 #pragma unroll
         for (int i = 0; i < 4; i++) {
-            const int t = tb + g * 4 + i;
-            const bool ok = t >= lo && t < t_end;
+            const int u = tb + g * 4 + i, t = u < kept_al ? u : u + gap;
+            const bool ok = (t >= lo || t < a.keep) && u < t_end;
             s[i] = ok ? score_of(s[i], scale_c, a.cap, soc) : -INFINITY;
             mx = fmaxf(mx, s[i]);
         }
@@ -437,8 +448,10 @@ static int decode_launch(DecodeArgs a, int n_seq, void* workspace, hipStream_t s
                "attention decode: %d groups of heads cannot share %d kv heads of the cache", a.KV, a.pool_kv);
     TP_REQUIRE(a.page >= 16 && (a.page & (a.page - 1)) == 0 && a.table_w > 0, "attention decode (matrix-core kernel): page size %d must be a power of two, at least 16", a.page);
     TP_REQUIRE(a.chunk >= 0, "attention decode: chunks of %d positions", a.chunk);
+    TP_REQUIRE(a.keep >= 0 && a.pin >= 0 && a.pin % a.page == 0 && (a.keep == 0 || (a.window > 0 && a.chunk == 0)), "attention decode: %d kept positions (%d rows before the ring) stand beside a window, without chunks", a.keep, a.pin);
+    TP_REQUIRE(a.rows_cap == 0 || (a.pin < a.rows_cap && a.keep <= a.pin), "attention decode: %d kept positions and %d rows before a ring do not fit a cache of %d rows", a.keep, a.pin, a.rows_cap);
     const int reach = a.window > 0 && a.chunk > 0 ? (a.window < a.chunk ? a.window : a.chunk) : (a.window > 0 ? a.window : a.chunk);
-    TP_REQUIRE(a.rows_cap == 0 || (reach > 0 && reach <= a.rows_cap), "attention decode: a reach of %d keys (window %d, chunk %d) does not fit a ring of %d rows", reach, a.window, a.chunk, a.rows_cap);
+    TP_REQUIRE(a.rows_cap == 0 || (reach > 0 && reach <= a.rows_cap - a.pin), "attention decode: a reach of %d keys (window %d, chunk %d) does not fit a ring of %d rows", reach, a.window, a.chunk, a.rows_cap - a.pin);
     TP_REQUIRE(a.rows_cap >= 0 && a.rows_cap % a.page == 0, "attention decode: ring of %d rows is no multiple of the page size %d", a.rows_cap, a.page);
     TP_REQUIRE(a.nsplit >= 1 && a.nsplit <= 128 && (a.nsplit == 1 || workspace), "attention decode: %d slices (at most 128) need a workspace", a.nsplit);
     TP_REQUIRE(a.KV <= 65535 && n_seq <= 65535, "attention decode: grid too large");
@@ -463,11 +476,11 @@ static int decode_launch(DecodeArgs a, int n_seq, void* workspace, hipStream_t s
 extern "C" int tp_attn_decode(const void* q, long q_stride, int n_seq, int H, int KV, const int* new_len,
                               const int* table, int table_w, const void* k_pool, const void* v_pool, int page,
                               int rows_cap, float scale, float cap, int window, int chunk, const float* head_scale,
-                              const float* sink, void* out, void* workspace, int nsplit, void* stream) {
+                              const float* sink, int keep, int pin, void* out, void* workspace, int nsplit, void* stream) {
     TP_REQUIRE(q_stride % 8 == 0 && (uintptr_t)q % 16 == 0, "attention decode: query rows must be 16-byte aligned");
     DecodeArgs a{(const bf16_t*)q, q_stride, H, KV, new_len, table, table_w, (bf16_t*)k_pool, (bf16_t*)v_pool,
                  page, rows_cap, scale, cap, window, (bf16_t*)out, nullptr, nullptr, nsplit,
-                 nullptr, 0, 1, 0, 0, nullptr, 0, 0, 0, chunk, head_scale, sink};
+                 nullptr, 0, 1, 0, 0, nullptr, 0, 0, 0, chunk, head_scale, sink, keep, pin};
     return decode_launch(a, n_seq, workspace, (hipStream_t)stream);
 }
 
@@ -492,7 +505,7 @@ extern "C" int tp_attn_decode_fused(const void* qkv, int qkv_dtype, int n_slices
                                     const float* inv_freq, int rot, int write_kv,
                                     int n_seq, int H, int KV, const int* new_len, const int* table, int table_w,
                                     void* k_pool, void* v_pool, int page, int rows_cap, float scale, float cap,
-                                    int window, void* out, void* workspace, int nsplit, void* stream) {
+                                    int window, const float* sink, int keep, int pin, void* out, void* workspace, int nsplit, void* stream) {
     TP_REQUIRE(qkv, "attention decode (fused): no projections");
     TP_REQUIRE(qkv_dtype == TP_BF16 || qkv_dtype == TP_F32, "attention decode (fused): projections of dtype %d", qkv_dtype);
     TP_REQUIRE(n_slices >= 1 && (n_slices == 1 || qkv_dtype == TP_F32), "attention decode (fused): %d slices must be float32", n_slices);
@@ -501,6 +514,6 @@ extern "C" int tp_attn_decode_fused(const void* qkv, int qkv_dtype, int n_slices
     TP_REQUIRE(row_stride >= (long)(H + (write_kv ? 2 * KV : 0)) * HD, "attention decode (fused): rows of %ld elements are too short", row_stride);
     DecodeArgs a{nullptr, 0, H, KV, new_len, table, table_w, (bf16_t*)k_pool, (bf16_t*)v_pool,
                  page, rows_cap, scale, cap, window, (bf16_t*)out, nullptr, nullptr, nsplit,
-                 qkv, qkv_dtype == TP_F32 ? 1 : 0, n_slices, slice_stride, row_stride, inv_freq, rot, write_kv};
+                 qkv, qkv_dtype == TP_F32 ? 1 : 0, n_slices, slice_stride, row_stride, inv_freq, rot, write_kv, 0, 0, nullptr, sink, keep, pin};
     return decode_launch(a, n_seq, workspace, (hipStream_t)stream);
 }

@@ -55,6 +55,7 @@ struct PrefillArgs {
     int chunk;                                // C > 0: the query at p sees keys from floor(p / C) C on only
     const float* head_scale;                  // [H] or null: a factor on every head's scores
     const float* sink;                        // [H] or null: a score without key or value that joins every softmax's sum once
+    int keep, pin;                            // the first `keep` positions stay visible behind the window; rows of the cache in front of its ring
     bf16_t* out;
 };
 
@@ -144,26 +145,33 @@ attn_prefill_k(PrefillArgs a) {
     if (a.chunk > 0) k_lo = max(k_lo, (start + q0) / a.chunk * a.chunk);     // the block's first query has the earliest chunk
     k_lo &= ~31;
     const int k_hi = min(L, start + q0 + PB);
-    const int n_rounds = (k_hi - k_lo + 32 * KG - 1) / (32 * KG);
+    // Kept positions are walked first, in whole tiles; the gap between them and the window's first tile is left out: tile
+    // place u stands for the keys from u below kept_al and from u + gap there and above.
+    const int kept_al = (a.keep + 31) & ~31;
+    const int u_lo = a.keep > 0 ? 0 : k_lo, gap = a.keep > 0 && k_lo > kept_al ? k_lo - kept_al : 0;
+    const int n_rounds = (k_hi - gap - u_lo + 32 * KG - 1) / (32 * KG);
+    auto tile_of = [&](int r) { const int u = u_lo + 32 * (r * KG + kg); return u < kept_al ? u : u + gap; };
 
     // ---- loads of a tile: wave cg of the key group fetches the tile's key octets cg, cg + CG, ..; lane l the
     // 16-byte chunk that belongs at place (key l / 8 of the octet, place l % 8 of its 128-byte row) -----------------
     constexpr int NOCT = 4 / CG;
-    const int ring_lo = PAGED && a.rows_cap > 0 ? k_lo % a.rows_cap : 0;
+    const int ring = a.rows_cap - a.pin, ring_from = max(k_lo, a.pin), ring_lo = PAGED && a.rows_cap > 0 ? (ring_from - a.pin) % ring : 0;
     const bf16_t* const k_rows = a.k + (size_t)kvh * HD;
     const bf16_t* const v_rows = a.v + (size_t)kvh * HD;
     auto row_of = [&](int key, const bf16_t*& kp, const bf16_t*& vp) {
         key = min(key, L - 1);                                    // past the end: a row that exists, hidden from every query
+        if (key >= a.keep && key < k_lo) key = 0;                 // in a tile of kept keys, none of them and before the window: likewise
         if (PAGED && key < start) {
             int row = key;
-            if (a.rows_cap > 0) {
-                // key % rows_cap without a division: a cached key lies less than window + 30 positions behind k_lo (the
+            if (a.rows_cap > 0 && key >= a.pin) {
+                // key % ring without a division: a cached key of the window lies less than window + 30 positions behind k_lo (the
                 // window's start rounded down to a tile), the window fits the ring and the ring has at least 16 rows,
-                // so the sum below is less than four rings: three conditional subtractions
-                row = ring_lo + (key - k_lo);
-                row = row >= a.rows_cap ? row - a.rows_cap : row;
-                row = row >= a.rows_cap ? row - a.rows_cap : row;
-                row = row >= a.rows_cap ? row - a.rows_cap : row;
+                // so the sum below is less than four rings: three conditional subtractions (a kept key is below pin)
+                row = ring_lo + (key - ring_from);
+                row = row >= ring ? row - ring : row;
+                row = row >= ring ? row - ring : row;
+                row = row >= ring ? row - ring : row;
+                row += a.pin;
             }
             const int pg = a.table[(size_t)seq * a.table_w + (row >> a.page_shift)];
             const size_t at = ((((size_t)pg * a.KV + kvh) << a.page_shift) + (row & a.page_mask)) * HD;
@@ -185,7 +193,7 @@ attn_prefill_k(PrefillArgs a) {
     const bf16_t* kp[NOCT];
     const bf16_t* vp[NOCT];
     auto rows_of_round = [&](int r) {
-        const int kt = k_lo + 32 * (r * KG + kg);
+        const int kt = tile_of(r);
 #pragma unroll
         for (int o = 0; o < NOCT; o++) row_of(kt + (cg + o * CG) * 8 + (lane >> 3), kp[o], vp[o]);
     };
@@ -264,9 +272,9 @@ attn_prefill_k(PrefillArgs a) {
     __syncthreads();
     float sc[16];                                    // lane: query `col`, keys kt + 8 (j / 4) + 4 hi + j % 4; in units of log 2
     for (int r = 0; r < n_rounds; r++) {
-        const int kt = k_lo + 32 * (r * KG + kg);
+        const int kt = tile_of(r);
         // wave-uniform: some key of the tile is visible to some query of the wave
-        const bool visible = kt < k_hi && kt <= qw0 + 31 && qw0 < L && (a.window <= 0 || kt + 31 > qw0 - a.window) && kt + 31 >= chunk_first;
+        const bool visible = kt < k_hi && kt <= qw0 + 31 && qw0 < L && (a.window <= 0 || kt + 31 > qw0 - a.window || kt < a.keep) && kt + 31 >= chunk_first;
         if (visible) {
             // two chains of accumulation where the registers allow it (at head size 256 they do not, and a second
             // chain measured no faster there: the SIMD's other wave fills in)
@@ -307,12 +315,21 @@ attn_prefill_k(PrefillArgs a) {
             issue_k();
         }
         if (visible) {
-            const bool whole = kt + 31 <= qw0 && (a.window <= 0 || qw0 + 31 - kt < a.window) && kt >= chunk_last;
+            const bool whole = kt + 31 <= qw0 && (a.window <= 0 || qw0 + 31 - kt < a.window || kt + 31 < a.keep) && kt >= chunk_last;
             if (!whole) {
                 const int d0 = qpos - kt - 4 * hi;   // distance to key j: d0 - 8 (j / 4) - j % 4; visible: 0 <= distance < window
+                if (kt < a.keep) {                   // (wave-uniform) ... or 0 <= distance and the key is a kept one
+                    const int k0 = kt + 4 * hi;
 #pragma unroll
-                for (int j = 0; j < 16; j++)
-                    sc[j] = (unsigned)(d0 - 8 * (j >> 2) - (j & 3)) < win ? sc[j] : -INFINITY;
+                    for (int j = 0; j < 16; j++) {
+                        const int e = 8 * (j >> 2) + (j & 3);
+                        sc[j] = d0 >= e && ((unsigned)(d0 - e) < win || k0 + e < a.keep) ? sc[j] : -INFINITY;
+                    }
+                } else {
+#pragma unroll
+                    for (int j = 0; j < 16; j++)
+                        sc[j] = (unsigned)(d0 - 8 * (j >> 2) - (j & 3)) < win ? sc[j] : -INFINITY;
+                }
             }
             float mx = sc[0];
 #pragma unroll
@@ -456,20 +473,22 @@ extern "C" int tp_attn_prefill(const void* q, long q_stride, const void* k, long
                                int M, int H, int KV, const int* cu_rows, int n_seq, int max_count,
                                const int* new_len, const int* table, int table_w, const void* k_pool, const void* v_pool,
                                int page, int rows_cap, float scale, float cap, int window, int chunk, const float* head_scale,
-                               const float* sink, void* out, int shape, void* stream) {
+                               const float* sink, int keep, int pin, void* out, int shape, void* stream) {
     TP_REQUIRE(M > 0 && H > 0 && KV > 0 && n_seq > 0 && max_count > 0, "attention prefill: empty shape");
     TP_REQUIRE(H % KV == 0, "attention: %d query heads are no multiple of %d kv heads", H, KV);
     TP_REQUIRE(q_stride % 8 == 0 && k_stride % 8 == 0 && v_stride % 8 == 0 && (uintptr_t)q % 16 == 0 &&
                (uintptr_t)k % 16 == 0 && (uintptr_t)v % 16 == 0, "attention prefill: rows must be 16-byte aligned");
     TP_REQUIRE(scale > 0.f, "attention prefill: the scale %g must be positive", scale);
     TP_REQUIRE(chunk >= 0, "attention prefill: chunks of %d positions", chunk);
+    TP_REQUIRE(keep >= 0 && (keep == 0 || (window > 0 && chunk == 0)), "attention prefill: %d kept positions stand beside a window, without chunks", keep);
     const bool paged = new_len != nullptr;
     if (paged) {
         TP_REQUIRE(table && k_pool && v_pool && table_w > 0, "attention prefill: cached positions need the page table and the pools");
         TP_REQUIRE(page >= 16 && (page & (page - 1)) == 0, "attention prefill (matrix-core kernel): page size %d must be a power of two, at least 16", page);
         TP_REQUIRE(rows_cap >= 0 && rows_cap % page == 0, "attention prefill: ring of %d rows is no multiple of the page size %d", rows_cap, page);
         const int reach = window > 0 && chunk > 0 ? (window < chunk ? window : chunk) : (window > 0 ? window : chunk);
-        TP_REQUIRE(rows_cap == 0 || (reach > 0 && reach <= rows_cap), "attention prefill: a reach of %d keys (window %d, chunk %d) does not fit a ring of %d rows", reach, window, chunk, rows_cap);
+        TP_REQUIRE(pin >= 0 && pin % page == 0 && (rows_cap == 0 || (pin < rows_cap && keep <= pin)), "attention prefill: %d kept positions and %d rows before a ring do not fit a cache of %d rows", keep, pin, rows_cap);
+        TP_REQUIRE(rows_cap == 0 || (reach > 0 && reach <= rows_cap - pin), "attention prefill: a reach of %d keys (window %d, chunk %d) does not fit a ring of %d rows", reach, window, chunk, rows_cap - pin);
         TP_REQUIRE((uintptr_t)k_pool % 16 == 0 && (uintptr_t)v_pool % 16 == 0, "attention prefill: the pools must be 16-byte aligned");
     }
     const int G = H / KV;
@@ -482,6 +501,7 @@ extern "C" int tp_attn_prefill(const void* q, long q_stride, const void* k, long
     a.page_shift = ps; a.page_mask = page - 1; a.rows_cap = paged ? rows_cap : 0;
     a.H = H; a.KV = KV; a.scale = scale; a.cap = cap; a.window = window; a.out = (bf16_t*)out;
     a.chunk = chunk; a.head_scale = head_scale; a.sink = sink;
+    a.keep = keep; a.pin = paged && rows_cap > 0 ? pin : 0;
     static int cus = 0;
     if (!cus) {
         int dev = 0;

@@ -8,7 +8,8 @@
 // sum of v, kv head = head / (heads / kv_heads); the scale is an argument (rsqrt(head_dim) there), and a
 // window W hides keys with p - t >= W (none there).  Beyond the reference: with chunks of C positions the query at p
 // sees only keys from floor(p / C) C on; a head may have a temperature that multiplies its scores and a sink, a score
-// without key or value whose exponential joins the denominator once, after the keys.
+// without key or value whose exponential joins the denominator once, after the keys.  With `keep` the first keep positions
+// of a sequence stay visible behind the window; in a ring they live in the `pin` rows in front of it.
 #include "common.h"
 
 struct AttnSimpleArgs {
@@ -23,6 +24,7 @@ struct AttnSimpleArgs {
     void* out;
     int H, KV, hd; float scale, cap; int window; int paged;
     int chunk; const float* head_scale; const float* sink;        // 0 and null: none
+    int keep, pin;                                       // positions seen beside the window; rows of the cache in front of its ring
 };
 
 // NJ: elements of a head a lane holds (head sizes up to 64 NJ)
@@ -50,13 +52,16 @@ attn_simple_k(AttnSimpleArgs a) {
         o[j] = 0.f;
     }
     float m = -INFINITY, l = 0.f;
+    // the keys in order: the kept ones before the window, then the window's; key i stands at position at(i)
+    const int kept = min(a.keep, lo), n_keys = kept + p - lo + 1;
+    auto at = [&](int i) { return i < kept ? i : lo + i - kept; };
     // a key's row and value row are fetched while the two keys before it are worked on (the arithmetic per key, and
     // its order, stay as they are: the loop would otherwise pay a trip to memory, or two through the page table, per key)
-    auto fetch = [&](int t, float (&kk)[NJ], float (&vv)[NJ]) {
-        t = t < p ? t : p;                               // past the last key: a row that exists, never used
+    auto fetch = [&](int i, float (&kk)[NJ], float (&vv)[NJ]) {
+        const int t = min(at(i), p);                     // past the last key: a row that exists, never used
         const T *kp, *vp;
         if (t < start) {
-            const int row = a.rows_cap > 0 ? t % a.rows_cap : t;
+            const int row = a.rows_cap > 0 && t >= a.pin ? a.pin + (t - a.pin) % (a.rows_cap - a.pin) : t;
             const int pg = a.table[(size_t)seq * a.table_w + row / a.page];
             const size_t off = (((size_t)pg * a.KV + g) * a.page + row % a.page) * a.hd;
             kp = (const T*)a.k_pool + off;
@@ -89,16 +94,16 @@ attn_simple_k(AttnSimpleArgs a) {
         m = m_new;
     };
     float k0[NJ], v0[NJ], k1[NJ], v1[NJ], k2[NJ], v2[NJ];
-    fetch(lo, k0, v0);
-    fetch(lo + 1, k1, v1);
-    for (int t = lo; t <= p; t += 3) {
-        fetch(t + 2, k2, v2);
+    fetch(0, k0, v0);
+    fetch(1, k1, v1);
+    for (int i = 0; i < n_keys; i += 3) {
+        fetch(i + 2, k2, v2);
         use(k0, v0);
-        if (t + 1 > p) break;
-        fetch(t + 3, k0, v0);
+        if (i + 1 >= n_keys) break;
+        fetch(i + 3, k0, v0);
         use(k1, v1);
-        if (t + 2 > p) break;
-        fetch(t + 4, k1, v1);
+        if (i + 2 >= n_keys) break;
+        fetch(i + 4, k1, v1);
         use(k2, v2);
     }
     if (a.sink) {
@@ -118,6 +123,8 @@ attn_simple_k(AttnSimpleArgs a) {
 }
 
 static int launch(const AttnSimpleArgs& a, int dtype, int M, hipStream_t s) {
+    TP_REQUIRE(a.keep >= 0 && a.pin >= 0 && (a.keep == 0 || (a.window > 0 && a.chunk == 0)), "attention: %d kept positions stand beside a window, without chunks", a.keep);
+    TP_REQUIRE(a.rows_cap == 0 || (a.pin < a.rows_cap && a.keep <= a.pin), "attention: %d kept positions and %d rows before a ring do not fit a cache of %d rows", a.keep, a.pin, a.rows_cap);
     TP_REQUIRE(M > 0 && a.H > 0 && a.KV > 0 && a.hd > 0, "attention: empty shape rows=%d heads=%d kv=%d head_dim=%d", M, a.H, a.KV, a.hd);
     TP_REQUIRE(a.H % a.KV == 0, "attention: %d query heads are no multiple of %d kv heads", a.H, a.KV);
     TP_REQUIRE(a.hd <= 1024, "attention (plain kernel): head_dim %d exceeds 1024", a.hd);
@@ -139,7 +146,7 @@ extern "C" int tp_attn_simple_prefill(const void* q, long q_stride, const void* 
                                       const int* row_pos, const int* new_len, const int* table, int table_w,
                                       const void* k_pool, const void* v_pool, int page, int rows_cap,
                                       float scale, float cap, int window, int chunk, const float* head_scale, const float* sink,
-                                      void* out, void* stream) {
+                                      int keep, int pin, void* out, void* stream) {
     TP_REQUIRE(chunk >= 0, "attention: chunks of %d positions", chunk);
     TP_REQUIRE(!new_len || (table && k_pool && v_pool && page > 0 && table_w > 0), "attention: cached positions need the page table and the pools");
     AttnSimpleArgs a{};
@@ -149,13 +156,14 @@ extern "C" int tp_attn_simple_prefill(const void* q, long q_stride, const void* 
     a.page = new_len ? page : 1; a.rows_cap = new_len ? rows_cap : 0;
     a.out = out; a.H = H; a.KV = KV; a.hd = hd; a.scale = scale; a.cap = cap; a.window = window; a.paged = 0;
     a.chunk = chunk; a.head_scale = head_scale; a.sink = sink;
+    a.keep = keep; a.pin = pin;
     return launch(a, dtype, M, (hipStream_t)stream);
 }
 
 extern "C" int tp_attn_simple_decode(const void* q, long q_stride, int dtype, int n_seq, int H, int KV, int hd,
                                      const int* new_len, const int* table, int table_w, const void* k_pool,
                                      const void* v_pool, int page, int rows_cap, float scale, float cap, int window,
-                                     int chunk, const float* head_scale, const float* sink, void* out, void* stream) {
+                                     int chunk, const float* head_scale, const float* sink, int keep, int pin, void* out, void* stream) {
     TP_REQUIRE(chunk >= 0, "attention: chunks of %d positions", chunk);
     TP_REQUIRE(page > 0 && table_w > 0, "attention: page size %d, table width %d", page, table_w);
     AttnSimpleArgs a{};
@@ -163,5 +171,6 @@ extern "C" int tp_attn_simple_decode(const void* q, long q_stride, int dtype, in
     a.k_pool = k_pool; a.v_pool = v_pool; a.page = page; a.rows_cap = rows_cap;
     a.out = out; a.H = H; a.KV = KV; a.hd = hd; a.scale = scale; a.cap = cap; a.window = window; a.paged = 1;
     a.chunk = chunk; a.head_scale = head_scale; a.sink = sink;
+    a.keep = keep; a.pin = pin;
     return launch(a, dtype, n_seq, (hipStream_t)stream);
 }

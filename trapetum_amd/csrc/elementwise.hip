@@ -356,6 +356,135 @@ extern "C" int tp_add_rms_norm(float* stream, const void* rows, int rows_dtype, 
     return tp_check_launch("add_rms_norm");
 }
 
+// ---- stream += a + b + vec + origin; out = norm(stream) --------------------------------------------------------------
+// For a block whose two sub-layers read one norm: their rows are added to the stream together.  a and b: rows of either
+// dtype, or float32 K slices of a product (added in slice order); b may be null, and a too (then only what follows is
+// added).  vec [D] and origin [M, D] (float32, or null) are what stands between two layers of a model: a vector that
+// every row gets, and earlier rows of the stream.  The sums are float32.  One block a row; PC: elements a lane takes at a
+// time (4 where every operand allows it).
+struct JoinArgs {
+    float* stream; const void* a; int a_f32, a_slices; long a_stride; const void* b; int b_f32, b_slices; long b_stride;
+    const float* vec; const float* origin; const float* gain; float eps; void* out; int D;
+};
+
+template <int PC>
+__device__ __forceinline__ void ld_piece(const float* p, float (&o)[PC]) {
+    if constexpr (PC == 4) ld4(p, o); else o[0] = *p;
+}
+template <int PC>
+__device__ __forceinline__ void add_rows_piece(const void* rows, int f32, int slices, long stride, size_t at, float (&v)[PC]) {
+    if (!f32) {
+        float t[PC];
+        if constexpr (PC == 4) ld4((const bf16_t*)rows + at, t); else t[0] = ld_f32((const bf16_t*)rows + at);
+#pragma unroll
+        for (int e = 0; e < PC; e++) v[e] += t[e];
+        return;
+    }
+    for (int s0 = 0; s0 < slices; s0 += 4) {              // four slices' loads in flight; past the last one it is repeated and not added
+        float t[4][PC];
+#pragma unroll
+        for (int u = 0; u < 4; u++) ld_piece<PC>((const float*)rows + (size_t)(s0 + u < slices ? s0 + u : slices - 1) * stride + at, t[u]);
+#pragma unroll
+        for (int u = 0; u < 4; u++)
+#pragma unroll
+            for (int e = 0; e < PC; e++) v[e] += s0 + u < slices ? t[u][e] : 0.f;
+    }
+}
+
+template <typename T, int PC, int CPT, int NTH>
+__global__ void __launch_bounds__(NTH)
+join_rms_norm_k(JoinArgs x) {
+    __shared__ float red[16];
+    const int D = x.D;
+    const size_t row = (size_t)blockIdx.x * D;
+    float v[CPT][PC], gn[CPT][PC];
+    float ss = 0.f;
+#pragma unroll
+    for (int j = 0; j < CPT; j++) {
+        const int i = (threadIdx.x + j * NTH) * PC;
+        const bool ok = i < D;
+        const int ic = ok ? i : 0;
+        ld_piece<PC>(x.stream + row + ic, v[j]);
+        if (x.gain) ld_piece<PC>(x.gain + ic, gn[j]);
+        float more[PC];
+#pragma unroll
+        for (int e = 0; e < PC; e++) more[e] = 0.f;
+        if (x.a) add_rows_piece<PC>(x.a, x.a_f32, x.a_slices, x.a_stride, row + ic, more);
+        if (x.b) add_rows_piece<PC>(x.b, x.b_f32, x.b_slices, x.b_stride, row + ic, more);
+#pragma unroll
+        for (int e = 0; e < PC; e++) v[j][e] += more[e];
+        if (x.origin) {
+            float t[PC];
+            ld_piece<PC>(x.origin + row + ic, t);
+#pragma unroll
+            for (int e = 0; e < PC; e++) v[j][e] += t[e];
+        }
+        if (x.vec) {
+            float t[PC];
+            ld_piece<PC>(x.vec + ic, t);
+#pragma unroll
+            for (int e = 0; e < PC; e++) v[j][e] += t[e];
+        }
+        if (ok) {
+            if constexpr (PC == 4) st4(x.stream + row + i, v[j]); else x.stream[row + i] = v[j][0];
+#pragma unroll
+            for (int e = 0; e < PC; e++) ss = __builtin_fmaf(v[j][e], v[j][e], ss);
+        }
+    }
+    if (!x.gain) return;
+    ss = block_sum_once(ss, red);
+    const float scale = rsqrtf(ss / (float)D + x.eps);
+    T* orow = (T*)x.out + row;
+#pragma unroll
+    for (int j = 0; j < CPT; j++) {
+        const int i = (threadIdx.x + j * NTH) * PC;
+        float o[PC];
+#pragma unroll
+        for (int e = 0; e < PC; e++) o[e] = (v[j][e] * scale) * gn[j][e];
+        if (i < D) { if constexpr (PC == 4) st4(orow + i, o); else st_f32(orow + i, o[0]); }
+    }
+}
+
+template <typename T>
+static int join_launch(const JoinArgs& x, int M, hipStream_t s) {
+    const auto al = [](const void* p) { return (uintptr_t)p % 16 == 0; };
+    const bool wide = x.D % 4 == 0 && x.a_stride % 4 == 0 && x.b_stride % 4 == 0 && al(x.stream) && al(x.a) && al(x.b) && al(x.vec) && al(x.origin) && al(x.gain) && al(x.out);
+    const int D = x.D;
+#define TP_JOIN(PC, CPT, NTH) join_rms_norm_k<T, PC, CPT, NTH><<<M, NTH, 0, s>>>(x)
+    if (wide) {
+        if (D <= 256 * 4) TP_JOIN(4, 1, 256);
+        else if (M <= 128 && D <= 640 * 4) TP_JOIN(4, 1, 640);
+        else if (M <= 128 && D <= 1024 * 4) TP_JOIN(4, 1, 1024);
+        else if (D <= 192 * 12) TP_JOIN(4, 3, 192);
+        else if (D <= 256 * 12) TP_JOIN(4, 3, 256);
+        else if (D <= 320 * 12) TP_JOIN(4, 3, 320);
+        else if (D <= 512 * 16) TP_JOIN(4, 4, 512);
+        else if (D <= 1024 * 32) TP_JOIN(4, 8, 1024);
+        else return tp_fail("join_rms_norm: rows of %d elements exceed %d", D, 1024 * 32);
+    } else {
+        if (D <= 256 * 4) TP_JOIN(1, 4, 256);
+        else if (D <= 1024 * 8) TP_JOIN(1, 8, 1024);
+        else return tp_fail("join_rms_norm: unaligned rows of %d elements exceed %d", D, 1024 * 8);
+    }
+#undef TP_JOIN
+    return tp_check_launch("join_rms_norm");
+}
+
+// gain null: no norm, no output.  a, b: [M, D] of a_dtype, b_dtype, float32 ones in a_slices, b_slices slices a stride apart
+extern "C" int tp_join_rms_norm(float* stream, const void* a, int a_dtype, int a_slices, long a_stride, const void* b, int b_dtype, int b_slices,
+                                long b_stride, const float* vec, const float* origin, const float* gain, float eps, void* out, int out_dtype,
+                                int M, int D, void* stream_) {
+    TP_REQUIRE(M > 0 && D > 0 && stream, "join_rms_norm: empty shape M=%d D=%d", M, D);
+    TP_REQUIRE(!gain || out, "join_rms_norm: a norm needs an output buffer");
+    TP_REQUIRE(a || !b, "join_rms_norm: a second operand without a first");
+    TP_REQUIRE(!a || ((a_dtype == TP_F32 || a_dtype == TP_BF16) && a_slices >= 1 && (a_slices == 1 || a_dtype == TP_F32)), "join_rms_norm: rows in %d slices of dtype %d", a_slices, a_dtype);
+    TP_REQUIRE(!b || ((b_dtype == TP_F32 || b_dtype == TP_BF16) && b_slices >= 1 && (b_slices == 1 || b_dtype == TP_F32)), "join_rms_norm: rows in %d slices of dtype %d", b_slices, b_dtype);
+    JoinArgs x{stream, a, a_dtype == TP_F32, a_slices, a_stride, b, b_dtype == TP_F32, b_slices, b_stride, vec, origin, gain, eps, out, D};
+    if (out_dtype == TP_BF16) return join_launch<bf16_t>(x, M, (hipStream_t)stream_);
+    if (out_dtype == TP_F32) return join_launch<float>(x, M, (hipStream_t)stream_);
+    return tp_fail("join_rms_norm: unknown output dtype %d", out_dtype);
+}
+
 // ---- the K slices of a product added in slice order (for a consumer that does not add them itself) --------------
 template <typename T>
 __global__ void sum_slices_k(const float* __restrict__ slices, int n_slices, long slice_stride, T* __restrict__ out, long count) {
@@ -393,7 +522,9 @@ extern "C" int tp_gather_rows(const float* x, const int* rows, float* out, int n
 // ---- RoPE on q and k in place, then k and v into the paged cache -----------------------------------------
 // Rotation: pair (d, d + rot/2), angle = pos * inv_freq[d], fp32 cos/sin (runtime/cuda/codebook_gemv.cu:219-230);
 // the cache keeps k after the rotation and v as projected (runtime/src/lib.rs:4487-4490).
-// A sequence's position p lives in row p (or p % rows_cap of a ring), found through its page list.
+// A sequence's position p lives in row p (or p % rows_cap of a ring), found through its page list.  With `pin` rows in
+// front of the ring (a window that keeps a sequence's first tokens) the positions below pin stay in their rows and the
+// others take the rows_cap - pin rows behind them in turn.
 // grid (rows, groups of heads): a block rotates `hpb` of the row's H + KV heads (query heads first); a thread
 // computes the cosine and sine of its pair once and applies them to all of them.  A key head goes into the
 // cache, with its value head, straight from registers; without a page table the keys are rotated and nothing is
@@ -405,7 +536,7 @@ rope_kv_write_k(T* __restrict__ q, long q_stride, T* __restrict__ k, long k_stri
                 const float* __restrict__ inv_freq, int rot,
                 const int* __restrict__ row_seq, const int* __restrict__ row_pos,
                 const int* __restrict__ new_len, const int* __restrict__ table, int table_w,
-                T* __restrict__ k_pool, T* __restrict__ v_pool, int page, int rows_cap, int hpb, int pairing) {
+                T* __restrict__ k_pool, T* __restrict__ v_pool, int page, int rows_cap, int pin, int hpb, int pairing) {
     const int r = blockIdx.x;
     const int j_begin = blockIdx.y * hpb, j_end = min(j_begin + hpb, H + (k ? KV : 0));
     const int pos = row_pos[r];
@@ -417,9 +548,9 @@ rope_kv_write_k(T* __restrict__ q, long q_stride, T* __restrict__ k, long k_stri
         const int seq = row_seq[r];
         int row = pos;
         bool keep = true;
-        if (rows_cap > 0) {
-            keep = pos + rows_cap >= new_len[seq];       // else a later row of this step takes the same ring row
-            row = pos % rows_cap;
+        if (rows_cap > 0 && pos >= pin) {
+            keep = pos + rows_cap - pin >= new_len[seq];       // else a later row of this step takes the same ring row
+            row = pin + (pos - pin) % (rows_cap - pin);
         }
         const int pg = keep ? table[(size_t)seq * table_w + row / page] : -1;
         cached = pg >= 0;
@@ -465,7 +596,7 @@ rope_kv_write_vec_k(bf16_t* __restrict__ q, long q_stride, bf16_t* __restrict__ 
                     const float* __restrict__ inv_freq, int rot,
                     const int* __restrict__ row_seq, const int* __restrict__ row_pos,
                     const int* __restrict__ new_len, const int* __restrict__ table, int table_w,
-                    bf16_t* __restrict__ k_pool, bf16_t* __restrict__ v_pool, int page, int rows_cap) {
+                    bf16_t* __restrict__ k_pool, bf16_t* __restrict__ v_pool, int page, int rows_cap, int pin) {
     // cosine and sine of pair f at [f % 8][f / 8]: the threads of a wave, which turn neighbouring pieces of 8 pairs, then
     // read neighbouring words (pair by pair in the pairs' own order, a wave's reads fell on four banks)
     __shared__ float cs[8 * 16], sn[8 * 16];
@@ -481,9 +612,9 @@ rope_kv_write_vec_k(bf16_t* __restrict__ q, long q_stride, bf16_t* __restrict__ 
         const int seq = row_seq[r];
         int row = pos;
         bool keep = true;
-        if (rows_cap > 0) {
-            keep = pos + rows_cap >= new_len[seq];       // else a later row of this step takes the same ring row
-            row = pos % rows_cap;
+        if (rows_cap > 0 && pos >= pin) {
+            keep = pos + rows_cap - pin >= new_len[seq];       // else a later row of this step takes the same ring row
+            row = pin + (pos - pin) % (rows_cap - pin);
         }
         const int pg = keep ? table[(size_t)seq * table_w + row / page] : -1;
         cached = pg >= 0;
@@ -535,7 +666,7 @@ extern "C" int tp_rope_kv_write(void* q, long q_stride, void* k, long k_stride, 
                                 int dtype, int M, int H, int KV, int hd, const float* inv_freq, int rot,
                                 const int* row_seq, const int* row_pos, const int* new_len,
                                 const int* table, int table_w, void* k_pool, void* v_pool,
-                                int page, int rows_cap, int pairing, void* stream) {
+                                int page, int rows_cap, int pin, int pairing, void* stream) {
     TP_REQUIRE(M > 0 && H > 0 && hd > 0, "rope_kv_write: empty shape M=%d H=%d hd=%d", M, H, hd);
     TP_REQUIRE(rot >= 0 && rot <= hd && rot % 2 == 0, "rope_kv_write: rotary_dim %d must be even and at most head_dim %d", rot, hd);
     TP_REQUIRE(rot == 0 || inv_freq, "rope_kv_write: a rotation needs its frequency table");
@@ -544,8 +675,9 @@ extern "C" int tp_rope_kv_write(void* q, long q_stride, void* k, long k_stride, 
     // table null: the keys are rotated and nothing is cached
     TP_REQUIRE(!k || (v && KV > 0), "rope_kv_write: keys without values");
     TP_REQUIRE(!k || !table || (k_pool && v_pool && page > 0 && table_w > 0), "rope_kv_write: a page table without cache pools");
-    if (!table) { page = 1; rows_cap = 0; }
+    if (!table) { page = 1; rows_cap = 0; pin = 0; }
     TP_REQUIRE(rows_cap >= 0 && (rows_cap == 0 || rows_cap % page == 0), "rope_kv_write: ring of %d rows is no multiple of the page size %d", rows_cap, page);
+    TP_REQUIRE(pin >= 0 && pin % page == 0 && (pin == 0 || pin < rows_cap), "rope_kv_write: %d rows before a ring must be whole pages and leave it some of %d", pin, rows_cap);
     hipStream_t s = (hipStream_t)stream;
     TP_REQUIRE(H + KV <= 65535, "rope_kv_write: %d heads exceed one launch", H + KV);
     const int heads = H + (k ? KV : 0);
@@ -553,7 +685,7 @@ extern "C" int tp_rope_kv_write(void* q, long q_stride, void* k, long k_stride, 
     if (pairing == TP_ROPE_HALVES && dtype == TP_BF16 && M >= 256 && hd % 8 == 0 && rot % 16 == 0 && rot <= 256 && piecewise(q, q_stride) && piecewise(k, k_stride) &&
         piecewise(v, v_stride) && piecewise(k_pool, 8) && piecewise(v_pool, 8)) {
         rope_kv_write_vec_k<<<M, 256, 0, s>>>((bf16_t*)q, q_stride, (bf16_t*)k, k_stride, (const bf16_t*)v, v_stride, H, KV, hd,
-            inv_freq, rot, row_seq, row_pos, new_len, table, table_w, (bf16_t*)k_pool, (bf16_t*)v_pool, page, rows_cap);
+            inv_freq, rot, row_seq, row_pos, new_len, table, table_w, (bf16_t*)k_pool, (bf16_t*)v_pool, page, rows_cap, pin);
         return tp_check_launch("rope_kv_write");
     }
     // many rows: one block per row shares each pair's cosine and sine over all heads; few rows: a block per head
@@ -562,10 +694,10 @@ extern "C" int tp_rope_kv_write(void* q, long q_stride, void* k, long k_stride, 
     const int threads = hd <= 64 ? 64 : 128;
     if (dtype == TP_BF16)
         rope_kv_write_k<bf16_t><<<grid, threads, 0, s>>>((bf16_t*)q, q_stride, (bf16_t*)k, k_stride, (const bf16_t*)v, v_stride, H, KV, hd,
-            inv_freq, rot, row_seq, row_pos, new_len, table, table_w, (bf16_t*)k_pool, (bf16_t*)v_pool, page, rows_cap, hpb, pairing);
+            inv_freq, rot, row_seq, row_pos, new_len, table, table_w, (bf16_t*)k_pool, (bf16_t*)v_pool, page, rows_cap, pin, hpb, pairing);
     else if (dtype == TP_F32)
         rope_kv_write_k<float><<<grid, threads, 0, s>>>((float*)q, q_stride, (float*)k, k_stride, (const float*)v, v_stride, H, KV, hd,
-            inv_freq, rot, row_seq, row_pos, new_len, table, table_w, (float*)k_pool, (float*)v_pool, page, rows_cap, hpb, pairing);
+            inv_freq, rot, row_seq, row_pos, new_len, table, table_w, (float*)k_pool, (float*)v_pool, page, rows_cap, pin, hpb, pairing);
     else return tp_fail("rope_kv_write: unknown dtype %d", dtype);
     return tp_check_launch("rope_kv_write");
 }
@@ -578,12 +710,12 @@ template <typename T>
 __global__ void __launch_bounds__(256)
 kv_write_k(const T* __restrict__ k, long k_stride, const T* __restrict__ v, long v_stride, int KV, int hd,
            const int* __restrict__ row_seq, const int* __restrict__ row_pos, const int* __restrict__ new_len,
-           const int* __restrict__ table, int table_w, T* __restrict__ k_pool, T* __restrict__ v_pool, int page, int rows_cap) {
+           const int* __restrict__ table, int table_w, T* __restrict__ k_pool, T* __restrict__ v_pool, int page, int rows_cap, int pin) {
     const int r = blockIdx.x, seq = row_seq[r], pos = row_pos[r];
     int row = pos;
-    if (rows_cap > 0) {
-        if (pos + rows_cap < new_len[seq]) return;       // a later row of this step takes the same ring row
-        row = pos % rows_cap;
+    if (rows_cap > 0 && pos >= pin) {
+        if (pos + rows_cap - pin < new_len[seq]) return; // a later row of this step takes the same ring row
+        row = pin + (pos - pin) % (rows_cap - pin);
     }
     const int pg = table[(size_t)seq * table_w + row / page];
     if (pg < 0) return;                                  // never for a position the cache has room for
@@ -611,18 +743,19 @@ kv_write_k(const T* __restrict__ k, long k_stride, const T* __restrict__ v, long
 
 extern "C" int tp_kv_write(const void* k, long k_stride, const void* v, long v_stride, int dtype, int M, int KV, int hd,
                            const int* row_seq, const int* row_pos, const int* new_len, const int* table, int table_w,
-                           void* k_pool, void* v_pool, int page, int rows_cap, void* stream) {
+                           void* k_pool, void* v_pool, int page, int rows_cap, int pin, void* stream) {
     TP_REQUIRE(M > 0 && KV > 0 && hd > 0 && page > 0 && table_w > 0, "kv_write: empty shape");
     TP_REQUIRE(k && v && row_seq && row_pos && new_len && table && k_pool && v_pool, "kv_write: a null operand");
     TP_REQUIRE(k_stride >= (long)KV * hd && v_stride >= (long)KV * hd, "kv_write: rows are too short for %d heads of %d", KV, hd);
     TP_REQUIRE(rows_cap >= 0 && (rows_cap == 0 || rows_cap % page == 0), "kv_write: ring of %d rows is no multiple of the page size %d", rows_cap, page);
+    TP_REQUIRE(pin >= 0 && pin % page == 0 && (pin == 0 || pin < rows_cap), "kv_write: %d rows before a ring must be whole pages and leave it some of %d", pin, rows_cap);
     hipStream_t s = (hipStream_t)stream;
     if (dtype == TP_BF16)
         kv_write_k<bf16_t><<<M, 256, 0, s>>>((const bf16_t*)k, k_stride, (const bf16_t*)v, v_stride, KV, hd, row_seq, row_pos, new_len,
-                                             table, table_w, (bf16_t*)k_pool, (bf16_t*)v_pool, page, rows_cap);
+                                             table, table_w, (bf16_t*)k_pool, (bf16_t*)v_pool, page, rows_cap, pin);
     else if (dtype == TP_F32)
         kv_write_k<float><<<M, 256, 0, s>>>((const float*)k, k_stride, (const float*)v, v_stride, KV, hd, row_seq, row_pos, new_len,
-                                            table, table_w, (float*)k_pool, (float*)v_pool, page, rows_cap);
+                                            table, table_w, (float*)k_pool, (float*)v_pool, page, rows_cap, pin);
     else return tp_fail("kv_write: unknown dtype %d", dtype);
     return tp_check_launch("kv_write");
 }

@@ -3,7 +3,7 @@
 #pragma once
 #include "common.h"
 
-enum { TP_EPI_NONE = 0, TP_EPI_SOFTCAP = 1, TP_EPI_GATED = 2 };
+enum { TP_EPI_NONE = 0, TP_EPI_SOFTCAP = 1, TP_EPI_GATED = 2, TP_EPI_RELU2 = 3 };
 // steps of 64 k a wave of the 8-row kernel has in flight at once: four waves a block read a K of 2,304 in one round of loads
 #define TP_R8_MAX_STEPS 9
 
@@ -26,6 +26,12 @@ static inline float4 epi_constants(const GemmArgs& a) {
     float4 e = make_float4(a.cap, 0.f, a.limit, a.shift);
     if (a.epilogue == TP_EPI_GATED) tp_gate_constants(a.act, &e.x, &e.y);
     return e;
+}
+
+// an output element of a product that is not gated: as summed, under a cap, or max(o, 0)^2 (a feed-forward without a gate)
+__device__ __forceinline__ float squared_relu_f(float o) { o = fmaxf(o, 0.f); return o * o; }
+__device__ __forceinline__ float plain_epilogue(int epilogue, float o, float4 epi) {
+    return epilogue == TP_EPI_SOFTCAP ? softcap_f(o, epi.x) : (epilogue == TP_EPI_RELU2 ? squared_relu_f(o) : o);
 }
 
 // plain tiled kernel, any dtype and shape; one fixed summation order per output element

@@ -12,7 +12,7 @@
 // for the few rows of a decode step, where a narrow product would otherwise run on a few dozen blocks.
 template <typename TI, typename TO, int R, int BK>
 __global__ void __launch_bounds__(256)
-gemm_simple_k(const TI* __restrict__ X, const TI* __restrict__ W, TO* __restrict__ Y, int M, int N, int K, float cap) {
+gemm_simple_k(const TI* __restrict__ X, const TI* __restrict__ W, TO* __restrict__ Y, int M, int N, int K, int epilogue, float4 epi) {
     constexpr int T = 16 * R;
     __shared__ float xs[BK][T + 1];
     __shared__ float ws[BK][T + 1];
@@ -48,9 +48,7 @@ gemm_simple_k(const TI* __restrict__ X, const TI* __restrict__ W, TO* __restrict
         for (int j = 0; j < R; j++) {
             const int n = n0 + tx * R + j;
             if (n >= N) continue;
-            float v = acc[i][j];
-            if (cap > 0.f) v = softcap_f(v, cap);
-            st_f32(Y + (size_t)m * N + n, v);
+            st_f32(Y + (size_t)m * N + n, plain_epilogue(epilogue, acc[i][j], epi));
         }
     }
 }
@@ -58,20 +56,21 @@ gemm_simple_k(const TI* __restrict__ X, const TI* __restrict__ W, TO* __restrict
 extern "C" int tp_gated_act(const float* y, void* out, int dtype, int M, int I, int act, float limit, float shift, void* stream);
 
 template <typename TI>
-static int simple_typed(const GemmArgs& a, void* y, int out_dtype, float cap) {
+static int simple_typed(const GemmArgs& a, void* y, int out_dtype, int epilogue) {
+    const float4 epi = make_float4(a.cap, 0.f, 0.f, 0.f);
     if (a.M <= 16) {
         dim3 grid(tp_cdiv(a.N, 16), 1);
         if (out_dtype == TP_F32)
-            gemm_simple_k<TI, float, 1, 64><<<grid, 256, 0, a.stream>>>((const TI*)a.x, (const TI*)a.w, (float*)y, a.M, a.N, a.K, cap);
+            gemm_simple_k<TI, float, 1, 64><<<grid, 256, 0, a.stream>>>((const TI*)a.x, (const TI*)a.w, (float*)y, a.M, a.N, a.K, epilogue, epi);
         else
-            gemm_simple_k<TI, bf16_t, 1, 64><<<grid, 256, 0, a.stream>>>((const TI*)a.x, (const TI*)a.w, (bf16_t*)y, a.M, a.N, a.K, cap);
+            gemm_simple_k<TI, bf16_t, 1, 64><<<grid, 256, 0, a.stream>>>((const TI*)a.x, (const TI*)a.w, (bf16_t*)y, a.M, a.N, a.K, epilogue, epi);
         return tp_check_launch("linear (plain kernel, few rows)");
     }
     dim3 grid(tp_cdiv(a.N, 64), tp_cdiv(a.M, 64));
     if (out_dtype == TP_F32)
-        gemm_simple_k<TI, float, 4, 16><<<grid, 256, 0, a.stream>>>((const TI*)a.x, (const TI*)a.w, (float*)y, a.M, a.N, a.K, cap);
+        gemm_simple_k<TI, float, 4, 16><<<grid, 256, 0, a.stream>>>((const TI*)a.x, (const TI*)a.w, (float*)y, a.M, a.N, a.K, epilogue, epi);
     else
-        gemm_simple_k<TI, bf16_t, 4, 16><<<grid, 256, 0, a.stream>>>((const TI*)a.x, (const TI*)a.w, (bf16_t*)y, a.M, a.N, a.K, cap);
+        gemm_simple_k<TI, bf16_t, 4, 16><<<grid, 256, 0, a.stream>>>((const TI*)a.x, (const TI*)a.w, (bf16_t*)y, a.M, a.N, a.K, epilogue, epi);
     return tp_check_launch("linear (plain kernel)");
 }
 
@@ -83,8 +82,8 @@ int gemm_simple_launch(const GemmArgs& a) {
         y = a.workspace;
         out_dtype = TP_F32;
     }
-    const float cap = a.epilogue == TP_EPI_SOFTCAP ? a.cap : 0.f;
-    int rc = a.in_dtype == TP_BF16 ? simple_typed<bf16_t>(a, y, out_dtype, cap) : simple_typed<float>(a, y, out_dtype, cap);
+    const int epilogue = a.epilogue == TP_EPI_GATED ? TP_EPI_NONE : a.epilogue;     // the activation of a gated product is a launch of its own here
+    int rc = a.in_dtype == TP_BF16 ? simple_typed<bf16_t>(a, y, out_dtype, epilogue) : simple_typed<float>(a, y, out_dtype, epilogue);
     if (rc) return rc;
     if (a.epilogue == TP_EPI_GATED) return tp_gated_act((const float*)y, a.y, a.out_dtype, a.M, a.units, a.act, a.limit, a.shift, a.stream);
     return 0;

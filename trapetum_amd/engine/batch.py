@@ -110,6 +110,7 @@ class StepContext:
         self.max_count = max(self.counts)
         self.entry = None               # schedule entry now running
         self.cache_owner = None         # entry whose cache it uses
+        self.origin = None              # the embedding's rows, where a model adds them again later in the step
         self.static = static
         self.length_bound = length_bound
         self._shared = set()            # entries whose cache a later entry reads

@@ -11,6 +11,7 @@ import torch
 
 from ..cache.store import ModelCache
 from ..models.spec import ModelSpec
+from ..parts.blocks import NormAfterAdd, join_then_norm
 from ..registry import build_part, part_class
 from .batch import StepContext, StepError, classify
 
@@ -53,6 +54,9 @@ class Model:
         self.places = [(self.embedding, spec.embedding_prefix)]
         for layer in self.layers:
             self.places.extend(layer.places)
+        # what the model adds to the stream before a run of a layer, by schedule entry
+        self.added = [build_part("stream_add", e.before) if e.before is not None else None for e in spec.schedule]
+        self.places.extend((p, e.before_prefix) for p, e in zip(self.added, spec.schedule) if p is not None)
         self.places.append((self.final_norm, spec.final_norm_prefix))
         self.places.append((self.head, spec.head_prefix))
         self.schedule = spec.schedule
@@ -178,6 +182,8 @@ class Model:
         cache = ctx.cache
         stream = self.embedding.forward(ctx, tok)
         ctx.dump("embed", stream)
+        if any(p is not None and p.needs_origin for p in self.added):
+            ctx.origin = stream.clone()
         whole = ctx.n_want == ctx.n_rows and ctx.identity_want
         normed = None
         last = len(self.schedule) - 1
@@ -191,6 +197,11 @@ class Model:
                 next_norm = self.final_norm if whole else None
             if next_norm is not None and next_norm.gain is None:
                 next_norm = None
+            if next_norm is not None and i < last and self.added[i + 1] is not None:
+                next_norm = NormAfterAdd(next_norm, self.added[i + 1])
+            if self.added[i] is not None and normed is None:     # else the block before has added it, with its last add
+                norm = self.layers[e.layer].block.entry_norm()
+                normed = join_then_norm(ctx, stream, None, None, NormAfterAdd(norm if norm is not None and norm.gain is not None else None, self.added[i]))
             stream, normed = self.layers[e.layer].block.forward(ctx, stream, cache.site(ctx.cache_owner),
                                                                  normed=normed, next_norm=next_norm)
         ctx.finish()

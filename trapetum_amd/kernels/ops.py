@@ -17,13 +17,14 @@ _CORE_SIGS = {
     "tp_embed_rows": [_P, _P, _I, _F, _P, _I, _I, _I, _P],
     "tp_rms_norm": [_P, _I, _P, _F, _P, _I, _I, _I, _I, _P],
     "tp_add_rms_norm": [_P, _P, _I, _I, _L, _P, _F, _P, _F, _P, _I, _I, _I, _I, _P],
+    "tp_join_rms_norm": [_P, _P, _I, _I, _L, _P, _I, _I, _L, _P, _P, _P, _F, _P, _I, _I, _I, _P],
     "tp_scale_rows": [_P, _L, _F, _P],
     "tp_causal_conv": [_P, _P, _P, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _I, _P],
     "tp_latent_prepare": [_P, _L, _I, _I, _I, _I, _I, _I, _P, _F, _P, _I, _P, _P, _P, _P, _I, _P, _I, _I, _P, _P, _I, _P, _L, _P],
     "tp_head_linear": [_P, _L, _L, _P, _P, _L, _L, _I, _I, _I, _I, _I, _I, _P],
-    "tp_route_top": [_P, _I, _I, _I, _I, _I, _P, _P, _P],
+    "tp_route_top": [_P, _I, _I, _I, _I, _I, _P, _F, _P, _P, _P],
     "tp_expert_ffn_workspace_bytes": [_I, _I, _I, _I, _I, _I],
-    "tp_expert_ffn": [_P, _I, _I, _I, _P, _P, _I, _I, _I, _P, _P, _F, _F, _F, _I, _P, _L, _P, _I, _P],
+    "tp_expert_ffn": [_P, _I, _I, _I, _P, _P, _I, _I, _I, _P, _P, _I, _F, _F, _F, _I, _P, _L, _P, _I, _P],
     "tp_conv_act": [_P, _L, _I, _P, _P, _P, _P, _P, _P, _P, _L, _I, _I, _I, _I, _I, _I, _I, _P],
     "tp_ssd_scan_workspace_bytes": [_I, _I, _I, _I, _I, _I],
     "tp_ssd_scan": [_P, _L, _P, _L, _P, _L, _I, _P, _P, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _I, _P, _L, _P],
@@ -31,8 +32,8 @@ _CORE_SIGS = {
     "tp_mul_sigmoid": [_P, _L, _P, _L, _I, _I, _I, _P],
     "tp_gather_rows": [_P, _P, _P, _I, _I, _I, _P],
     "tp_sum_slices": [_P, _I, _L, _P, _I, _L, _P],
-    "tp_rope_kv_write": [_P, _L, _P, _L, _P, _L, _I, _I, _I, _I, _I, _P, _I, _P, _P, _P, _P, _I, _P, _P, _I, _I, _I, _P],
-    "tp_kv_write": [_P, _L, _P, _L, _I, _I, _I, _I, _P, _P, _P, _P, _I, _P, _P, _I, _I, _P],
+    "tp_rope_kv_write": [_P, _L, _P, _L, _P, _L, _I, _I, _I, _I, _I, _P, _I, _P, _P, _P, _P, _I, _P, _P, _I, _I, _I, _I, _P],
+    "tp_kv_write": [_P, _L, _P, _L, _I, _I, _I, _I, _P, _P, _P, _P, _I, _P, _P, _I, _I, _I, _P],
     "tp_gated_act": [_P, _P, _I, _I, _I, _I, _F, _F, _P],
     "tp_linear": [_P, _P, _P, _I, _I, _I, _I, _I, _I, _F, _I, _I, _F, _F, _P, _L, _I, _I, _P],
     "tp_shift_mix": [_P, _I, _P, _I, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _P],
@@ -48,11 +49,13 @@ _CORE_SIGS = {
     "tp_head_norm_gate": [_P, _P, _P, _L, _I, _F, _P, _I, _I, _I, _I, _I, _P],
     "tp_time_mix_scan": [_P, _L, _P, _L, _P, _L, _I, _P, _P, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _P, _P],
     "tp_matrix_memory_scan": [_P, _L, _P, _L, _P, _L, _I, _P, _F, _F, _P, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _P, _P],
+    "tp_delta_scan": [_P, _L, _P, _L, _P, _L, _P, _P, _L, _I, _P, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _F, _I, _P, _L, _P],
+    "tp_delta_scan_workspace_bytes": [_I, _I, _I, _I, _I],
     "tp_time_mix_scan_workspace_floats": [_I, _I, _I, _I],
     "tp_matrix_memory_scan_workspace_floats": [_I, _I, _I, _I, _I],
     "tp_linear_workspace_bytes": [_I, _I, _I, _I, _I, _I, _I, _I, _I],
-    "tp_attn_simple_prefill": [_P, _L, _P, _L, _P, _L, _I, _I, _I, _I, _I, _P, _P, _P, _P, _P, _I, _P, _P, _I, _I, _F, _F, _I, _I, _P, _P, _P, _P],
-    "tp_attn_simple_decode": [_P, _L, _I, _I, _I, _I, _I, _P, _P, _I, _P, _P, _I, _I, _F, _F, _I, _I, _P, _P, _P, _P],
+    "tp_attn_simple_prefill": [_P, _L, _P, _L, _P, _L, _I, _I, _I, _I, _I, _P, _P, _P, _P, _P, _I, _P, _P, _I, _I, _F, _F, _I, _I, _P, _P, _I, _I, _P, _P],
+    "tp_attn_simple_decode": [_P, _L, _I, _I, _I, _I, _I, _P, _P, _I, _P, _P, _I, _I, _F, _F, _I, _I, _P, _P, _I, _I, _P, _P],
     "tp_argmax": [_P, _I, _I, _P, _P, _P],
     "tp_argmax_workspace_bytes": [_I, _I],
     "tp_repetition_penalty": [_P, _I, _I, _P, _I, _F, _P],
@@ -64,18 +67,20 @@ _CORE_SIGS = {
     "tp_probe_mfma": [_I, _I, _I, _P, _P, _P],
 }
 _ATTN_SIGS = {
-    "tp_attn_prefill": [_P, _L, _P, _L, _P, _L, _I, _I, _I, _P, _I, _I, _P, _P, _I, _P, _P, _I, _I, _F, _F, _I, _I, _P, _P, _P, _I, _P],
-    "tp_attn_decode": [_P, _L, _I, _I, _I, _P, _P, _I, _P, _P, _I, _I, _F, _F, _I, _I, _P, _P, _P, _P, _I, _P],
+    "tp_attn_prefill": [_P, _L, _P, _L, _P, _L, _I, _I, _I, _P, _I, _I, _P, _P, _I, _P, _P, _I, _I, _F, _F, _I, _I, _P, _P, _I, _I, _P, _I, _P],
+    "tp_attn_decode": [_P, _L, _I, _I, _I, _P, _P, _I, _P, _P, _I, _I, _F, _F, _I, _I, _P, _P, _I, _I, _P, _P, _I, _P],
     "tp_attn_decode_shared": [_P, _L, _I, _I, _I, _I, _P, _P, _I, _P, _P, _I, _I, _F, _F, _I, _P, _P, _I, _P],
     "tp_attn_decode_workspace_floats": [_I, _I, _I],
     "tp_attn_pooled_tile": [_P, _L, _P, _L, _P, _L, _I, _I, _I, _I, _P, _P, _P, _I, _P, _P, _I, _I, _P, _I, _P, _P, _I, _F, _F, _I, _I, _P, _P],
-    "tp_attn_decode_fused": [_P, _I, _I, _L, _L, _P, _I, _I, _I, _I, _I, _P, _P, _I, _P, _P, _I, _I, _F, _F, _I, _P, _P, _I, _P],
+    "tp_attn_decode_fused": [_P, _I, _I, _L, _L, _P, _I, _I, _I, _I, _I, _P, _P, _I, _P, _P, _I, _I, _F, _F, _I, _P, _I, _I, _P, _P, _I, _P],
 }
 
-EPI_NONE, EPI_SOFTCAP, EPI_GATED = 0, 1, 2
+EPI_NONE, EPI_SOFTCAP, EPI_GATED, EPI_RELU2 = 0, 1, 2, 3
+PLAIN_ACTIVATIONS = {"relu2": EPI_RELU2}              # what a product without a gate can apply to its sums: max(z, 0)^2
 ROPE_PAIRINGS = {"halves": 0, "neighbours": 1}          # the kernel library's TP_ROPE_* enumerators
 GATE_ACTIVATIONS = {"gelu_tanh": 0, "silu": 1, "relu": 2, "quick_gelu": 3}       # what a gated product's epilogue can apply to the gate
 HEAD_GATES = {"sigmoid": 0, "silu": 1}               # what `head_norm_gate` multiplies a normed head by: act(g)
+EXPERT_KINDS = {"gated": 1, "relu2": 2}              # g sigmoid(alpha g) (u + shift) of two matrices; max(z, 0)^2 of one
 ROUTE_SCORES = {"softmax": 0, "sigmoid": 1}          # how a router's logits become scores
 CONV_ACTIVATIONS = {None: 0, "silu": 1}
 BIAS_ACTIVATIONS = {None: 0, "gelu_erf": 1}          # what `bias_act` applies after the bias
@@ -271,6 +276,35 @@ class HipOps:
                    out.data_ptr() if out is not None else None, _code(out_dtype), m, d, int(groups), self._stream())
         return out
 
+    def join_rms_norm(self, stream, a, b, gain, eps, out_dtype, vec=None, origin=None):
+        """stream += a + b (+ vec) (+ origin); returns norm(stream), or None without a gain.  a, b: rows [M, D] (a tensor of
+        either dtype, or SplitRows), b or both may be None; vec float32 [D] goes to every row, origin float32 [M, D]."""
+        m, d = stream.shape
+        self._dev(stream, gain, vec, origin)
+        if stream.dtype != torch.float32 or not stream.is_contiguous():
+            raise KernelError("join_rms_norm: the stream must be contiguous float32")
+        args, held = [], []
+        for r in (a, b):
+            if r is None:
+                args += [None, 0, 1, 0]
+                continue
+            n_slices, stride = 1, 0
+            if isinstance(r, SplitRows):
+                n_slices, stride, r = r.slices.shape[0], r.slices.stride(0), r.slices[0]
+            self._dev(r)
+            if tuple(r.shape) != (m, d) or not r.is_contiguous():
+                raise KernelError(f"join_rms_norm: rows {tuple(r.shape)} do not match the stream {(m, d)}")
+            held.append(r)
+            args += [r.data_ptr(), _code(r.dtype), n_slices, stride]
+        for t, n, what in ((gain, d, "gain"), (vec, d, "vector"), (origin, m * d, "earlier rows")):
+            if t is not None and (t.dtype != torch.float32 or t.numel() != n or not t.is_contiguous()):
+                raise KernelError(f"join_rms_norm: the {what} must be contiguous float32 of {n} elements")
+        out = torch.empty((m, d), dtype=out_dtype, device=self.device) if gain is not None else None
+        ptr = lambda t: t.data_ptr() if t is not None else None
+        self._call(self.lib, "tp_join_rms_norm", stream.data_ptr(), *args, ptr(vec), ptr(origin), ptr(gain), float(eps), ptr(out),
+                   _code(out_dtype), m, d, self._stream())
+        return out
+
     def scale_rows(self, x, scale):
         """x *= scale, in place (float32)."""
         self._dev(x)
@@ -369,9 +403,10 @@ class HipOps:
         return out
 
     # ---- mixture of experts ------------------------------------------------------------------------------------
-    def route_top(self, logits, top, renormalize=False, score="softmax"):
+    def route_top(self, logits, top, renormalize=False, score="softmax", correction=None, scale=1.0):
         """Scores: softmax over all experts, or the sigmoid of each logit; the `top` largest scores (ties: the smaller
-        index): int32 [M, top], float32 [M, top]."""
+        index): int32 [M, top], float32 [M, top].  correction: float32 [experts] added to the scores for the choice alone.
+        renormalize: the chosen scores over their sum (+ 1e-20).  scale: a factor on every weight."""
         if score not in ROUTE_SCORES:
             raise KernelError(f"route_top: score '{score}' has no kernel ({', '.join(ROUTE_SCORES)})")
         self._dev(logits)
@@ -380,17 +415,24 @@ class HipOps:
         m, e = logits.shape
         if not 0 < top <= e:
             raise KernelError(f"route_top: {top} of {e} experts cannot be chosen")
+        if correction is not None and (correction.dtype != torch.float32 or correction.numel() != e or not correction.is_contiguous()):
+            raise KernelError(f"route_top: the correction must be contiguous float32 [{e}]")
+        self._dev(correction)
         chosen = torch.empty((m, top), dtype=torch.int32, device=self.device)
         weight = torch.empty((m, top), dtype=torch.float32, device=self.device)
-        self._call(self.lib, "tp_route_top", logits.data_ptr(), m, e, int(top), 1 if renormalize else 0, ROUTE_SCORES[score], chosen.data_ptr(),
-                   weight.data_ptr(), self._stream())
+        self._call(self.lib, "tp_route_top", logits.data_ptr(), m, e, int(top), 1 if renormalize else 0, ROUTE_SCORES[score],
+                   correction.data_ptr() if correction is not None else None, float(scale), chosen.data_ptr(), weight.data_ptr(), self._stream())
         return chosen, weight
 
-    def expert_ffn(self, x, chosen, weights, w_gate_up, w_down, limit, alpha, shift, weight_input=False, out=None):
+    def expert_ffn(self, x, chosen, weights, w_gate_up, w_down, limit, alpha, shift, weight_input=False, out=None, kind="gated"):
         """float32 [M, D]: sum over a row's chosen experts of weight * W_down,e (g' sigmoid(alpha g') (u' + shift)), with
         g' = min(W_gate,e x, limit), u' = clamp(W_up,e x, -limit, limit).  w_gate_up [E, 2 F, D] (gate rows, then up
         rows), w_down [E, D, F].  limit None: no clamp.  weight_input: the weight multiplies the expert's input instead,
-        expert(weight * x), and the outputs are summed as they are.  out: a contiguous float32 [M, D] to fill."""
+        expert(weight * x), and the outputs are summed as they are.  out: a contiguous float32 [M, D] to fill.
+        kind "relu2": experts without a gate, W_down,e max(W_up,e x, 0)^2 with w_gate_up [E, F, D] (limit, alpha and shift
+        say nothing).  A choice of E and above is no expert with matrices: its output is the row x itself (times the weight)."""
+        if kind not in EXPERT_KINDS:
+            raise KernelError(f"expert_ffn: kind '{kind}' has no kernel ({', '.join(EXPERT_KINDS)})")
         limit = float("inf") if limit is None else limit
         self._dev(x, chosen, weights, w_gate_up, w_down)
         if x.dim() != 2 or not x.is_contiguous() or x.dtype != w_gate_up.dtype or x.dtype != w_down.dtype:
@@ -399,8 +441,8 @@ class HipOps:
         if w_gate_up.dim() != 3 or w_down.dim() != 3 or not w_gate_up.is_contiguous() or not w_down.is_contiguous():
             raise KernelError("expert_ffn: the experts' matrices must be contiguous [experts, rows, columns]")
         e, f2, _ = w_gate_up.shape
-        f = f2 // 2
-        if f2 % 2 or w_gate_up.shape[2] != d or tuple(w_down.shape) != (e, d, f):
+        f = f2 // 2 if kind == "gated" else f2
+        if (kind == "gated" and f2 % 2) or w_gate_up.shape[2] != d or tuple(w_down.shape) != (e, d, f):
             raise KernelError(f"expert_ffn: matrices {tuple(w_gate_up.shape)} and {tuple(w_down.shape)} do not fit rows of {d}")
         top = chosen.shape[1]
         if chosen.dtype != torch.int32 or tuple(chosen.shape) != (m, top) or weights.dtype != torch.float32 or tuple(weights.shape) != (m, top) \
@@ -414,7 +456,7 @@ class HipOps:
             raise KernelError(f"expert_ffn: the output must be contiguous float32 {(m, d)}")
         self._dev(out)
         self._call(self.lib, "tp_expert_ffn", x.data_ptr(), _code(x.dtype), m, d, chosen.data_ptr(), weights.data_ptr(), top, e, f,
-                   w_gate_up.data_ptr(), w_down.data_ptr(), float(limit), float(alpha), float(shift), 1 if weight_input else 0,
+                   w_gate_up.data_ptr(), w_down.data_ptr(), EXPERT_KINDS[kind], float(limit), float(alpha), float(shift), 1 if weight_input else 0,
                    ws.data_ptr(), nbytes,
                    out.data_ptr(), 1 if self.force_linear == 1 else 0, self._stream())
         return out
@@ -632,6 +674,48 @@ class HipOps:
                    self._stream())
         return y
 
+    DELTA_CHUNK = 64               # tokens of a chunk (the kernel library's)
+    DELTA_CHUNKS_FROM = 48         # rows of the longest sequence from which a bfloat16 step runs in chunks
+
+    def delta_scan(self, q, k, v, b, a, a_log, dt_bias, state, slot_ids, cu_rows, max_count, heads, kv_heads, dk, dv, q_scale, chunks=None):
+        """The gated delta rule over the step's rows, sequence by sequence, from state[slot] (float32 [slots, heads, dk,
+        dv]), which it leaves updated: with unit vectors k and q (q also times q_scale), beta = sigmoid(b) and
+        g = exp(-exp(a_log) softplus(a + dt_bias)),
+            S <- g S,  u = beta (v - S^T k),  S <- S + k u^T,  o = S^T q.
+        q, k [M, kv_heads dk] (head h uses q and k of h // (heads / kv_heads)), v [M, heads dv], b and a [M, heads]: views of wider
+        rows of one dtype, b and a of the same rows.  Returns float32 [M, heads dv].  chunks: whether the step runs in
+        chunks on the matrix cores (None: where it can and pays)."""
+        self._dev(q, k, v, b, a, a_log, dt_bias, state, slot_ids, cu_rows)
+        m = q.shape[0]
+        qs, ks, vs = self._rows(q, "delta_scan q"), self._rows(k, "delta_scan k"), self._rows(v, "delta_scan v")
+        bs, as_ = self._rows(b, "delta_scan b"), self._rows(a, "delta_scan a")
+        if tuple(q.shape) != (m, kv_heads * dk) or tuple(k.shape) != (m, kv_heads * dk) or tuple(v.shape) != (m, heads * dv) \
+                or tuple(a.shape) != (m, heads) or tuple(b.shape) != (m, heads) or bs != as_:
+            raise KernelError(f"delta_scan: q, k {(m, kv_heads * dk)}, v {(m, heads * dv)}, and b and a {(m, heads)} of the same rows")
+        if not (q.dtype == k.dtype == v.dtype == a.dtype == b.dtype):
+            raise KernelError("delta_scan: q, k, v, b and a share one dtype")
+        if heads % kv_heads or dk > self.MAX_SCAN_DIM:
+            raise KernelError(f"delta_scan: {heads} heads on {kv_heads} kv heads of {dk} key elements (at most {self.MAX_SCAN_DIM})")
+        for t in (a_log, dt_bias):
+            if t.dtype != torch.float32 or t.numel() != heads or not t.is_contiguous():
+                raise KernelError(f"delta_scan: a_log and dt_bias must be contiguous float32 [{heads}]")
+        if state.dtype != torch.float32 or state.dim() != 4 or tuple(state.shape[1:]) != (heads, dk, dv) or not state.is_contiguous():
+            raise KernelError(f"delta_scan: the state must be contiguous float32 [slots, {heads}, {dk}, {dv}]")
+        n_seq = self._geometry("delta_scan", m, slot_ids, cu_rows)
+        can = q.dtype == torch.bfloat16 and dk % 8 == 0 and qs % 8 == 0 and ks % 8 == 0 and q.data_ptr() % 16 == 0 and k.data_ptr() % 16 == 0
+        if chunks is None:
+            chunks = can and int(max_count) >= self.DELTA_CHUNKS_FROM
+        elif chunks and not can:
+            raise KernelError("delta_scan: chunks need bfloat16 rows of whole 16-byte pieces")
+        n_chunks = -(-int(max_count) // self.DELTA_CHUNK) if chunks else 0
+        nbytes = self.lib.tp_delta_scan_workspace_bytes(n_seq, n_chunks, heads, kv_heads, dk) if chunks else 0
+        ws = torch.empty(nbytes, dtype=torch.uint8, device=self.device) if nbytes else None
+        y = torch.empty((m, heads * dv), dtype=torch.float32, device=self.device)
+        self._call(self.lib, "tp_delta_scan", q.data_ptr(), qs, k.data_ptr(), ks, v.data_ptr(), vs, b.data_ptr(), a.data_ptr(), bs, _code(q.dtype),
+                   a_log.data_ptr(), dt_bias.data_ptr(), state.data_ptr(), slot_ids.data_ptr(), cu_rows.data_ptr(), y.data_ptr(), n_seq, heads,
+                   kv_heads, dk, dv, float(q_scale), n_chunks, ws.data_ptr() if ws is not None else None, nbytes, self._stream())
+        return y
+
     def pair_norm_mean(self, a, b, gain_a, gain_b, eps):
         """float32 [M, D]: 0.5 (a / rms(a) * gain_a + b / rms(b) * gain_b), each row over its own root mean square."""
         self._dev(a, b, gain_a, gain_b)
@@ -709,7 +793,7 @@ class HipOps:
         return out
 
     def rope_kv_write(self, q, k, v, H, KV, hd, inv_freq, rotary_dim, row_seq, row_pos, new_len, table,
-                      k_pool, v_pool, rows_cap, pairing="halves", write=True):
+                      k_pool, v_pool, rows_cap, pairing="halves", write=True, pin=0):
         """Rotate q and k in place and write k, v into the cache.  write=False: rotate only (a step whose attention
         reads the cache as earlier steps left it caches its rows afterwards, with `kv_write`).
         pairing: one of ROPE_PAIRINGS, which elements of a head turn together."""
@@ -741,9 +825,9 @@ class HipOps:
                    inv_freq.data_ptr() if rotary_dim else None, rotary_dim, row_seq.data_ptr(), row_pos.data_ptr(),
                    new_len.data_ptr(), table.data_ptr() if write else None, table_w,
                    k_pool.data_ptr() if write else None, v_pool.data_ptr() if write else None,
-                   page, rows_cap if write else 0, ROPE_PAIRINGS[pairing], self._stream())
+                   page, rows_cap if write else 0, int(pin) if write else 0, ROPE_PAIRINGS[pairing], self._stream())
 
-    def kv_write(self, k, v, KV, hd, row_seq, row_pos, new_len, table, k_pool, v_pool, rows_cap):
+    def kv_write(self, k, v, KV, hd, row_seq, row_pos, new_len, table, k_pool, v_pool, rows_cap, pin=0):
         """The step's keys (rotated already) and values into the cache: what `rope_kv_write(write=False)` left undone."""
         self._dev(k, v, row_seq, row_pos, new_len, table, k_pool, v_pool)
         m = k.shape[0]
@@ -756,7 +840,7 @@ class HipOps:
         self._check_pools("kv_write", k.dtype, new_len.numel(), KV, hd, new_len, table, k_pool, v_pool)
         self._call(self.lib, "tp_kv_write", k.data_ptr(), ks, v.data_ptr(), vs, _code(k.dtype), m, KV, hd, row_seq.data_ptr(),
                    row_pos.data_ptr(), new_len.data_ptr(), table.data_ptr(), table.shape[1], k_pool.data_ptr(),
-                   v_pool.data_ptr(), k_pool.shape[2], rows_cap, self._stream())
+                   v_pool.data_ptr(), k_pool.shape[2], rows_cap, int(pin), self._stream())
 
     # ---- attention over a window and pooled blocks ------------------------------------------------------
     def qkv_prepare(self, x, bias, H, KV, row, dim, inv_freq, rotary_dim, row_pos, unit_eps, out_dtype, pairing="halves"):
@@ -897,6 +981,12 @@ class HipOps:
                    ws.data_ptr() if ws is not None else None, nbytes, 0, algo, self._stream())
         return out
 
+    def linear_act(self, x, w, out_dtype, activation):
+        """act(x @ w^T), the activation applied to the float32 sums before they are rounded; one of PLAIN_ACTIVATIONS."""
+        if activation not in PLAIN_ACTIVATIONS:
+            raise KernelError(f"linear_act: activation '{activation}' has no kernel ({', '.join(PLAIN_ACTIVATIONS)})")
+        return self._linear(x, w, out_dtype, PLAIN_ACTIVATIONS[activation], 0.0, 0)
+
     def linear(self, x, w, out_dtype, softcap=None, defer=False, bias=None, out=None):
         """x @ w^T (+ bias).  defer: the caller hands the result to `add_rms_norm` (or through `rows()`), so a product
         computed in K slices may come back as SplitRows.  bias: float32 [rows of w], added by a kernel of its own
@@ -940,7 +1030,8 @@ class HipOps:
             (not decode or H // KV <= self.DECODE_GROUP)
 
     def attention_prefill(self, q, k, v, H, KV, hd, cu_rows, max_count, scale, softcap, window, out_dtype,
-                          row_seq=None, row_pos=None, cached=None, shape=0, wide_weights=False, chunk=0, head_scale=None, sink=None):
+                          row_seq=None, row_pos=None, cached=None, shape=0, wide_weights=False, chunk=0, head_scale=None, sink=None,
+                          keep=0, pin=0):
         """Causal attention of the step's queries over the step's own rows of keys and values and, with
         `cached` = (new_len, table, k_pool, v_pool, rows_cap), over the positions before them, read in place from the
         cache as earlier steps left it (the step's own rows are not looked for there).  Without `cached` every sequence
@@ -949,7 +1040,8 @@ class HipOps:
         wide_weights: the matrix-core kernel multiplies the values by softmax weights of 16 bits of mantissa (two bf16
         terms) instead of 8; the plain kernel's weights are float32 in any case.
         chunk C: a query at position p sees keys from floor(p / C) C on only.  head_scale, sink: float32 [H], a factor on
-        every head's scores and a score without key or value in every head's softmax."""
+        every head's scores and a score without key or value in every head's softmax.  keep: the first keep positions are
+        seen beside the window; pin: the rows of the cache in front of its ring that hold them (`CacheSite.pinned`)."""
         self._dev(q, k, v, cu_rows, head_scale, sink)
         self._head_vectors("attention_prefill", H, chunk, head_scale, sink)
         m = q.shape[0]
@@ -973,7 +1065,7 @@ class HipOps:
             self._call(lib, "tp_attn_prefill", q.data_ptr(), qs, k.data_ptr(), ks, v.data_ptr(), vs,
                        m, H, KV, cu_rows.data_ptr(), n_seq, int(max_count), ptr(new_len), ptr(table), table_w,
                        ptr(k_pool), ptr(v_pool), page, rows_cap,
-                       float(scale), float(softcap), int(window), int(chunk), ptr(head_scale), ptr(sink), out.data_ptr(), int(shape),
+                       float(scale), float(softcap), int(window), int(chunk), ptr(head_scale), ptr(sink), int(keep), int(pin), out.data_ptr(), int(shape),
                        self._stream())
             return out
         if cached is not None and (row_seq is None or row_pos is None):
@@ -985,7 +1077,7 @@ class HipOps:
         self._call(self.lib, "tp_attn_simple_prefill", q.data_ptr(), qs, k.data_ptr(), ks, v.data_ptr(), vs, _code(q.dtype),
                    m, H, KV, hd, cu_rows.data_ptr(), row_seq.data_ptr(), row_pos.data_ptr(), ptr(new_len), ptr(table), table_w,
                    ptr(k_pool), ptr(v_pool), page, rows_cap, float(scale), float(softcap),
-                   int(window), int(chunk), ptr(head_scale), ptr(sink), out.data_ptr(), self._stream())
+                   int(window), int(chunk), ptr(head_scale), ptr(sink), int(keep), int(pin) if cached is not None else 0, out.data_ptr(), self._stream())
         return out
 
     def _head_vectors(self, what, H, chunk, head_scale, sink):
@@ -1017,13 +1109,14 @@ class HipOps:
             raise KernelError(f"{what}: the page table must be contiguous int32 [sequences, pages]")
 
     def attention_decode(self, q, H, KV, hd, new_len, table, k_pool, v_pool, rows_cap, scale, softcap, window,
-                         out_dtype, max_keys=None, splits=None, head_groups=None, chunk=0, head_scale=None, sink=None):
+                         out_dtype, max_keys=None, splits=None, head_groups=None, chunk=0, head_scale=None, sink=None,
+                         keep=0, pin=0):
         """head_groups: cut the query heads into that many groups (a multiple of KV), each read the pool head
         `group % KV` by a block of its own: for caches whose one kv head serves many heads, where one block would
         otherwise form all their weighted sums.  The plain kernel takes any grouping as it is.
-        chunk, head_scale, sink: as in `attention_prefill`."""
+        chunk, head_scale, sink, keep, pin: as in `attention_prefill`."""
         self._dev(q, new_len, table, k_pool, v_pool, head_scale, sink)
-        per_head = self._head_vectors("attention_decode", H, chunk, head_scale, sink)
+        per_head = self._head_vectors("attention_decode", H, chunk, head_scale, sink) or keep > 0
         n = q.shape[0]
         qs = self._rows(q, "attention q")
         if q.shape[1] != H * hd:
@@ -1049,13 +1142,13 @@ class HipOps:
             self._call(lib, "tp_attn_decode", q.data_ptr(), qs, n, H, KV, new_len.data_ptr(), table.data_ptr(),
                        table.shape[1], k_pool.data_ptr(), v_pool.data_ptr(), k_pool.shape[2], rows_cap, float(scale),
                        float(softcap), int(window), int(chunk), head_scale.data_ptr() if head_scale is not None else None,
-                       sink.data_ptr() if sink is not None else None, out.data_ptr(), ws.data_ptr() if ws is not None else None, nsplit,
+                       sink.data_ptr() if sink is not None else None, int(keep), int(pin), out.data_ptr(), ws.data_ptr() if ws is not None else None, nsplit,
                        self._stream())
             return out
         self._call(self.lib, "tp_attn_simple_decode", q.data_ptr(), qs, _code(q.dtype), n, H, KV, hd, new_len.data_ptr(),
                    table.data_ptr(), table.shape[1], k_pool.data_ptr(), v_pool.data_ptr(), k_pool.shape[2], rows_cap,
                    float(scale), float(softcap), int(window), int(chunk), head_scale.data_ptr() if head_scale is not None else None,
-                   sink.data_ptr() if sink is not None else None, out.data_ptr(), self._stream())
+                   sink.data_ptr() if sink is not None else None, int(keep), int(pin), out.data_ptr(), self._stream())
         return out
 
     def fuses_decode_step(self, dtype, H, KV, hd, k_pool):
@@ -1064,10 +1157,12 @@ class HipOps:
         return self._fast_attention(dtype, H, KV, hd) and page >= 16 and page & (page - 1) == 0
 
     def attention_decode_step(self, qkv, H, KV, hd, inv_freq, rotary_dim, new_len, table, k_pool, v_pool, rows_cap,
-                              scale, softcap, window, out_dtype, max_keys=None, write_kv=True, splits=None):
+                              scale, softcap, window, out_dtype, max_keys=None, write_kv=True, splits=None, sink=None, keep=0, pin=0):
         """A decode step's rotation, cache write and attention in one launch.  qkv: each sequence's projections
         [queries | keys | values] (queries only when write_kv is false), a bf16 tensor or what
-        `linear(..., defer=True)` returned; sequence i's token has position new_len[i] - 1."""
+        `linear(..., defer=True)` returned; sequence i's token has position new_len[i] - 1.  sink, keep, pin: as in `attention_prefill`."""
+        self._head_vectors("attention_decode_step", H, 0, None, sink)
+        self._dev(sink)
         split = isinstance(qkv, SplitRows)
         rows = qkv.slices if split else qkv
         self._dev(rows, inv_freq, new_len, table, k_pool, v_pool)
@@ -1097,8 +1192,8 @@ class HipOps:
         self._call(lib, "tp_attn_decode_fused", rows.data_ptr(), _code(rows.dtype), n_slices, slice_stride, row_stride,
                    inv_freq.data_ptr() if rotary_dim else None, int(rotary_dim), 1 if write_kv else 0,
                    n, H, KV, new_len.data_ptr(), table.data_ptr(), table.shape[1], k_pool.data_ptr(), v_pool.data_ptr(),
-                   k_pool.shape[2], rows_cap, float(scale), float(softcap), int(window), out.data_ptr(),
-                   ws.data_ptr() if ws is not None else None, nsplit, self._stream())
+                   k_pool.shape[2], rows_cap, float(scale), float(softcap), int(window), sink.data_ptr() if sink is not None else None,
+                   int(keep), int(pin), out.data_ptr(), ws.data_ptr() if ws is not None else None, nsplit, self._stream())
         return out
 
     # ---- token choice -------------------------------------------------------------------------------------

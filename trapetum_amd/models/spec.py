@@ -15,7 +15,7 @@ PartRef = Tuple[str, dict]          # (registered name, constructor parameters)
 class TensorSpec:
     """One tensor a part needs: its shape and how a random model fills it."""
     shape: tuple
-    init: str = "matrix"            # "matrix", "norm", "embedding": which sigma; "gain": one plus "norm"; "talk": unit matrix plus noise; "zeros"; "ones"
+    init: str = "matrix"            # "matrix", "norm", "embedding": which sigma; "gain": one plus "norm"; "conv": taps of a convolution over time; "talk": unit matrix plus noise; "zeros"; "ones"
     dtype: str = "float"            # "float": kept as stored (bf16, or fp32 if stored so); "int": int32 table
     free: tuple = ()                # dimensions whose size the checkpoint gives (no configuration key names it): `shape` there
                                     # holds what a random model takes, and the part reads the real size when it binds
@@ -38,9 +38,12 @@ class LayerSpec:
 @dataclasses.dataclass
 class ScheduleEntry:
     """One run of a layer.  `cache_of` names an earlier entry whose cache this run reads
-    instead of keeping one of its own."""
+    instead of keeping one of its own.  `before`: a registered stream_add, what the model adds to the
+    stream before this run, with the checkpoint prefix of its tensors."""
     layer: int
     cache_of: Optional[int] = None
+    before: Optional[PartRef] = None
+    before_prefix: str = ""
 
 
 @dataclasses.dataclass

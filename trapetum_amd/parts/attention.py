@@ -43,6 +43,12 @@ product's float32 sums, one rounding), `ops.pool_write` (the block means go to a
 one row per P tokens; an unfinished block's sums wait in a float32 state), `ops.attention_pooled` and
 `ops.talk_mix`.  The cache's ring keeps the window only; the step's rows are cached after the attention in every
 kind of step, so one sequence of launches serves prompts, portions of prompts and decode steps.
+
+And three more: `conv` taps of a short causal convolution over time on every channel of the projected queries, keys and
+values (y_t = sum_j w[:, j] u_(t - taps + 1 + j), zeros before the sequence; the last taps - 1 projected rows are a
+state), before the rotation and the cache; `keep_first` F: beside the window the first F positions of the sequence stay
+visible, and the cache keeps them in rows in front of its ring; and a `sink` given as a number, the same score for
+every head (0: softmax with one added to its denominator).
 """
 from ..cache.store import TokenSpec
 from ..models.spec import TensorSpec
@@ -56,17 +62,19 @@ class Attention(Mixer):
                  precise_weights=False,
                  tensors=("q_proj.weight", "k_proj.weight", "v_proj.weight", "o_proj.weight", "g_proj.weight"),
                  bias_suffix=None, chunk=None, head_temperature=None, sink=None, value_rotation=None,
-                 unit_norm_eps=None, pool=None, talk=None):
+                 unit_norm_eps=None, pool=None, talk=None, conv=None, conv_suffix=".conv", keep_first=0):
         """value_dim: elements of a value head when they differ from a key's head_dim.  output_gate: the heads' outputs
         are multiplied by sigmoid(W_g x) before the output projection.  own_kv False: the layer has no key and value
         projections; its schedule entry names the run whose cache it reads.  precise_weights: the softmax weights meet
         the values with 16 bits of mantissa or more in every kernel (the kernel of many queries rounds them to bfloat16
         otherwise; a decode step's are float32 anyway).  tensors: local names of W_q, W_k, W_v, W_o (and W_g).
         bias_suffix: q, k and v have biases, named like their matrices with this suffix.  chunk: positions per chunk.
-        head_temperature, sink: local names of float vectors [heads].  value_rotation: the base theta of the values'
+        head_temperature, sink: local names of float vectors [heads]; a sink may also be a number, the same for all heads.  value_rotation: the base theta of the values'
         rotation by their position.  unit_norm_eps: the eps of the norm without gain on every query and key head (None:
         no such norm).  pool: positions per pooled block before the window.  talk: local name of the matrix
-        [heads, heads] that mixes the heads' softmax weights."""
+        [heads, heads] that mixes the heads' softmax weights.  conv: taps of the convolutions over time on q, k and v, named
+        like their matrices with conv_suffix (None: none).  keep_first: positions at a sequence's start that stay visible
+        beside the window."""
         if num_heads % num_kv_heads:
             raise ValueError(f"{num_heads} query heads are no multiple of {num_kv_heads} kv heads")
         self.hidden_size = hidden_size
@@ -90,12 +98,14 @@ class Attention(Mixer):
             raise ValueError(f"rotary_dim {self.position.rotary_dim} exceeds head_dim {head_dim}")
         self.bias_suffix = bias_suffix
         self.chunk = int(chunk) if chunk else 0
-        self.temperature_name, self.sink_name = head_temperature, sink
+        self.temperature_name = head_temperature
+        self.sink_name, self.sink_value = (sink, None) if isinstance(sink, str) or sink is None else (None, float(sink))
+        has_sink = sink is not None
         self.value_position = None
         if value_rotation is not None:
             self.value_position = build_part("position", ("rope", {"rotary_dim": self.value_dim, "theta": value_rotation}))
         self.output_dtype = None         # a mixer that holds this one may ask for its last product in another dtype
-        self.per_head = bool(self.chunk or head_temperature or sink)
+        self.per_head = bool(self.chunk or head_temperature or has_sink)
         if (self.per_head or value_rotation is not None) and (self.output_gate or not self.own_kv):
             raise ValueError("chunks, temperatures, sinks and rotated values go with an ungated attention on its own cache")
         self.unit_norm_eps = None if unit_norm_eps is None else float(unit_norm_eps)
@@ -105,6 +115,12 @@ class Attention(Mixer):
         if self.pooled and (self.per_head or value_rotation is not None or not self.own_kv):
             raise ValueError("unit norms, pooled blocks and talking heads go with an attention on its own cache, without chunks, "
                              "temperatures, sinks or rotated values")
+        self.taps, self.conv_suffix = (int(conv) if conv else 0), conv_suffix
+        self.keep_first = int(keep_first)
+        if self.keep_first and (not self.window or self.chunk or self.pooled or not self.own_kv):
+            raise ValueError("first positions are kept beside a window, by an attention on its own cache, without chunks or pooled blocks")
+        if self.taps and (self.pooled or not self.own_kv or bias_suffix):
+            raise ValueError("convolutions go with an attention on its own cache, without biases, unit norms, pooled blocks or talking heads")
         if self.pool and not self.window:
             raise ValueError("pooled blocks stand before a window: the layer needs one")
 
@@ -125,6 +141,9 @@ class Attention(Mixer):
         if self.bias_suffix:
             for s in ("q", "k", "v") if self.own_kv else ("q",):
                 specs[n[s] + self.bias_suffix] = TensorSpec((specs[n[s]].shape[0],), init="norm")
+        if self.taps:
+            for s in ("q", "k", "v"):
+                specs[n[s] + self.conv_suffix] = TensorSpec((specs[n[s]].shape[0], self.taps), init="conv")
         if self.temperature_name:
             specs[self.temperature_name] = TensorSpec((self.num_heads,), init="gain")
         if self.sink_name:
@@ -135,7 +154,7 @@ class Attention(Mixer):
 
     def cache_spec(self):
         per_token = (self.num_kv_heads, self.row)
-        return TokenSpec.of(self.reach or None, k=per_token, v=per_token)
+        return TokenSpec.of(self.reach or None, keep_first=self.keep_first, k=per_token, v=per_token)
 
     def token_specs(self):
         """The pooled blocks: one mean key and value per `pool` tokens, of all tokens."""
@@ -145,11 +164,14 @@ class Attention(Mixer):
         return {"blocks": TokenSpec.of(None, every=self.pool, k=per_block, v=per_block)}
 
     def state_specs(self):
-        """The sums of the keys and of the values of the block that is not finished yet."""
-        if not self.pool:
-            return {}
+        """The sums of the keys and of the values of the block that is not finished yet; the convolutions' last inputs."""
         from ..cache.store import StateSpec
-        return {"block_sums": StateSpec((2, self.num_kv_heads * self.row), "float32")}
+        specs = {}
+        if self.pool:
+            specs["block_sums"] = StateSpec((2, self.num_kv_heads * self.row), "float32")
+        if self.taps > 1:
+            specs["conv"] = StateSpec((self.taps - 1, (self.num_heads + 2 * self.num_kv_heads) * self.row), "float32")
+        return specs
 
     def _heads(self, w, heads, size, turned=False):
         """[heads * size, d] -> [heads * row, d]: zero rows fill a head up to `row`.  turned: a rotation of neighbouring
@@ -188,6 +210,13 @@ class Attention(Mixer):
                                     for s, heads, size, t in sides]).float().contiguous()
         self.temperature = tensors[self.temperature_name].float().contiguous() if self.temperature_name else None
         self.sink = tensors[self.sink_name].float().contiguous() if self.sink_name else None
+        if self.sink_value is not None:
+            self.sink = torch.full((H,), self.sink_value, dtype=torch.float32, device=rt.device)
+        self.conv_t = None
+        if self.taps:                                        # [taps, heads x row], the filled-up rows of a head with taps of zero
+            sides = (("q", H, self.head_dim, True), ("k", KV, self.head_dim, True), ("v", KV, self.value_dim, False))
+            self.conv_t = torch.cat([self._heads(tensors[n[s] + self.conv_suffix], heads, size, turned=t)
+                                     for s, heads, size, t in sides]).float().t().contiguous()
         self.talk = None
         if self.pooled:            # heads that do not talk are mixed by the unit matrix, in the same launch that rounds
             self.talk = (tensors[self.talk_name].float() if self.talk_name else torch.eye(H, device=self.w_o.device)).contiguous()
@@ -207,6 +236,11 @@ class Attention(Mixer):
         """Turn every head of `rows` by its position, over the values' elements, in place."""
         ctx.ops.rope_kv_write(rows, None, None, heads, 0, self.row, freq, self.value_dim, ctx.row_seq, ctx.row_pos, ctx.new_len,
                               None, None, None, 0, write=False)
+
+    def _convolve(self, ctx, qkv):
+        """The projected rows of a step through the convolutions over time; the state takes the last of them."""
+        return ctx.ops.conv_act(qkv, self.conv_t, None, self.state(ctx, "conv") if self.taps > 1 else None, ctx.slot_ids, ctx.cu_rows,
+                                ctx.row_seq, one_row_each=ctx.mode == "decode")
 
     def _forward_pooled(self, ctx, x, site):
         import torch
@@ -246,6 +280,8 @@ class Attention(Mixer):
         H, KV, hd = self.num_heads, self.num_kv_heads, self.row
         Q, KVD = H * hd, KV * hd
         owns_cache = ctx.cache_owner == ctx.entry
+        if self.taps and not owns_cache:
+            raise ValueError("an attention with convolutions runs on its own cache")
         if owns_cache and not self.own_kv:
             raise ValueError("an attention without key and value projections must read another run's cache")
         w_in = self.w_qkv if owns_cache else self.w_qkv[:Q]          # a run on another run's cache projects its queries only
@@ -258,37 +294,48 @@ class Attention(Mixer):
         rows_cap = site.rows_cap or 0
         bias = None if self.b_qkv is None else (self.b_qkv if owns_cache else self.b_qkv[:Q])
         more = dict(chunk=self.chunk, head_scale=self.temperature, sink=self.sink) if self.per_head else {}
-        if ctx.mode == "decode" and bias is None and not self.per_head and self.value_freq is None and ops.fuses_decode_step(ctx.dtype, H, KV, hd, k_pool):
+        kept = dict(keep=self.keep_first, pin=site.pinned) if self.keep_first else {}
+        pin = dict(pin=site.pinned) if site.pinned else {}
+        fuses = bias is None and not self.chunk and self.temperature is None and self.value_freq is None
+        fuses = fuses and ctx.mode == "decode" and ops.fuses_decode_step(ctx.dtype, H, KV, hd, k_pool)
+        if fuses:
             # one launch rotates, writes the cache and attends; the projections may stay in K slices until then
-            qkv = ops.linear(x, w_in, ctx.dtype, defer=True)
+            if self.taps:
+                qkv = self._convolve(ctx, ops.linear(x, w_in, ctx.dtype))
+            else:
+                qkv = ops.linear(x, w_in, ctx.dtype, defer=True)
             out = ops.attention_decode_step(qkv, H, KV, hd, self.inv_freq, self.position.rotary_dim, ctx.new_len,
                                             table, k_pool, v_pool, rows_cap, self.query_scale, self.softcap,
-                                            self.window, ctx.dtype, max_keys=ctx.max_rows_visible(site), write_kv=owns_cache)
+                                            self.window, ctx.dtype, max_keys=ctx.max_rows_visible(site), write_kv=owns_cache,
+                                            **(dict(sink=self.sink) if self.sink is not None else {}), **kept)
             return self._project_out(ctx, x, out)
         qkv = ops.linear(x, w_in, ctx.dtype, bias=bias) if bias is not None else ops.linear(x, w_in, ctx.dtype)
+        if self.taps:
+            qkv = self._convolve(ctx, qkv)
         if owns_cache:
             q, k, v = qkv[:, :Q], qkv[:, Q:Q + KVD], qkv[:, Q + KVD:]
         else:
             q, k, v = qkv, None, None
         if self.value_freq is not None:
             self._turn(ctx, v, KV, self.value_freq)
-        if ctx.mode == "decode":
-            ops.rope_kv_write(q, k, v, H, KV, hd, self.inv_freq, self.position.rotary_dim,
-                              ctx.row_seq, ctx.row_pos, ctx.new_len, table, k_pool, v_pool, rows_cap)
-            out = ops.attention_decode(q, H, KV, hd, ctx.new_len, table, k_pool, v_pool, rows_cap,
-                                       self.query_scale, self.softcap, self.window, ctx.dtype,
-                                       max_keys=ctx.max_rows_visible(site), **more)
-            if self.value_back is not None:
-                self._turn(ctx, out, H, self.value_back)
-            return self._project_out(ctx, x, out)
         # Sequences that go on by several tokens (or some start while others go on) see cached positions and the
         # step's own rows.  The attention reads the cached ones where they lie, as earlier steps left them, and the
         # step's rows from the step; only then are the step's rows cached: in a window's ring without a row to spare
         # they take the places of positions that the step's earlier queries still see.
         extend = ctx.mode == "extend"
-        ops.rope_kv_write(q, k, v, H, KV, hd, self.inv_freq, self.position.rotary_dim,
-                          ctx.row_seq, ctx.row_pos, ctx.new_len, table, k_pool, v_pool, rows_cap,
-                          write=not extend)
+        if self.position.rotary_dim or not owns_cache:
+            ops.rope_kv_write(q, k, v, H, KV, hd, self.inv_freq, self.position.rotary_dim,
+                              ctx.row_seq, ctx.row_pos, ctx.new_len, table, k_pool, v_pool, rows_cap,
+                              write=not extend, **pin)
+        elif not extend:                                     # nothing turns: the rows are cached as they are
+            ops.kv_write(k, v, KV, hd, ctx.row_seq, ctx.row_pos, ctx.new_len, table, k_pool, v_pool, rows_cap, **pin)
+        if ctx.mode == "decode":
+            out = ops.attention_decode(q, H, KV, hd, ctx.new_len, table, k_pool, v_pool, rows_cap,
+                                       self.query_scale, self.softcap, self.window, ctx.dtype,
+                                       max_keys=ctx.max_rows_visible(site), **more, **kept)
+            if self.value_back is not None:
+                self._turn(ctx, out, H, self.value_back)
+            return self._project_out(ctx, x, out)
         if owns_cache:
             ctx.offer_step_rows(k=k, v=v)
         else:
@@ -298,12 +345,12 @@ class Attention(Mixer):
                                     self.query_scale, self.softcap, self.window, ctx.dtype,
                                     row_seq=ctx.row_seq, row_pos=ctx.row_pos,
                                     cached=(ctx.new_len, table, k_pool, v_pool, rows_cap) if extend else None,
-                                    wide_weights=self.precise_weights, **more)
+                                    wide_weights=self.precise_weights, **more, **kept)
         if self.value_back is not None:
             self._turn(ctx, out, H, self.value_back)
         if extend and owns_cache:
             row_seq, row_pos, new_len = ctx.row_seq, ctx.row_pos, ctx.new_len
-            ctx.after_readers(lambda: ops.kv_write(k, v, KV, hd, row_seq, row_pos, new_len, table, k_pool, v_pool, rows_cap))
+            ctx.after_readers(lambda: ops.kv_write(k, v, KV, hd, row_seq, row_pos, new_len, table, k_pool, v_pool, rows_cap, **pin))
         return self._project_out(ctx, x, out)
 
 

@@ -24,6 +24,9 @@ step (`forward`).  Interfaces:
                with tensors of their own that the block builds (a convolution in front of a sub-layer).
   Conv         state_spec() -> StateSpec | None;  forward(ctx, stream, state) -> rows: what a sub-layer reads
                of the fp32 stream when a short causal convolution over time stands in front of it.
+  StreamAdd    operands(ctx) -> (vec, origin): what a model adds to the stream before a run of a layer, a float32 vector
+               [hidden] for every row and float32 rows [M, hidden] (either may be None); `needs_origin` asks the engine
+               to keep the embedding's rows for the step (`ctx.origin`).
   Embedding    forward(ctx, tokens) -> fp32 stream;  Head  forward(ctx, rows) -> fp32 logits.
 
 `ctx` is the step's StepContext: batch geometry on the device, the kernels
@@ -118,6 +121,13 @@ class Conv(Part):
         return None
 
     def forward(self, ctx, stream, state):
+        raise NotImplementedError
+
+
+class StreamAdd(Part):
+    needs_origin = False
+
+    def operands(self, ctx):
         raise NotImplementedError
 
 

@@ -9,12 +9,14 @@ pre_norm  x += mixer(pre_mixer_norm(x));  x += ff(pre_ff_norm(x)); the feed-forw
 post_norm x += post_mixer_norm(mixer(c1(x)));  x += post_ff_norm(ff(c2(x))): no norm in front of a sub-layer; c1
           and c2 are what it reads of the stream, the stream itself or (input_conv) the stream through a short
           causal convolution whose last rows are a state of the sequence.  The feed-forward may be absent.
+parallel  x += mixer(n(x)) + ff(n(x)): one norm, and both sub-layers read its output; the feed-forward may be absent.
 
 The stream is fp32 and the sum is formed in fp32 (the reference adds in fp32 and
 stores fp16: runtime/cuda/codebook_gemv.cu:539-542).  Where a norm of a sub-layer's
 output is followed by the add and by the next norm, one kernel does all three; that
 includes the first norm of the block that runs next (`next_norm`), whose result the
-next block receives as `normed`.
+next block receives as `normed`.  What a model adds to the stream between two layers (`NormAfterAdd`) is added in
+that kernel too.
 """
 from ..registry import register_part
 from .base import Block
@@ -23,6 +25,11 @@ from .base import Block
 def add_then_norm(ctx, stream, rows, post, nxt):
     """stream += post(rows) (or rows); returns nxt(stream) (or None).  One kernel when both norms
     expose an RMS gain, else the norms' own forward around a plain add."""
+    if isinstance(nxt, NormAfterAdd):
+        if post is None:
+            return join_then_norm(ctx, stream, rows, None, nxt)
+        add_then_norm(ctx, stream, rows, post, None)
+        return nxt.forward(ctx, stream)
     fusable = all(n is None or n.gain is not None for n in (post, nxt))
     groups = {getattr(n, "groups", 1) for n in (post, nxt) if n is not None}      # one kernel cuts both norms alike
     if fusable and len(groups) <= 1:
@@ -36,6 +43,31 @@ def add_then_norm(ctx, stream, rows, post, nxt):
         rows = post.forward(ctx, rows)
     ctx.ops.add_rms_norm(stream, rows, None, 0.0, None, 0.0, ctx.dtype)
     return nxt.forward(ctx, stream, getattr(nxt, "reader_dtype", None)) if nxt is not None else None
+
+
+class NormAfterAdd:
+    """A block's first norm with what the model adds to the stream before that block: `added` is a StreamAdd part."""
+
+    def __init__(self, norm, added):
+        self.norm, self.added = norm, added                # norm None: the add alone
+        self.gain = norm.gain if norm is not None else None
+
+    def forward(self, ctx, stream, out_dtype=None):
+        return join_then_norm(ctx, stream, None, None, self)
+
+
+def join_then_norm(ctx, stream, a, b, nxt):
+    """stream += a + b (either may be None) and what `nxt` adds before its norm; returns its norm of the stream (or None)."""
+    vec = origin = None
+    norm = nxt
+    if isinstance(nxt, NormAfterAdd):
+        norm = nxt.norm
+        vec, origin = nxt.added.operands(ctx)
+    plain = norm is None or (norm.gain is not None and getattr(norm, "groups", 1) == 1)
+    dtype = getattr(norm, "reader_dtype", None) or ctx.dtype
+    gain, eps = (norm.gain, norm.eps) if plain and norm is not None else (None, 0.0)
+    out = ctx.ops.join_rms_norm(stream, a, b, gain, eps, dtype, vec=vec, origin=origin)
+    return out if plain else norm.forward(ctx, stream, getattr(norm, "reader_dtype", None))
 
 
 class SandwichBlock(Block):
@@ -182,6 +214,32 @@ class PostNormBlock(Block):
         return stream, normed_next
 
 
+class ParallelBlock(Block):
+    def __init__(self, mixer, feed_forward, make_norm):
+        super().__init__(mixer, feed_forward, make_norm)
+
+    @classmethod
+    def norm_sites(cls):
+        return ("pre_norm",)
+
+    def entry_norm(self):
+        return self.norms["pre_norm"]
+
+    def forward(self, ctx, stream, site, normed=None, next_norm=None):
+        x = normed if normed is not None else self.norms["pre_norm"].forward(ctx, stream)
+        ctx.dump("mixer_in", x)
+        a = self.mixer.forward(ctx, x, site)
+        ctx.dump("mixer_out", a)
+        m = None
+        if self.feed_forward is not None:
+            m = self.feed_forward.forward(ctx, x)
+            ctx.dump("ff_out", m)
+        normed_next = join_then_norm(ctx, stream, a, m, next_norm)       # with what the model adds before the next layer
+        ctx.dump("layer_out", stream)
+        return stream, normed_next
+
+
+register_part("block", "parallel", ParallelBlock)
 register_part("block", "sandwich", SandwichBlock)
 register_part("block", "post_norm", PostNormBlock)
 register_part("block", "pre_norm", PreNormBlock)

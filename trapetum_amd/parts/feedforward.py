@@ -92,5 +92,33 @@ class BiasedMLP(FeedForward):
         return ctx.ops.linear(act, self.w_down, torch.float32, bias=self.b_down)
 
 
+class PlainMLP(FeedForward):
+    """down(act(up x)): one product up, one down, no gate and no biases; the activation is applied to the first product's
+    float32 sums in its epilogue."""
+
+    def __init__(self, hidden_size, intermediate_size, activation="relu2", tensors=("up", "down")):
+        """activation: relu2, max(z, 0)^2."""
+        self.hidden_size, self.intermediate_size = int(hidden_size), int(intermediate_size)
+        self.activation = activation
+        self.names = tuple(tensors)
+
+    def tensor_specs(self):
+        d, i, (up, dn) = self.hidden_size, self.intermediate_size, self.names
+        return {up: TensorSpec((i, d)), dn: TensorSpec((d, i))}
+
+    def bind(self, tensors, rt):
+        self.rt = rt
+        up, dn = self.names
+        self.w_up, self.w_down = rt.matrix(tensors[up]), rt.matrix(tensors[dn])
+
+    def forward(self, ctx, x, out=None):
+        """out: as in GatedMLP."""
+        act = ctx.ops.linear_act(x, self.w_up, ctx.dtype, self.activation)
+        if out is not None:
+            return ctx.ops.linear(act, self.w_down, out.dtype, out=out)
+        return ctx.ops.linear(act, self.w_down, ctx.dtype, defer=True)
+
+
+register_part("feed_forward", "plain_mlp", PlainMLP)
 register_part("feed_forward", "gated_mlp", GatedMLP)
 register_part("feed_forward", "biased_mlp", BiasedMLP)
