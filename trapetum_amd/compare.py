@@ -1,7 +1,7 @@
-"""Two designs side by side at equal layer sizes: Golepel or Lutovik next to Gemma-2, Besulix or Vogunex next to Lutovik,
-random weights, one MI355X.
+"""Two designs side by side at equal layer sizes: Golepel or Lutovik next to Gemma-2, Besulix, Vogunex or Solulix next to
+Lutovik, random weights, one MI355X.
 
-    python bench.py --compare golepel|lutovik|besulix|vogunex [--sizes 2b|9b] [--layers L] [--steps K] [--warmup W]
+    python bench.py --compare golepel|lutovik|besulix|vogunex|solulix [--sizes 2b|9b] [--layers L] [--steps K] [--warmup W]
 
 For each design: tokens per second of a prefill of 2,048 tokens and of the generation loop's decode steps at batch 8
 and 1 (HIP graphs, greedy choice on the device), and the time of the kernels a step spends its time in, one by one at
@@ -27,6 +27,12 @@ feed-forward of Gemma's width, the second an attention through a latent (16 head
 of 192, a query latent of 768, a window of 1,024, gated heads), the third runs on the first one's weights, the fourth is
 a state-space layer of Lutovik's sizes; the second and fourth have 8 experts of half the dense width, 2 chosen, and a
 gated shared expert of a quarter of it (`time_vogunex_kernels`).
+The Solulix sizes: the same width and vocabulary and as many runs of a layer (four layers in the middle run twice); of every
+four layers the first and third are attention layers (Gemma-2's heads; a window of 1,024 positions beside the first 64,
+4 taps), the second and fourth gated-delta layers (heads of 128 key and 128 value elements, the value heads filling the
+width and half as many kv heads, 4 taps); the second and third have 8 squared-ReLU experts of half the dense width and 2
+identity outputs, 2 chosen, and a shared expert of a quarter of it, the others a dense feed-forward
+(`time_solulix_kernels`).
 """
 import json
 import sys
@@ -115,6 +121,142 @@ def vogunex_config(which, layers=0):
             out.append({"type": "mamba2", "mixer": ssm, "mlp": moe})
     return VogunexConfig.from_dict({"architecture": "Vogunex", "vocab": g["vocab_size"], "width": D, "embedding": {"scale": D ** 0.5},
                                     "norm": {"eps": 1e-6}, "layers": out})
+
+
+def solulix_config(which, layers=0):
+    from .config import SolulixConfig
+    g = dict(SIZES, **OTHER_SIZES[which])
+    runs = layers or g["num_hidden_layers"]
+    looped = 4 if runs >= 12 else 0
+    n = runs - looped
+    D, I, H, KV, hd = g["hidden_size"], g["intermediate_size"], g["num_attention_heads"], g["num_key_value_heads"], g["head_dim"]
+    att = {"heads": H, "kv_heads": KV, "dim": hd, "vdim": hd, "conv": 4, "scale": hd ** -0.5, "mask": {"size": 1024, "keep_first": 64}}
+    delta = {"heads": D // 128, "kv_heads": D // 256, "dim": 128, "vdim": 128, "conv": 4}
+    moe = {"kind": "moe", "expert": {"ff": I // 2}, "router": {"experts": 8, "identity": 2, "scale": 1.5, "top": 2}, "shared": {"ff": I // 4}}
+    dense = {"kind": "dense", "ff": I}
+    out = [{"type": "delta" if i % 2 else "attention", "mixer": delta if i % 2 else att, "mlp": moe if i % 4 in (1, 2) else dense} for i in range(n)]
+    d = {"architecture": "Solulix", "vocab": g["vocab_size"], "width": D, "norm": {"eps": 1e-6}, "layers": out}
+    if looped:
+        start = (n // 2) // 4 * 4
+        d["loop"] = {"start": start, "stop": start + looped, "times": 2}
+    return SolulixConfig.from_dict(d)
+
+
+def time_solulix_kernels(engine, cfg, batch, context, prefill_tokens):
+    """Microseconds of Solulix's kernels at a decode step of `batch` sequences over `context` cached tokens and at a
+    prefill of `prefill_tokens`, each called once per layer on that layer's own weights, replayed from a HIP graph.
+    Products are priced by their weights' bytes (decode) or their flops against the bf16 matrix peak (prefill); the delta
+    scan by its state's bytes (decode) or by the flops of its rows taken one by one, 7 key_dim value_dim a head, against the
+    float32 peak (prefill); the attention by the keys and values a query sees (decode) or by its flops (prefill)."""
+    import torch
+    from .engine.batch import StepContext
+    model, ops, dev = engine.model, engine.model.rt.ops, engine.model.rt.device
+    bf, f32 = torch.bfloat16, torch.float32
+    blocks = [l.block for l in model.layers]
+    att = [b for b in blocks if hasattr(b.mixer, "w_qkv")]
+    rec = [b for b in blocks if hasattr(b.mixer, "a_log")]
+    moe = [b for b in blocks if hasattr(b.feed_forward, "w_router")]
+    dense = [b for b in blocks if hasattr(b.feed_forward, "w_gate_up") and not hasattr(b.feed_forward, "w_router")]
+    D = cfg.hidden_size
+    out = {}
+    timed = _timer(dev, out)
+    cache = engine.cache
+    entry = lambda group: next(i for i, e in enumerate(model.schedule) if model.layers[e.layer].block is group[0])
+    elems = lambda w: float(w.numel())
+    for rows, tag in ((batch, f"decode_b{batch}"), (prefill_tokens, f"prefill_{prefill_tokens}")):
+        decode = rows == batch
+        slots = [cache.acquire() for _ in range(batch if decode else 1)]
+        try:
+            for s in slots:
+                cache.grow(s, context if decode else rows)
+            counts = [1] * batch if decode else [rows]
+            starts = [context - 1] * batch if decode else [0]
+            ctx = StepContext(model.rt, cache, slots, counts, starts, [])
+            x = torch.randn((rows, D), device=dev).to(bf)
+            one = lambda f, **kw: timed(f"{tag}.{kw.pop('name')}", f, **kw)
+            prod = (lambda name, calls, w, m=rows: one(calls, name=name, bytes_each=2.0 * elems(w)) if decode
+                    else one(calls, name=name, flops_each=2.0 * m * elems(w)))
+
+            def conv(name, mixer, u, e, activation):
+                ch = mixer.conv_t.shape[1]
+                state = cache.entry_state(e, "mixer.conv")
+                call = lambda: ops.conv_act(u[:, :ch], mixer.conv_t, None, state, ctx.slot_ids, ctx.cu_rows, ctx.row_seq, activation=activation,
+                                            one_row_each=decode)
+                one([call] * 16, name=name, bytes_each=rows * ch * 4.0 + (rows * (mixer.taps - 1) * ch * 8.0 if decode else 0.0))
+                return call()
+            if att:
+                e = entry(att)
+                a = att[0].mixer
+                H, KV, row, W, F = a.num_heads, a.num_kv_heads, a.row, a.window, a.keep_first
+                site = cache.site(e)
+                table, kp, vp, cap = ctx.page_table(site.group_index), site.tensor("k"), site.tensor("v"), site.rows_cap or 0
+                kept = dict(keep=F, pin=site.pinned)
+                prod("qkv", [(lambda b=b: ops.linear(x, b.mixer.w_qkv, bf)) for b in att], a.w_qkv)
+                qkv = conv("qkv_conv", a, torch.randn((rows, (H + 2 * KV) * row), device=dev).to(bf), e, None)
+                seen = lambda p: min(p + 1, W + min(F, max(0, p + 1 - W)))
+                if decode:
+                    one([lambda: ops.attention_decode_step(qkv, H, KV, row, None, 0, ctx.new_len, table, kp, vp, cap, a.query_scale, 0.0, W, bf,
+                                                           max_keys=ctx.max_rows_visible(site), sink=a.sink, **kept)] * 8,
+                        name=f"attention_{seen(context - 1)}_keys_of_{context}", bytes_each=2.0 * batch * seen(context - 1) * 2 * KV * row)
+                else:
+                    q, k, v = qkv[:, :H * row], qkv[:, H * row:(H + KV) * row], qkv[:, (H + KV) * row:]
+                    one([lambda: ops.kv_write(k, v, KV, row, ctx.row_seq, ctx.row_pos, ctx.new_len, table, kp, vp, cap, pin=site.pinned)] * 16,
+                        name="kv_write", bytes_each=rows * 2 * KV * row * 4.0)
+                    one([lambda: ops.attention_prefill(q, k, v, H, KV, row, ctx.cu_rows, rows, a.query_scale, 0.0, W, bf, wide_weights=True,
+                                                       sink=a.sink, **kept)] * 4,
+                        name=f"attention_window_{W}_and_{F}", flops_each=4.0 * sum(seen(p) for p in range(rows)) * H * row)
+                xa = torch.randn((rows, H * row), device=dev).to(bf)
+                prod("o", [(lambda b=b: ops.linear(xa, b.mixer.w_o, bf, defer=True)) for b in att], a.w_o)
+            if rec:
+                e = entry(rec)
+                mx = rec[0].mixer
+                H, G, dk, dv, ch = mx.num_heads, mx.num_kv_heads, mx.key_dim, mx.value_dim, mx.conv_channels
+                prod("delta_in", [(lambda b=b: ops.linear(x, b.mixer.w_in, bf)) for b in rec], mx.w_in)
+                p = (torch.randn((rows, mx.w_in.shape[0]), device=dev) * 0.7).to(bf)
+                u = conv("delta_conv", mx, p, e, "silu")
+                state = cache.entry_state(e, "mixer.memory")
+                scan = lambda: ops.delta_scan(u[:, :G * dk], u[:, G * dk:2 * G * dk], u[:, 2 * G * dk:], p[:, ch + H * dv:ch + H * dv + H],
+                                              p[:, ch + H * dv + H:ch + H * dv + 2 * H], mx.a_log, mx.dt_bias, state, ctx.slot_ids, ctx.cu_rows,
+                                              ctx.max_count, H, G, dk, dv, dk ** -0.5)
+                if decode:
+                    one([scan] * 8, name="delta_scan", bytes_each=batch * H * dk * dv * 8.0)
+                else:
+                    one([scan] * 4, name="delta_scan", flops_each=7.0 * rows * H * dk * dv, peak=PEAK_FLOPS["float32"])
+                y = torch.randn((rows, H * dv), device=dev)
+                one([lambda: ops.head_norm_gate(y, mx.norm_gain, p[:, ch:ch + H * dv], 1e-6, H, "silu", bf)] * 16, name="head_norm_gate",
+                    bytes_each=rows * H * dv * 8.0)
+                xo = torch.randn((rows, H * dv), device=dev).to(bf)
+                prod("delta_o", [(lambda b=b: ops.linear(xo, b.mixer.w_o, bf, defer=True)) for b in rec], mx.w_o)
+            if dense:
+                ff = dense[0].feed_forward
+                prod("gate_up_silu", [(lambda b=b: ops.gated_linear(x, b.feed_forward.w_gate_up, ff.intermediate_size, "silu", bf)) for b in dense],
+                     ff.w_gate_up[:2 * ff.intermediate_size])
+                xi = torch.randn((rows, ff.intermediate_size), device=dev).to(bf)
+                prod("down", [(lambda b=b: ops.linear(xi, b.feed_forward.w_down, bf, defer=True)) for b in dense], ff.w_down)
+            if moe:
+                ff = moe[0].feed_forward
+                logits = torch.randn((rows, ff.n_experts + ff.identity), device=dev)
+                route = lambda: ops.route_top(logits, ff.top, True, correction=ff.correction, scale=ff.weight_scale)
+                chosen, weights = route()
+                one([route] * 16, name="route_top")
+                used = len({c for c in chosen.reshape(-1).tolist() if c < ff.n_experts})
+                pairs = int((chosen < ff.n_experts).sum())
+                per_expert = float(ff.w_gate_up[0].numel() + ff.w_down[0].numel())
+                calls = [(lambda b=b: ops.expert_ffn(x, chosen, weights, b.feed_forward.w_gate_up, b.feed_forward.w_down, None, 1.0, 0.0, kind="relu2"))
+                         for b in moe]
+                if decode:
+                    one(calls, name=f"experts_{used}_used", bytes_each=2.0 * used * per_expert)
+                else:
+                    one(calls, name="experts", flops_each=2.0 * pairs * per_expert)
+                sh = ff.shared
+                prod("shared_up_relu2", [(lambda b=b: ops.linear_act(x, b.feed_forward.shared.w_up, bf, "relu2")) for b in moe], sh.w_up)
+            stream = torch.randn((rows, D), device=dev)
+            rows_b, g = torch.randn((rows, D), device=dev).to(bf), torch.ones(D, device=dev)
+            one([lambda: ops.join_rms_norm(stream, rows_b, rows_b, g, 1e-6, bf)] * 16, name="join_rms_norm", bytes_each=rows * D * (4 + 4 + 2 + 2 + 2) + 4.0 * D)
+        finally:
+            for s in slots:
+                cache.release(s)
+    return out
 
 
 def time_vogunex_kernels(engine, cfg, batch, context, prefill_tokens):
@@ -748,10 +890,11 @@ def main(args):
     prompt, batch = args.prompt, args.batch
     design = args.compare
     build, time_design = {"golepel": (golepel_config, time_golepel_kernels), "lutovik": (lutovik_config, time_lutovik_kernels),
-                          "besulix": (besulix_config, time_besulix_kernels), "vogunex": (vogunex_config, time_vogunex_kernels)}[design]
+                          "besulix": (besulix_config, time_besulix_kernels), "vogunex": (vogunex_config, time_vogunex_kernels),
+                          "solulix": (solulix_config, time_solulix_kernels)}[design]
     # the design it stands next to: the closest of the others
     beside_lutovik = ("lutovik", lutovik_config, time_lutovik_kernels, "Lutovik")
-    other, build_other, time_other, title = {"besulix": beside_lutovik, "vogunex": beside_lutovik}.get(
+    other, build_other, time_other, title = {"besulix": beside_lutovik, "vogunex": beside_lutovik, "solulix": beside_lutovik}.get(
         design, ("gemma2", gemma_config, time_kernels, "Gemma-2"))
     line = {"metric": f"{design.capitalize()} next to {title} at {which} layer sizes: prefill and decode tok/s", "unit": "tok/s", "n_gpus": 1,
             "steps": steps, "warmup": warmup, "dtype": "bf16", "data": "synthetic: seeded random weights N(0, 0.02) and uniform-random token ids",
@@ -760,7 +903,7 @@ def main(args):
     for name, cfg in ((design, build(which, args.layers)), (other, build_other(which, args.layers))):
         run = Run(cfg, max(batch, 8), most, name)
         pre = run.prefill()
-        d = {"layers": len(cfg.layers) if hasattr(cfg, "layers") else cfg.num_hidden_layers, "weights_GB": round(run.weight_bytes / 1e9, 2),
+        d = {"layers": len(cfg.layers) if hasattr(cfg, "layers") else cfg.num_hidden_layers, "runs": len(run.model.schedule), "weights_GB": round(run.weight_bytes / 1e9, 2),
              f"prefill_{PREFILL_TOKENS}_tok_s": round(PREFILL_TOKENS / pre, 1), f"prefill_{PREFILL_TOKENS}_ms": round(pre * 1e3, 2)}
         for b in (batch, 1):
             dt = run.decode([prompt] * b, steps, warmup)

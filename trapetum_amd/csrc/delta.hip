@@ -29,7 +29,7 @@ struct DeltaArgs {
     const float* a_log; const float* dt_bias;            // [H]
     float* state;                                        // [slots, H, dk, dv]
     const int* slot_ids; const int* cu_rows; float* y;   // y [M, H dv]
-    int H, G, dk, dv; float q_scale;
+    int n_seq, H, G, dk, dv; float q_scale;
     // chunks: for (sequence, chunk) c and head h, at (c H + h): T' and A in three terms of [64][64], four rows of 64 scalars
     // (e^G / |k|, q_scale e^G / |q|, e^(G_C - G) / |k|, e^(G_C)); for kv head j, at (c G + j): K transposed [dkp][64]
     int n_chunks, dkp; bf16_t* ws_mat; float* ws_scal; bf16_t* ws_kt;
@@ -167,37 +167,37 @@ delta_rows_k(DeltaArgs x) {
 // ---- chunks --------------------------------------------------------------------------------------------------------------
 namespace {
 union DFrag { uint4 u; dl_bf16x8 v; bf16_t h[8]; };
-struct Terms { bf16_t t[3]; };
-__device__ __forceinline__ bf16_t dl_bits(float f) { __bf16 b = (__bf16)f; return __builtin_bit_cast(bf16_t, b); }
-__device__ __forceinline__ Terms split(float f) {         // f = the sum of three bfloat16 numbers, to float32's 24 bits
-    Terms r;
-    r.t[0] = dl_bits(f);
-    f -= bf16_to_f32(r.t[0]);
-    r.t[1] = dl_bits(f);
-    f -= bf16_to_f32(r.t[1]);
-    r.t[2] = dl_bits(f);
-    return r;
+typedef __attribute__((__vector_size__(2 * sizeof(float)))) float dl_f32x2;
+typedef __attribute__((__vector_size__(2 * sizeof(__bf16)))) __bf16 dl_bf16x2;
+// a and b as sums of three bfloat16 numbers, to float32's 24 bits: word n holds their nth terms
+__device__ __forceinline__ void split_pair(float a, float b, uint32_t (&word)[3]) {
+#pragma unroll
+    for (int n = 0; n < 3; n++) {
+        word[n] = __builtin_bit_cast(uint32_t, __builtin_convertvector((dl_f32x2){a, b}, dl_bf16x2));
+        a -= __uint_as_float(word[n] << 16);
+        b -= __uint_as_float(word[n] & 0xffff0000u);
+    }
 }
 // four neighbouring elements of a row of terms, term n at dst + n * apart
 __device__ __forceinline__ void put4(bf16_t* dst, int apart, float f0, float f1, float f2, float f3) {
-    const Terms a = split(f0), b = split(f1), c = split(f2), d = split(f3);
+    uint32_t lo[3], hi[3];
+    split_pair(f0, f1, lo);
+    split_pair(f2, f3, hi);
 #pragma unroll
-    for (int n = 0; n < 3; n++) {
-        uint2 pk;
-        pk.x = (uint32_t)a.t[n] | ((uint32_t)b.t[n] << 16);
-        pk.y = (uint32_t)c.t[n] | ((uint32_t)d.t[n] << 16);
-        *reinterpret_cast<uint2*>(dst + n * apart) = pk;
-    }
+    for (int n = 0; n < 3; n++) *reinterpret_cast<uint2*>(dst + n * apart) = make_uint2(lo[n], hi[n]);
 }
 __device__ __forceinline__ dl_f32x4 mma(const DFrag& a, const DFrag& b, dl_f32x4 c) {
     return __builtin_amdgcn_mfma_f32_16x16x32_bf16(a.v, b.v, c, 0, 0, 0);
 }
-// (a0 + a1 + a2)(b0 + b1 + b2) without the products below 2^-24 of the whole
-__device__ __forceinline__ dl_f32x4 mma_terms(const DFrag (&a)[3], const DFrag (&b)[3], dl_f32x4 c) {
-    c = mma(a[0], b[2], c); c = mma(a[2], b[0], c); c = mma(a[1], b[1], c);
-    c = mma(a[0], b[1], c); c = mma(a[1], b[0], c);
-    return mma(a[0], b[0], c);
+// (a0 + a1 + a2)(b0 + b1 + b2) without the products below 2^-24 of the whole, in two chains of sums
+__device__ __forceinline__ void mma_terms(const DFrag (&a)[3], const DFrag (&b)[3], dl_f32x4& c, dl_f32x4& d) {
+    c = mma(a[0], b[2], c); d = mma(a[1], b[1], d);
+    c = mma(a[2], b[0], c); d = mma(a[0], b[1], d);
+    c = mma(a[1], b[0], c); d = mma(a[0], b[0], d);
 }
+// A barrier for what the waves pass through LDS.  (__syncthreads() would also wait for every load from memory that is
+// under way, and a chunk's loads are asked for a chunk ahead.)
+__device__ __forceinline__ void lds_barrier() { asm volatile("s_waitcnt lgkmcnt(0)\n\ts_barrier" ::: "memory"); }
 // where head h of (sequence, chunk) c keeps its two matrices' terms, its scalars, and the kv head's K transposed
 __device__ __forceinline__ bf16_t* ws_terms(const DeltaArgs& x, size_t c, int h, int which) { return x.ws_mat + ((c * x.H + h) * 2 + which) * 3 * DC * DC; }
 __device__ __forceinline__ float* ws_scalars(const DeltaArgs& x, size_t c, int h) { return x.ws_scal + (c * x.H + h) * 4 * DC; }
@@ -207,10 +207,10 @@ __device__ __forceinline__ float* ws_scalars(const DeltaArgs& x, size_t c, int h
 template <int KS>
 __global__ void __launch_bounds__(256)
 delta_prepare_k(DeltaArgs x) {
-    constexpr int LS = DC + 4;
-    __shared__ __attribute__((aligned(16))) float Ls[DC * LS];        // L, then its inverse with the steps
+    constexpr int LS = DC + 4, KP = KS * 32 + 8;
+    __shared__ __attribute__((aligned(16))) float Ls[DC * LS];        // L, then the inverse of I + L
     __shared__ __attribute__((aligned(16))) float As[DC * LS];        // A
-    __shared__ __attribute__((aligned(16))) bf16_t Kt[KS * 32 * DCP];
+    __shared__ __attribute__((aligned(16))) bf16_t Kr[DC * KP], Kt[KS * 32 * DCP];      // the chunk's keys by rows, and transposed
     __shared__ double Gs[DC];
     __shared__ float beta_s[DC], ik_s[DC], iq_s[DC];
     const int seq = blockIdx.x / x.n_chunks, chunk = blockIdx.x % x.n_chunks, h = blockIdx.y;
@@ -218,20 +218,16 @@ delta_prepare_k(DeltaArgs x) {
     if (n <= 0) return;
     const int per = x.H / x.G, kvh = h / per, dk = x.dk;
     const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, r = lane & 15, g = lane >> 4;
-    const bf16_t* qp = (const bf16_t*)x.q + (size_t)kvh * dk;
-    const bf16_t* kp = (const bf16_t*)x.k + (size_t)kvh * dk;
-    const uint4 zero = make_uint4(0, 0, 0, 0);
-    // 8 elements of row t from d on, zeros past the chunk's end and the head's
-    auto piece = [&](const bf16_t* p, long stride, int t, int d) {
-        const bool ok = t < n && d < dk;
-        const uint4 u = *reinterpret_cast<const uint4*>(p + (size_t)(begin + (ok ? t : 0)) * stride + (ok ? d : 0));
-        return ok ? u : zero;
-    };
+    // the wave's 16 rows of K and Q (a row past the chunk's end: its last row once more, of a token whose step is zero)
+    const size_t at = (size_t)(begin + min(wave * 16 + r, n - 1));
+    const bf16_t* kp = (const bf16_t*)x.k + at * x.k_stride + (size_t)kvh * dk;
+    const bf16_t* qp = (const bf16_t*)x.q + at * x.q_stride + (size_t)kvh * dk;
     DFrag kf[KS], qf[KS];
 #pragma unroll
     for (int s = 0; s < KS; s++) {
-        kf[s].u = piece(kp, x.k_stride, wave * 16 + r, s * 32 + g * 8);
-        qf[s].u = piece(qp, x.q_stride, wave * 16 + r, s * 32 + g * 8);
+        const int d = min(s * 32 + g * 8, dk - 8);
+        kf[s].u = *reinterpret_cast<const uint4*>(kp + d);
+        qf[s].u = *reinterpret_cast<const uint4*>(qp + d);
     }
     if (wave == 0) {                                     // the tokens' decays and steps, a token a lane
         double G = 0.0;
@@ -249,6 +245,14 @@ delta_prepare_k(DeltaArgs x) {
         Gs[lane] = G;
         beta_s[lane] = beta;
     }
+    if (dk < KS * 32) {                                  // elements past the head's are zeros
+        const uint4 zero = make_uint4(0, 0, 0, 0);
+#pragma unroll
+        for (int s = 0; s < KS; s++)
+            if (s * 32 + g * 8 >= dk) { kf[s].u = zero; qf[s].u = zero; }
+    }
+#pragma unroll
+    for (int s = 0; s < KS; s++) *reinterpret_cast<uint4*>(Kr + (wave * 16 + r) * KP + s * 32 + g * 8) = kf[s].u;
     {
         float kk = 0.f, qq = 0.f;
 #pragma unroll
@@ -279,7 +283,7 @@ delta_prepare_k(DeltaArgs x) {
 #pragma unroll
             for (int s = 0; s < KS; s++) {
                 DFrag kb;
-                kb.u = piece(kp, x.k_stride, j * 16 + r, s * 32 + g * 8);
+                kb.u = *reinterpret_cast<const uint4*>(Kr + (j * 16 + r) * KP + s * 32 + g * 8);
                 kkt = mma(kf[s], kb, kkt);
                 qkt = mma(qf[s], kb, qkt);
             }
@@ -296,25 +300,36 @@ delta_prepare_k(DeltaArgs x) {
         }
     }
     __syncthreads();
-    float T[DC];                                         // (wave 0) lane: a column of the inverse of I + L
-    if (wave == 0) {
+    // The inverse of I + L by blocks of 16: wave w inverts the diagonal block w, a column a lane, then the blocks left of it,
+    // one diagonal after the other:  T_wj = -T_ww (sum over k = j .. w - 1 of L_wk T_kj).  A wave holds its rows of L, so
+    // that T may take L's place.  The products are float32 ones; a result's rows 4 g + i are the k of its next use at step i.
+    dl_f32x4 Lf[3];                                      // L_wk, lane: row r, columns 4 g + i
 #pragma unroll
-        for (int t = 0; t < DC; t++) {
-            float s0 = 0.f, s1 = 0.f, s2 = 0.f, s3 = 0.f;
-#pragma unroll
-            for (int s = 0; s < t; s += 4) {
-                const float4 l = *reinterpret_cast<const float4*>(Ls + t * LS + s);     // zero from s = t on
-                s0 = __builtin_fmaf(l.x, T[s], s0);
-                if (s + 1 < t) s1 = __builtin_fmaf(l.y, T[s + 1], s1);
-                if (s + 2 < t) s2 = __builtin_fmaf(l.z, T[s + 2], s2);
-                if (s + 3 < t) s3 = __builtin_fmaf(l.w, T[s + 3], s3);
-            }
-            T[t] = (t == lane ? 1.f : 0.f) - ((s0 + s1) + (s2 + s3));
+    for (int k = 0; k < 3; k++)
+        if (k < wave) {
+            const float4 l = *reinterpret_cast<const float4*>(Ls + (wave * 16 + r) * LS + k * 16 + g * 4);
+            Lf[k] = (dl_f32x4){l.x, l.y, l.z, l.w};
         }
-        const float beta = beta_s[lane];
+    {
+        float T[16];
 #pragma unroll
-        for (int t = 0; t < DC; t++) Ls[t * LS + lane] = T[t] * beta;       // only this wave read L
-    } else if (wave == 1) {
+        for (int t = 0; t < 16; t++) {
+            float s0 = 0.f, s1 = 0.f;
+#pragma unroll
+            for (int c = 0; c < t; c += 4) {
+                const float4 l = *reinterpret_cast<const float4*>(Ls + (wave * 16 + t) * LS + wave * 16 + c);     // zero from c = t on
+                s0 = __builtin_fmaf(l.x, T[c], s0);
+                if (c + 1 < t) s1 = __builtin_fmaf(l.y, T[c + 1], s1);
+                if (c + 2 < t) s0 = __builtin_fmaf(l.z, T[c + 2], s0);
+                if (c + 3 < t) s1 = __builtin_fmaf(l.w, T[c + 3], s1);
+            }
+            T[t] = (t == r ? 1.f : 0.f) - (s0 + s1);
+        }
+        if (g == 0)
+#pragma unroll
+            for (int t = 0; t < 16; t++) Ls[(wave * 16 + t) * LS + wave * 16 + r] = T[t];
+    }
+    if (wave == 1) {
         float* sc = ws_scalars(x, blockIdx.x, h);
         const double G = Gs[lane], end = Gs[DC - 1];
         const float eg = expf((float)G);
@@ -322,14 +337,34 @@ delta_prepare_k(DeltaArgs x) {
         sc[DC + lane] = eg * iq_s[lane];
         sc[2 * DC + lane] = expf((float)(end - G)) * ik_s[lane];
         sc[3 * DC + lane] = expf((float)end);
-    } else if (transposes) {
+    }
+    if (transposes) {
         bf16_t* kt = x.ws_kt + ((size_t)blockIdx.x * x.G + kvh) * x.dkp * DC;
-        for (int i = tid - 128; i < KS * 32 * 8; i += 128) {
+        for (int i = tid; i < KS * 32 * 8; i += 256) {
             const int d = i >> 3, c = (i & 7) * 8;
             *reinterpret_cast<uint4*>(kt + d * DC + c) = *reinterpret_cast<const uint4*>(Kt + d * DCP + c);
         }
     }
     __syncthreads();
+#pragma unroll
+    for (int d = 1; d < 4; d++) {
+        const int j = wave - d;
+        if (j >= 0) {
+            dl_f32x4 sum = {0.f, 0.f, 0.f, 0.f}, t = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+            for (int k = 0; k < 3; k++)
+                if (k >= j && k < wave)
+#pragma unroll
+                    for (int i = 0; i < 4; i++)
+                        sum = __builtin_amdgcn_mfma_f32_16x16x4f32(Lf[k][i], Ls[(k * 16 + g * 4 + i) * LS + j * 16 + r], sum, 0, 0, 0);
+#pragma unroll
+            for (int i = 0; i < 4; i++)
+                t = __builtin_amdgcn_mfma_f32_16x16x4f32(-Ls[(wave * 16 + r) * LS + wave * 16 + g * 4 + i], sum[i], t, 0, 0, 0);
+#pragma unroll
+            for (int i = 0; i < 4; i++) Ls[(wave * 16 + g * 4 + i) * LS + j * 16 + r] = t[i];
+        }
+        __syncthreads();
+    }
     // the two matrices in terms: a thread takes 16 columns of a row
     const int row = tid >> 2, col = (tid & 3) * 16;
     if (col < 32 * (row / 32 + 1)) {                     // what a row of tiles is multiplied by: whole k steps up to its diagonal
@@ -339,14 +374,15 @@ delta_prepare_k(DeltaArgs x) {
             bf16_t* dst = ws_terms(x, blockIdx.x, h, which) + row * DC + col;
 #pragma unroll
             for (int e = 0; e < 16; e += 4) {
-                const float4 f = *reinterpret_cast<const float4*>(src + e);
+                float4 f = *reinterpret_cast<const float4*>(src + e);
+                if (which == 0) { f.x *= beta_s[col + e]; f.y *= beta_s[col + e + 1]; f.z *= beta_s[col + e + 2]; f.w *= beta_s[col + e + 3]; }
                 put4(dst + e, DC * DC, f.x, f.y, f.z, f.w);
             }
         }
     }
 }
 
-// grid (sequences, heads, blocks of 16 columns), four waves: wave w takes the tokens 16 w .. 16 w + 15 of a chunk and the 16-row
+// grid (8 dies x units of a (sequence, head) a die takes x blocks of 16 columns), four waves: wave w takes the tokens 16 w .. 16 w + 15 of a chunk and the 16-row
 // tiles w, w + 4, .. of the state, which it keeps in float32; the state's terms, R = V - diag(e^G) K S_0 and U pass between the
 // waves through LDS.
 template <int KS>
@@ -355,17 +391,18 @@ delta_chunks_k(DeltaArgs x) {
     constexpr int DKP = KS * 32, SP = DKP + 8, TILES = (2 * KS + 3) / 4;
     __shared__ __attribute__((aligned(16))) bf16_t S_lds[3][16][SP];
     __shared__ __attribute__((aligned(16))) bf16_t R_lds[3][16][DCP], U_lds[3][16][DCP], C_lds[3][16][DCP];
-    const int seq = blockIdx.x, h = blockIdx.y, c0 = blockIdx.z * 16;
+    // blocks of one head follow one another on one of the eight dies (block b runs on die b % 8), so that a chunk's matrices
+    // and keys come from its cache for all but the first
+    const int places = (x.n_seq * x.H + 7) / 8, blocks_h = (x.dv + 15) / 16, slot = blockIdx.x >> 3;
+    const int unit = (blockIdx.x & 7) * places + slot / blocks_h;
+    if (unit >= x.n_seq * x.H) return;
+    const int seq = unit / x.H, h = unit % x.H, c0 = slot % blocks_h * 16;
     const int row_first = x.cu_rows[seq], count = x.cu_rows[seq + 1] - row_first;
     if (count <= 0) return;
     const int kvh = h / (x.H / x.G), dk = x.dk, dv = x.dv;
     const int tid = threadIdx.x, wave = __builtin_amdgcn_readfirstlane(tid >> 6), lane = tid & 63, r = lane & 15, g = lane >> 4;
     const int col = c0 + r, colc = min(col, dv - 1);
     float* st = x.state + ((size_t)x.slot_ids[seq] * x.H + h) * dk * dv;
-    const bf16_t* qp = (const bf16_t*)x.q + (size_t)kvh * dk;
-    const bf16_t* kp = (const bf16_t*)x.k + (size_t)kvh * dk;
-    const bf16_t* vp = (const bf16_t*)x.v + (size_t)h * dv + colc;
-    const uint4 zero = make_uint4(0, 0, 0, 0);
     dl_f32x4 S[TILES];
 #pragma unroll
     for (int j = 0; j < TILES; j++) {
@@ -378,126 +415,134 @@ delta_chunks_k(DeltaArgs x) {
         }
         if (tile < 2 * KS) put4(&S_lds[0][r][tile * 16 + g * 4], 16 * SP, S[j][0], S[j][1], S[j][2], S[j][3]);
     }
-    // what a chunk needs from memory: asked for a chunk ahead, into the registers it has just left
-    DFrag kf[KS], qf[KS], tf[2][3], af[2][3], ktf[TILES][2];
-    float v[4];
-    float4 ka, qa, kc;
-    float all;
+    // What a chunk needs from memory is asked for a chunk ahead, into the registers it has just left, by loads without a
+    // condition: rows past the sequence's end and elements past a head's read something that exists.  It comes to nothing: such
+    // a token's step is zero (its U with it), the state's rows past dk are zero, and neither is stored.
     const int n_chunks = (count + DC - 1) / DC;
+    const size_t c_first = (size_t)seq * x.n_chunks;
+    DFrag kf[KS], qf[KS], tf[2][3], af[2][3], ktf[TILES][2];
+    bf16_t v[4];
+    float4 ka, qa, kc, ka_next, qa_next, kc_next;
+    float all, all_next;
+    const char* const q_seq = (const char*)((const bf16_t*)x.q + (size_t)row_first * x.q_stride + (size_t)kvh * dk);
+    const char* const k_seq = (const char*)((const bf16_t*)x.k + (size_t)row_first * x.k_stride + (size_t)kvh * dk);
+    const char* const v_seq = (const char*)((const bf16_t*)x.v + (size_t)row_first * x.v_stride + (size_t)h * dv);
     auto rows_of = [&](int c) {                          // K, Q and V of the wave's 16 tokens
-        const int t0 = c * DC + wave * 16;
+        const int first = c * DC, last = count - 1 - first;
+        const char* kb = k_seq + (size_t)first * x.k_stride * 2;
+        const char* qb = q_seq + (size_t)first * x.q_stride * 2;
+        const char* vb = v_seq + (size_t)first * x.v_stride * 2;
+        const unsigned t = (unsigned)min(wave * 16 + r, last);
+        const unsigned ko = t * (unsigned)x.k_stride * 2u, qo = t * (unsigned)x.q_stride * 2u;
 #pragma unroll
         for (int s = 0; s < KS; s++) {
-            const int d = s * 32 + g * 8;
-            const bool ok = t0 + r < count && d < dk;
-            const size_t t = (size_t)(row_first + (ok ? t0 + r : 0));
-            const uint4 ku = *reinterpret_cast<const uint4*>(kp + t * x.k_stride + (ok ? d : 0));
-            const uint4 qu = *reinterpret_cast<const uint4*>(qp + t * x.q_stride + (ok ? d : 0));
-            kf[s].u = ok ? ku : zero;
-            qf[s].u = ok ? qu : zero;
+            const unsigned d = (unsigned)min(s * 32 + g * 8, dk - 8) * 2u;
+            kf[s].u = *reinterpret_cast<const uint4*>(kb + (ko + d));
+            qf[s].u = *reinterpret_cast<const uint4*>(qb + (qo + d));
         }
 #pragma unroll
-        for (int i = 0; i < 4; i++) {
-            const int t = t0 + g * 4 + i;
-            const float e = bf16_to_f32(vp[(size_t)(row_first + min(t, count - 1)) * x.v_stride]);
-            v[i] = t < count && col < dv ? e : 0.f;
-        }
+        for (int i = 0; i < 4; i++)
+            v[i] = *reinterpret_cast<const bf16_t*>(vb + ((unsigned)min(wave * 16 + g * 4 + i, last) * (unsigned)x.v_stride + (unsigned)colc) * 2u);
     };
     auto scalars_of = [&](size_t c) {
-        const float* sc = ws_scalars(x, c, h) + wave * 16 + g * 4;
-        ka = *reinterpret_cast<const float4*>(sc);
-        qa = *reinterpret_cast<const float4*>(sc + DC);
-        kc = *reinterpret_cast<const float4*>(sc + 2 * DC);
-        all = sc[3 * DC];
+        const float* sc = ws_scalars(x, c, h) + wave * 16;
+        ka_next = *reinterpret_cast<const float4*>(sc + g * 4);
+        qa_next = *reinterpret_cast<const float4*>(sc + DC + g * 4);
+        kc_next = *reinterpret_cast<const float4*>(sc + 2 * DC + g * 4);
+        all_next = sc[3 * DC + r];
     };
+    const unsigned term_at = (unsigned)((wave * 16 + r) * DC + g * 8) * 2u;
     auto terms_of = [&](size_t c, int which, DFrag (&f)[2][3]) {
-        const bf16_t* p = ws_terms(x, c, h, which) + (wave * 16 + r) * DC + g * 8;
+        const char* p = (const char*)ws_terms(x, c, h, which);
 #pragma unroll
         for (int s = 0; s < 2; s++)
 #pragma unroll
-            for (int n = 0; n < 3; n++) if (s <= (wave >> 1)) f[s][n].u = *reinterpret_cast<const uint4*>(p + n * DC * DC + s * 32);
+            for (int n = 0; n < 3; n++) f[s][n].u = *reinterpret_cast<const uint4*>(p + (term_at + (unsigned)(n * DC * DC + s * 32) * 2u));
     };
     auto keys_of = [&](size_t c) {
-        const bf16_t* p = x.ws_kt + (c * x.G + kvh) * x.dkp * DC + g * 8;
+        const char* p = (const char*)(x.ws_kt + (c * x.G + kvh) * x.dkp * DC);
 #pragma unroll
         for (int j = 0; j < TILES; j++)
 #pragma unroll
             for (int s = 0; s < 2; s++)
-                if (wave + 4 * j < 2 * KS) ktf[j][s].u = *reinterpret_cast<const uint4*>(p + ((wave + 4 * j) * 16 + r) * DC + s * 32);
+                ktf[j][s].u = *reinterpret_cast<const uint4*>(p + (unsigned)((min(wave + 4 * j, 2 * KS - 1) * 16 + r) * DC + g * 8 + s * 32) * 2u);
     };
-    const size_t c_first = (size_t)seq * x.n_chunks;
     rows_of(0);
     scalars_of(c_first);
     terms_of(c_first, 0, tf);
-    terms_of(c_first, 1, af);
     keys_of(c_first);
-    __syncthreads();
+    terms_of(c_first, 1, af);
+    lds_barrier();
+    const bool both = wave >= 2;                         // the upper two waves' rows of the matrices reach into the second k step
     for (int c = 0; c < n_chunks; c++) {
-        const bool more = c + 1 < n_chunks;
+        const int next = min(c + 1, n_chunks - 1);       // (after the last chunk: once more what is there)
+        ka = ka_next; qa = qa_next; kc = kc_next; all = all_next;
         // K S_0 and Q S_0
-        dl_f32x4 ks = {0.f, 0.f, 0.f, 0.f}, qs = {0.f, 0.f, 0.f, 0.f};
+        dl_f32x4 ks[2], qs[2];
+#pragma unroll
+        for (int i = 0; i < 2; i++) { ks[i] = (dl_f32x4){0.f, 0.f, 0.f, 0.f}; qs[i] = ks[i]; }
 #pragma unroll
         for (int n = 2; n >= 0; n--)
 #pragma unroll
             for (int s = 0; s < KS; s++) {
                 DFrag b;
                 b.u = *reinterpret_cast<const uint4*>(&S_lds[n][r][s * 32 + g * 8]);
-                ks = mma(kf[s], b, ks);
-                qs = mma(qf[s], b, qs);
+                ks[s & 1] = mma(kf[s], b, ks[s & 1]);
+                qs[s & 1] = mma(qf[s], b, qs[s & 1]);
             }
-        put4(&R_lds[0][r][wave * 16 + g * 4], 16 * DCP, v[0] - ka.x * ks[0], v[1] - ka.y * ks[1], v[2] - ka.z * ks[2], v[3] - ka.w * ks[3]);
-        dl_f32x4 o = {qa.x * qs[0], qa.y * qs[1], qa.z * qs[2], qa.w * qs[3]};
-        if (more) rows_of(c + 1);
-        __syncthreads();
-        dl_f32x4 u = {0.f, 0.f, 0.f, 0.f};
+        ks[0] = ks[0] + ks[1];
+        put4(&R_lds[0][r][wave * 16 + g * 4], 16 * DCP, bf16_to_f32(v[0]) - ka.x * ks[0][0], bf16_to_f32(v[1]) - ka.y * ks[0][1],
+             bf16_to_f32(v[2]) - ka.z * ks[0][2], bf16_to_f32(v[3]) - ka.w * ks[0][3]);
+        qs[0] = qs[0] + qs[1];
+        dl_f32x4 o = {qa.x * qs[0][0], qa.y * qs[0][1], qa.z * qs[0][2], qa.w * qs[0][3]}, o1 = {0.f, 0.f, 0.f, 0.f};
+        rows_of(next);
+        scalars_of(c_first + next);
+        lds_barrier();
+        dl_f32x4 u = {0.f, 0.f, 0.f, 0.f}, u1 = u;
 #pragma unroll
         for (int s = 0; s < 2; s++)
-            if (s <= (wave >> 1)) {
+            if (s == 0 || both) {
                 DFrag b[3];
 #pragma unroll
                 for (int n = 0; n < 3; n++) b[n].u = *reinterpret_cast<const uint4*>(&R_lds[n][r][s * 32 + g * 8]);
-                u = mma_terms(tf[s], b, u);
+                mma_terms(tf[s], b, u, u1);
             }
-        put4(&U_lds[0][r][wave * 16 + g * 4], 16 * DCP, u[0], u[1], u[2], u[3]);
+        u = u + u1;
+        terms_of(c_first + next, 0, tf);
         put4(&C_lds[0][r][wave * 16 + g * 4], 16 * DCP, kc.x * u[0], kc.y * u[1], kc.z * u[2], kc.w * u[3]);
-        if (more) terms_of(c_first + c + 1, 0, tf);
-        __syncthreads();
+        put4(&U_lds[0][r][wave * 16 + g * 4], 16 * DCP, u[0], u[1], u[2], u[3]);
 #pragma unroll
         for (int j = 0; j < TILES; j++) S[j] = S[j] * all;
+        lds_barrier();
 #pragma unroll
         for (int s = 0; s < 2; s++) {
             DFrag b[3];
 #pragma unroll
             for (int n = 0; n < 3; n++) b[n].u = *reinterpret_cast<const uint4*>(&C_lds[n][r][s * 32 + g * 8]);
 #pragma unroll
-            for (int j = 0; j < TILES; j++)
-                if (wave + 4 * j < 2 * KS) {
-                    S[j] = mma(ktf[j][s], b[2], S[j]);
-                    S[j] = mma(ktf[j][s], b[1], S[j]);
-                    S[j] = mma(ktf[j][s], b[0], S[j]);
-                }
-        }
-        if (more)
+            for (int n = 2; n >= 0; n--)
 #pragma unroll
-            for (int j = 0; j < TILES; j++)
-                if (wave + 4 * j < 2 * KS) put4(&S_lds[0][r][(wave + 4 * j) * 16 + g * 4], 16 * SP, S[j][0], S[j][1], S[j][2], S[j][3]);
+                for (int j = 0; j < TILES; j++) S[j] = mma(ktf[j][s], b[n], S[j]);
+        }
+        keys_of(c_first + next);
+#pragma unroll
+        for (int j = 0; j < TILES; j++)
+            if (2 * KS % 4 == 0 || wave + 4 * j < 2 * KS) put4(&S_lds[0][r][(wave + 4 * j) * 16 + g * 4], 16 * SP, S[j][0], S[j][1], S[j][2], S[j][3]);
 #pragma unroll
         for (int s = 0; s < 2; s++)
-            if (s <= (wave >> 1)) {
+            if (s == 0 || both) {
                 DFrag b[3];
 #pragma unroll
                 for (int n = 0; n < 3; n++) b[n].u = *reinterpret_cast<const uint4*>(&U_lds[n][r][s * 32 + g * 8]);
-                o = mma_terms(af[s], b, o);
+                mma_terms(af[s], b, o, o1);
             }
+        terms_of(c_first + next, 1, af);
+        o = o + o1;
         const int t0 = c * DC + wave * 16 + g * 4;
+        float* yr = x.y + ((size_t)(row_first + t0) * x.H + h) * dv + col;
 #pragma unroll
-        for (int i = 0; i < 4; i++) if (t0 + i < count && col < dv) x.y[((size_t)(row_first + t0 + i) * x.H + h) * dv + col] = o[i];
-        if (more) {
-            terms_of(c_first + c + 1, 1, af);
-            keys_of(c_first + c + 1);
-            scalars_of(c_first + c + 1);
-        }
-        __syncthreads();
+        for (int i = 0; i < 4; i++) if (t0 + i < count && col < dv) yr[(size_t)i * x.H * dv] = o[i];
+        lds_barrier();
     }
 #pragma unroll
     for (int j = 0; j < TILES; j++)
@@ -532,7 +577,7 @@ extern "C" int tp_delta_scan(const void* q, long q_stride, const void* k, long k
     TP_REQUIRE(q && k && v && b && a && a_log && dt_bias && state && slot_ids && cu_rows && y, "delta_scan: null operand");
     TP_REQUIRE(dtype == TP_BF16 || dtype == TP_F32, "delta_scan: unknown dtype %d", dtype);
     hipStream_t s = (hipStream_t)stream;
-    DeltaArgs x{q, q_stride, k, k_stride, v, v_stride, b, a, gate_stride, a_log, dt_bias, state, slot_ids, cu_rows, y, H, G, dk, dv, q_scale,
+    DeltaArgs x{q, q_stride, k, k_stride, v, v_stride, b, a, gate_stride, a_log, dt_bias, state, slot_ids, cu_rows, y, n_seq, H, G, dk, dv, q_scale,
                 0, 0, nullptr, nullptr, nullptr};
     dim3 grid(n_seq, H, tp_cdiv(dv, 16));
     if (n_chunks > 0) {
@@ -547,7 +592,9 @@ extern "C" int tp_delta_scan(const void* q, long q_stride, const void* k, long k
         x.ws_scal = (float*)((char*)workspace + delta_mat_bytes(units));
         x.ws_kt = (bf16_t*)((char*)x.ws_scal + delta_scal_bytes(units));
         dim3 pgrid(n_seq * n_chunks, H);
-#define TP_DELTA_CHUNKS(KS) do { delta_prepare_k<KS><<<pgrid, 256, 0, s>>>(x); delta_chunks_k<KS><<<grid, 256, 0, s>>>(x); } while (0)
+        const long cgrid = 8L * ((n_seq * (long)H + 7) / 8) * tp_cdiv(dv, 16);
+        TP_REQUIRE(cgrid <= 0x7fffffffL, "delta_scan: %ld blocks exceed one launch", cgrid);
+#define TP_DELTA_CHUNKS(KS) do { delta_prepare_k<KS><<<pgrid, 256, 0, s>>>(x); delta_chunks_k<KS><<<(unsigned)cgrid, 256, 0, s>>>(x); } while (0)
         switch (x.dkp / 32) {
             case 1: TP_DELTA_CHUNKS(1); break;
             case 2: TP_DELTA_CHUNKS(2); break;

@@ -409,7 +409,7 @@ __global__ void __launch_bounds__(256)
 expert_stream_k(const bf16_t* __restrict__ a, const bf16_t* __restrict__ w, const int* __restrict__ order, const int* __restrict__ first,
                 int E, int top, int N, int K, float limit, float alpha, float shift, const float* __restrict__ in_scale, void* __restrict__ out, int k_slice, long out_slice) {
     constexpr bool GATED = KIND == TP_EXPERT_GATED, GATHER = KIND != TP_EXPERT_DOWN;
-    constexpr int TM = 16, UN = 8;
+    constexpr int TM = 16, UN = GATED ? 8 : 12;          // (measured: 12 against 8 is 106 -> 99 us for 7 experts of 4,608 at width 2,304, 16 is 115)
     int t = blockIdx.y, e = 0, lo = 0, hi = 0;
     for (; e < E; e++) {
         lo = first[e]; hi = first[e + 1];

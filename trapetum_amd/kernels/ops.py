@@ -675,7 +675,7 @@ class HipOps:
         return y
 
     DELTA_CHUNK = 64               # tokens of a chunk (the kernel library's)
-    DELTA_CHUNKS_FROM = 48         # rows of the longest sequence from which a bfloat16 step runs in chunks
+    DELTA_CHUNKS_FROM = 16         # rows of the longest sequence from which a bfloat16 step runs in chunks
 
     def delta_scan(self, q, k, v, b, a, a_log, dt_bias, state, slot_ids, cu_rows, max_count, heads, kv_heads, dk, dv, q_scale, chunks=None):
         """The gated delta rule over the step's rows, sequence by sequence, from state[slot] (float32 [slots, heads, dk,
