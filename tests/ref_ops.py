@@ -375,6 +375,14 @@ def conv_act(x, w_t, bias, state, slot_ids, cu_rows, row_seq, activation=None, o
     return out.to(x.dtype)
 
 
+def conv_step(rows, w_t, state, slot_ids, out_dtype, activation=None):
+    x = rows.slices.sum(0) if hasattr(rows, "slices") else rows
+    x, c = x.to(out_dtype), w_t.shape[1]
+    n = x.shape[0]
+    out = conv_act(x[:, :c], w_t, None, state, slot_ids, torch.arange(n + 1), torch.arange(n), activation=activation, one_row_each=True)
+    return torch.cat([out, x[:, c:]], dim=1)
+
+
 def ssd_scan(xbc, z, dt, dt_bias, a_log, skip, state, slot_ids, cu_rows, max_count, heads, groups, n_state, head_dim):
     """S <- exp(-exp(a_log) d) S + d B x^T, y = (S^T C + skip x) * silu(z), d = softplus(dt + dt_bias), row after row of
     every sequence from state[slot] [heads, n_state, head_dim], which is left updated.  float32 [M, heads head_dim]."""

@@ -100,6 +100,25 @@ def test_delta_part(rt, H, G, dim, vdim, taps, a_log):
         assert rel_l2(got[i][0], plain.delta(wide[i], W, "", sizes, EPS)) < tolerance(rt) * (1 if rt.dtype == torch.float32 else 2), i
 
 
+@pytest.mark.parametrize("m,n,c,taps,slices,act", [(1, 40, 40, 3, 0, None), (5, 700, 333, 4, 3, "silu"), (8, 96, 64, 1, 5, "silu"), (3, 130, 130, 2, 1, None),
+                                                   (64, 300, 20, 6, 2, "silu")])
+def test_convolution_of_single_rows(rt, m, n, c, taps, slices, act):
+    """One row per sequence, from a product in K slices or in one piece: the first columns are convolved, the others pass; the
+    states move on by the rows as they were used."""
+    rows = rnd(slices, m, n, seed=1) if slices else acts(rt, rnd(m, n, seed=1))[1].to(rt.dtype)
+    w_t, state = rnd(taps, c, seed=2, scale=0.5), rnd(m + 3, max(taps - 1, 1), c, seed=3)
+    slots = torch.randperm(m + 3, generator=torch.Generator().manual_seed(4))[:m].to(torch.int32)
+    want_state, got_state = state.clone(), state.to(rt.device)
+    x = ref_ops.SplitRows(rows) if slices else rows
+    want = ref_ops.conv_step(x, w_t, want_state if taps > 1 else None, slots, rt.dtype, act)
+    x = rt.ops.SplitRows(rows.to(rt.device)) if slices else rows.to(rt.device)
+    got = rt.ops.conv_step(x, w_t.to(rt.device), got_state if taps > 1 else None, slots.to(rt.device), rt.dtype, act)
+    assert got.shape == (m, n) and rel_l2(got, want) < (1e-6 if rt.dtype == torch.float32 else 3e-3)
+    assert rel_l2(got_state, want_state) < (1e-6 if rt.dtype == torch.float32 else 3e-3)
+    untouched = [s for s in range(m + 3) if s not in slots.tolist()]
+    assert torch.equal(got_state[untouched].cpu(), state[untouched])
+
+
 def test_delta_remembers_and_unlearns(rt):
     """Decays of almost one and steps of almost one: hundreds of tokens after its first tokens the memory still answers to a
     key with what was written there last, not with what that key held before."""

@@ -177,12 +177,17 @@ def time_solulix_kernels(engine, cfg, batch, context, prefill_tokens):
             prod = (lambda name, calls, w, m=rows: one(calls, name=name, bytes_each=2.0 * elems(w)) if decode
                     else one(calls, name=name, flops_each=2.0 * m * elems(w)))
 
-            def conv(name, mixer, u, e, activation):
-                ch = mixer.conv_t.shape[1]
-                state = cache.entry_state(e, "mixer.conv")
-                call = lambda: ops.conv_act(u[:, :ch], mixer.conv_t, None, state, ctx.slot_ids, ctx.cu_rows, ctx.row_seq, activation=activation,
-                                            one_row_each=decode)
-                one([call] * 16, name=name, bytes_each=rows * ch * 4.0 + (rows * (mixer.taps - 1) * ch * 8.0 if decode else 0.0))
+            def conv(name, mixer, w, e, activation):
+                """The convolution on a product of the matrices w, as the step hands it over (in K slices where they are left)."""
+                ch, state = mixer.conv_t.shape[1], cache.entry_state(e, "mixer.conv")
+                u = ops.linear(x, w, bf, defer=decode)
+                if decode:
+                    call = lambda: ops.conv_step(u, mixer.conv_t, state, ctx.slot_ids, bf, activation=activation)
+                    size = 4.0 * u.slices.numel() if isinstance(u, ops.SplitRows) else 2.0 * u.numel()
+                    one([call] * 16, name=name, bytes_each=size + rows * (w.shape[0] * 2.0 + (mixer.taps - 1) * ch * 8.0))
+                else:
+                    call = lambda: ops.conv_act(u[:, :ch], mixer.conv_t, None, state, ctx.slot_ids, ctx.cu_rows, ctx.row_seq, activation=activation)
+                    one([call] * 16, name=name, bytes_each=rows * ch * 4.0)
                 return call()
             if att:
                 e = entry(att)
@@ -191,8 +196,8 @@ def time_solulix_kernels(engine, cfg, batch, context, prefill_tokens):
                 site = cache.site(e)
                 table, kp, vp, cap = ctx.page_table(site.group_index), site.tensor("k"), site.tensor("v"), site.rows_cap or 0
                 kept = dict(keep=F, pin=site.pinned)
-                prod("qkv", [(lambda b=b: ops.linear(x, b.mixer.w_qkv, bf)) for b in att], a.w_qkv)
-                qkv = conv("qkv_conv", a, torch.randn((rows, (H + 2 * KV) * row), device=dev).to(bf), e, None)
+                prod("qkv", [(lambda b=b: ops.linear(x, b.mixer.w_qkv, bf, defer=decode)) for b in att], a.w_qkv)
+                qkv = conv("qkv_conv", a, a.w_qkv, e, None)
                 seen = lambda p: min(p + 1, W + min(F, max(0, p + 1 - W)))
                 if decode:
                     one([lambda: ops.attention_decode_step(qkv, H, KV, row, None, 0, ctx.new_len, table, kp, vp, cap, a.query_scale, 0.0, W, bf,
@@ -211,11 +216,11 @@ def time_solulix_kernels(engine, cfg, batch, context, prefill_tokens):
                 e = entry(rec)
                 mx = rec[0].mixer
                 H, G, dk, dv, ch = mx.num_heads, mx.num_kv_heads, mx.key_dim, mx.value_dim, mx.conv_channels
-                prod("delta_in", [(lambda b=b: ops.linear(x, b.mixer.w_in, bf)) for b in rec], mx.w_in)
+                prod("delta_in", [(lambda b=b: ops.linear(x, b.mixer.w_in, bf, defer=decode)) for b in rec], mx.w_in)
+                u = conv("delta_conv", mx, mx.w_in, e, "silu")
                 p = (torch.randn((rows, mx.w_in.shape[0]), device=dev) * 0.7).to(bf)
-                u = conv("delta_conv", mx, p, e, "silu")
                 state = cache.entry_state(e, "mixer.memory")
-                scan = lambda: ops.delta_scan(u[:, :G * dk], u[:, G * dk:2 * G * dk], u[:, 2 * G * dk:], p[:, ch + H * dv:ch + H * dv + H],
+                scan = lambda: ops.delta_scan(u[:, :G * dk], u[:, G * dk:2 * G * dk], u[:, 2 * G * dk:ch], p[:, ch + H * dv:ch + H * dv + H],
                                               p[:, ch + H * dv + H:ch + H * dv + 2 * H], mx.a_log, mx.dt_bias, state, ctx.slot_ids, ctx.cu_rows,
                                               ctx.max_count, H, G, dk, dv, dk ** -0.5)
                 if decode:

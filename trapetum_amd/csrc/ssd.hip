@@ -3,6 +3,8 @@
 //
 //   conv_act      out_t = act(b + sum_j w[:, j] u_(t - taps + 1 + j)) on every channel of the step's rows, the rows before
 //                 the step kept per sequence as a state (float32, the projection's values as they were)
+//   conv_step     the same for a step that brings one row per sequence, from a product that is still in K slices; columns behind
+//                 the convolution's are added up and passed through
 //   ssd_scan      S_t = exp(-exp(a) dt_t) S_(t-1) + dt_t B_t x_t^T,  y_t = (S_t^T C_t + D x_t) * silu(z_t),
 //                 dt_t = softplus(raw_t + bias); S, dt, the decay and y in float32
 //   pair_norm_mean  0.5 (a / rms(a) * wa + b / rms(b) * wb) over rows
@@ -137,6 +139,62 @@ extern "C" int tp_conv_act(const void* x, long x_stride, int in_dtype, const flo
         return tp_check_launch("conv_act (state)");
     }
     return 0;
+}
+
+// grid (rows, column blocks of 256).  rows: [n_slices][M, N] float32 slices (or one of the output's dtype) of a product whose first C
+// columns pass the convolution.  A sum of slices is rounded to the output's dtype before it is used, as the product's own
+// rows are; the state takes what was used.
+template <typename TR, typename T>
+__global__ void __launch_bounds__(256)
+conv_step_k(const TR* __restrict__ rows, int n_slices, long slice_stride, long row_stride, const float* __restrict__ wt, float* __restrict__ state,
+            const int* __restrict__ slot_ids, T* __restrict__ out, int N, int C, int taps, int act) {
+    const int r = blockIdx.x, c = blockIdx.y * 256 + threadIdx.x;
+    if (c >= N) return;
+    const TR* src = rows + (size_t)r * row_stride + c;
+    const int S = taps - 1;
+    const bool conv = c < C;
+    float* st = conv && S > 0 ? state + (size_t)slot_ids[r] * S * C + c : nullptr;
+    float sum = 0.f;
+    for (int s0 = 0; s0 < n_slices; s0 += 4) {           // four slices' loads in flight, added in slice order
+        float t[4];
+#pragma unroll
+        for (int u = 0; u < 4; u++) t[u] = ld_f32(src + (size_t)(s0 + u < n_slices ? s0 + u : n_slices - 1) * slice_stride);
+#pragma unroll
+        for (int u = 0; u < 4; u++) sum += s0 + u < n_slices ? t[u] : 0.f;
+    }
+    T* dst = out + (size_t)r * N + c;
+    T kept;
+    st_f32(&kept, sum);
+    if (!conv) { *dst = kept; return; }
+    const float x = ld_f32(&kept);
+    float acc = 0.f;
+    for (int j = 0; j < S; j++) {                        // the state moves on by one row behind the read
+        const float v = st[(size_t)j * C];
+        acc = __builtin_fmaf(wt[(size_t)j * C + c], v, acc);
+        if (j > 0) st[(size_t)(j - 1) * C] = v;
+    }
+    acc = __builtin_fmaf(wt[(size_t)S * C + c], x, acc);
+    if (S > 0) st[(size_t)(S - 1) * C] = x;
+    if (act == TP_CONV_ACT_SILU) acc = acc / (1.f + expf(-acc));
+    st_f32(dst, acc);
+}
+
+extern "C" int tp_conv_step(const void* rows, int rows_dtype, int n_slices, long slice_stride, long row_stride, const float* wt, float* state,
+                            const int* slot_ids, void* out, int out_dtype, int M, int N, int C, int taps, int act, void* stream) {
+    TP_REQUIRE(M > 0 && N > 0 && C > 0 && C <= N && taps >= 1, "conv_step: empty shape M=%d N=%d C=%d taps=%d", M, N, C, taps);
+    TP_REQUIRE(rows && wt && out && (taps == 1 || (state && slot_ids)), "conv_step: a null operand");
+    TP_REQUIRE(n_slices >= 1 && (n_slices == 1 || rows_dtype == TP_F32), "conv_step: rows in %d slices must be float32", n_slices);
+    TP_REQUIRE(act == TP_CONV_ACT_NONE || act == TP_CONV_ACT_SILU, "conv_step: unknown activation %d", act);
+    hipStream_t s = (hipStream_t)stream;
+    dim3 grid(M, tp_cdiv(N, 256));
+    if (rows_dtype == TP_F32 && out_dtype == TP_BF16)
+        conv_step_k<float, bf16_t><<<grid, 256, 0, s>>>((const float*)rows, n_slices, slice_stride, row_stride, wt, state, slot_ids, (bf16_t*)out, N, C, taps, act);
+    else if (rows_dtype == TP_F32 && out_dtype == TP_F32)
+        conv_step_k<float, float><<<grid, 256, 0, s>>>((const float*)rows, n_slices, slice_stride, row_stride, wt, state, slot_ids, (float*)out, N, C, taps, act);
+    else if (rows_dtype == TP_BF16 && out_dtype == TP_BF16)
+        conv_step_k<bf16_t, bf16_t><<<grid, 256, 0, s>>>((const bf16_t*)rows, n_slices, slice_stride, row_stride, wt, state, slot_ids, (bf16_t*)out, N, C, taps, act);
+    else return tp_fail("conv_step: no kernel from dtype %d to dtype %d", rows_dtype, out_dtype);
+    return tp_check_launch("conv_step");
 }
 
 // ---- the scan ---------------------------------------------------------------------------------------------------

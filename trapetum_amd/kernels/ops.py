@@ -26,6 +26,7 @@ _CORE_SIGS = {
     "tp_expert_ffn_workspace_bytes": [_I, _I, _I, _I, _I, _I],
     "tp_expert_ffn": [_P, _I, _I, _I, _P, _P, _I, _I, _I, _P, _P, _I, _F, _F, _F, _I, _P, _L, _P, _I, _P],
     "tp_conv_act": [_P, _L, _I, _P, _P, _P, _P, _P, _P, _P, _L, _I, _I, _I, _I, _I, _I, _I, _P],
+    "tp_conv_step": [_P, _I, _I, _L, _L, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _P],
     "tp_ssd_scan_workspace_bytes": [_I, _I, _I, _I, _I, _I],
     "tp_ssd_scan": [_P, _L, _P, _L, _P, _L, _I, _P, _P, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _I, _P, _L, _P],
     "tp_pair_norm_mean": [_P, _P, _I, _P, _P, _F, _P, _I, _I, _P],
@@ -486,6 +487,32 @@ class HipOps:
         self._call(self.lib, "tp_conv_act", x.data_ptr(), stride, _code(x.dtype), w_t.data_ptr(), bias.data_ptr() if bias is not None else None,
                    state.data_ptr() if taps > 1 else None, slot_ids.data_ptr(), cu_rows.data_ptr(), row_seq.data_ptr(), out.data_ptr(), c,
                    _code(out.dtype), m, n_seq, c, taps, CONV_ACTIVATIONS[activation], 1 if one_row_each else 0, self._stream())
+        return out
+
+    def conv_step(self, rows, w_t, state, slot_ids, out_dtype, activation=None):
+        """`conv_act` without a bias for a step of one row per sequence, on a product as `linear(..., defer=True)` gave it: rows
+        [M, N] or SplitRows, of which the first C columns (w_t float32 [taps, C]) pass the convolution and the others are
+        passed through.  Row i belongs to the sequence whose state is state[slot_ids[i]].  Returns [M, N] of out_dtype."""
+        if activation not in CONV_ACTIVATIONS:
+            raise KernelError(f"conv_step: activation '{activation}' has no kernel")
+        n_slices, slice_stride = 1, 0
+        if isinstance(rows, SplitRows):
+            n_slices, slice_stride, rows = rows.slices.shape[0], rows.slices.stride(0), rows.slices[0]
+        self._dev(rows, w_t, state, slot_ids)
+        row_stride = self._rows(rows, "conv_step rows")
+        m, n = rows.shape
+        if w_t.dtype != torch.float32 or w_t.dim() != 2 or not 0 < w_t.shape[1] <= n or not w_t.is_contiguous():
+            raise KernelError(f"conv_step: the taps must be contiguous float32 [taps, channels] of at most {n} channels")
+        taps, c = w_t.shape
+        if slot_ids.dtype != torch.int32 or slot_ids.numel() != m:
+            raise KernelError("conv_step: slot_ids must be int32, one entry per row")
+        if taps > 1 and (state is None or state.dtype != torch.float32 or state.dim() != 3 or tuple(state.shape[1:]) != (taps - 1, c)
+                         or not state.is_contiguous()):
+            raise KernelError(f"conv_step: the state must be contiguous float32 [slots, {taps - 1}, {c}]")
+        out = torch.empty((m, n), dtype=out_dtype, device=self.device)
+        self._call(self.lib, "tp_conv_step", rows.data_ptr(), _code(rows.dtype), n_slices, slice_stride, row_stride, w_t.data_ptr(),
+                   state.data_ptr() if taps > 1 else None, slot_ids.data_ptr(), out.data_ptr(), _code(out_dtype), m, n, c, taps,
+                   CONV_ACTIVATIONS[activation], self._stream())
         return out
 
     SSD_CHUNK = 64                 # rows of a piece when a long scan is cut into pieces that run side by side

@@ -237,10 +237,13 @@ class Attention(Mixer):
         ctx.ops.rope_kv_write(rows, None, None, heads, 0, self.row, freq, self.value_dim, ctx.row_seq, ctx.row_pos, ctx.new_len,
                               None, None, None, 0, write=False)
 
-    def _convolve(self, ctx, qkv):
-        """The projected rows of a step through the convolutions over time; the state takes the last of them."""
-        return ctx.ops.conv_act(qkv, self.conv_t, None, self.state(ctx, "conv") if self.taps > 1 else None, ctx.slot_ids, ctx.cu_rows,
-                                ctx.row_seq, one_row_each=ctx.mode == "decode")
+    def _convolved(self, ctx, x, w_in):
+        """The step's projected rows through the convolutions over time; the state takes the last of them.  In a decode step
+        the product may stay in K slices until then."""
+        ops, state = ctx.ops, self.state(ctx, "conv") if self.taps > 1 else None
+        if ctx.mode == "decode":
+            return ops.conv_step(ops.linear(x, w_in, ctx.dtype, defer=True), self.conv_t, state, ctx.slot_ids, ctx.dtype)
+        return ops.conv_act(ops.linear(x, w_in, ctx.dtype), self.conv_t, None, state, ctx.slot_ids, ctx.cu_rows, ctx.row_seq)
 
     def _forward_pooled(self, ctx, x, site):
         import torch
@@ -300,18 +303,16 @@ class Attention(Mixer):
         fuses = fuses and ctx.mode == "decode" and ops.fuses_decode_step(ctx.dtype, H, KV, hd, k_pool)
         if fuses:
             # one launch rotates, writes the cache and attends; the projections may stay in K slices until then
-            if self.taps:
-                qkv = self._convolve(ctx, ops.linear(x, w_in, ctx.dtype))
-            else:
-                qkv = ops.linear(x, w_in, ctx.dtype, defer=True)
+            qkv = self._convolved(ctx, x, w_in) if self.taps else ops.linear(x, w_in, ctx.dtype, defer=True)
             out = ops.attention_decode_step(qkv, H, KV, hd, self.inv_freq, self.position.rotary_dim, ctx.new_len,
                                             table, k_pool, v_pool, rows_cap, self.query_scale, self.softcap,
                                             self.window, ctx.dtype, max_keys=ctx.max_rows_visible(site), write_kv=owns_cache,
                                             **(dict(sink=self.sink) if self.sink is not None else {}), **kept)
             return self._project_out(ctx, x, out)
-        qkv = ops.linear(x, w_in, ctx.dtype, bias=bias) if bias is not None else ops.linear(x, w_in, ctx.dtype)
         if self.taps:
-            qkv = self._convolve(ctx, qkv)
+            qkv = self._convolved(ctx, x, w_in)
+        else:
+            qkv = ops.linear(x, w_in, ctx.dtype, bias=bias) if bias is not None else ops.linear(x, w_in, ctx.dtype)
         if owns_cache:
             q, k, v = qkv[:, :Q], qkv[:, Q:Q + KVD], qkv[:, Q + KVD:]
         else:

@@ -74,10 +74,13 @@ class GatedDelta(Mixer):
     def forward(self, ctx, x, site):
         ops, H = ctx.ops, self.num_heads
         qk, vv, ch = self.num_kv_heads * self.key_dim, H * self.value_dim, self.conv_channels
-        p = ops.linear(x, self.w_in, ctx.dtype)                                                   # [M, q | k | v | g | b | a]
-        u = ops.conv_act(p[:, :ch], self.conv_t, None, self.state(ctx, "conv") if self.taps > 1 else None, ctx.slot_ids, ctx.cu_rows,
-                         ctx.row_seq, activation="silu", one_row_each=ctx.mode == "decode")
-        y = ops.delta_scan(u[:, :qk], u[:, qk:2 * qk], u[:, 2 * qk:], p[:, ch + vv:ch + vv + H], p[:, ch + vv + H:ch + vv + 2 * H],
+        state = self.state(ctx, "conv") if self.taps > 1 else None
+        if ctx.mode == "decode":                 # the product may stay in K slices until the convolution's launch
+            p = u = ops.conv_step(ops.linear(x, self.w_in, ctx.dtype, defer=True), self.conv_t, state, ctx.slot_ids, ctx.dtype, activation="silu")
+        else:
+            p = ops.linear(x, self.w_in, ctx.dtype)                                               # [M, q | k | v | g | b | a]
+            u = ops.conv_act(p[:, :ch], self.conv_t, None, state, ctx.slot_ids, ctx.cu_rows, ctx.row_seq, activation="silu")
+        y = ops.delta_scan(u[:, :qk], u[:, qk:2 * qk], u[:, 2 * qk:ch], p[:, ch + vv:ch + vv + H], p[:, ch + vv + H:ch + vv + 2 * H],
                            self.a_log, self.dt_bias, self.state(ctx, "memory"), ctx.slot_ids, ctx.cu_rows, ctx.max_count, H,
                            self.num_kv_heads, self.key_dim, self.value_dim, self.key_dim ** -0.5)
         y = ops.head_norm_gate(y, self.norm_gain, p[:, ch:ch + vv], self.norm_eps, H, "silu", ctx.dtype)
