@@ -46,10 +46,19 @@ def add_rms_norm(stream, rows, gain_post, eps_post, gain_next, eps_next, out_dty
     return _norm(stream, gain_next, eps_next, groups).to(out_dtype)
 
 
-def join_rms_norm(stream, a, b, gain, eps, out_dtype, vec=None, origin=None):
-    for r in (a, b):
+def join_rms_norm(stream, a, b, gain, eps, out_dtype, vec=None, origin=None, wa=1.0, wb=1.0, fresh=False, stack=0):
+    """stream += wa a + wb b (+ vec + origin), or (fresh) becomes it; returns its norm, or (stack) the operand rows of a product
+    over [stream | origin]: as they are, or in bfloat16 terms, two of the stream and `stack` of origin."""
+    if fresh:
+        stream.zero_()
+    for r, w in ((a, wa), (b, wb)):
         if r is not None:
-            stream += r.slices.sum(0) if hasattr(r, "slices") else r.float()
+            stream += w * (r.slices.sum(0) if hasattr(r, "slices") else r.float())
+    if stack:
+        if out_dtype == torch.float32:
+            return torch.cat([stream, origin], dim=1)
+        terms = lambda x: [x.to(out_dtype), (x - x.to(out_dtype).float()).to(out_dtype)]
+        return torch.cat(terms(stream) + terms(origin)[:stack], dim=1)
     if origin is not None:
         stream += origin
     if vec is not None:
@@ -102,9 +111,12 @@ def latent_prepare(proj, H, dn, dr, R, gain, eps, inv_freq, rot, row_seq, row_po
     return q.reshape(m, H * (dr + R)), mine
 
 
-def head_linear(x, w, out=None):
-    """x [M, H, K] (any strides), w [H, N, K] -> out [M, H, N] (a view to fill, or a new tensor of x's dtype)."""
+def head_linear(x, w, out=None, gate=None):
+    """x [M, H, K] (any strides), w [H, N, K] -> out [M, H, N] (a view to fill, or a new tensor of x's dtype), times
+    sigmoid(gate) with gate [M, H N]."""
     y = torch.einsum("mhk,hnk->mhn", x.float(), w.float())
+    if gate is not None:
+        y = y * torch.sigmoid(gate.float()).reshape(y.shape)
     if out is None:
         return y.to(x.dtype).contiguous()
     out.copy_(y.to(out.dtype))
@@ -149,8 +161,12 @@ def expert_ffn(x, chosen, weights, w_gate_up, w_down, limit, alpha, shift, weigh
     return out
 
 
-def linear_act(x, w, out_dtype, activation):
-    assert activation == "relu2"
+def linear_act(x, w, out_dtype, activation, columns=None):
+    if activation == "silu":
+        y = x.float() @ w.float().T
+        n = y.shape[1] if columns is None else columns
+        return torch.cat([y[:, :n] * torch.sigmoid(y[:, :n]), y[:, n:]], dim=1).to(out_dtype)
+    assert activation == "relu2" and columns is None
     return (torch.clamp(x.float() @ w.float().T, min=0.0) ** 2).to(out_dtype)
 
 
@@ -234,11 +250,31 @@ def kv_write(k, v, KV, hd, row_seq, row_pos, new_len, table, k_pool, v_pool, row
     _cache_rows(k, v, row_seq, row_pos, new_len, table, k_pool, v_pool, rows_cap, pin)
 
 
-def _attend(qrow, keys, vals, scale, softcap, sink=None):
-    """qrow [hd], keys/vals [n, hd], fp32.  sink: a score without key or value that joins the denominator."""
+class ByPosition:
+    """temperature (coef, every), bias [H, reach + 1] by distance, gate [rows, H]: each may be absent."""
+
+    def __init__(self, temperature=None, bias=None, gate=None):
+        self.temperature, self.bias, self.gate = temperature, bias, gate
+
+    def of_query(self, p, see, row, h):
+        """(factor on the scores, what is added to them after the cap, factor on the output)."""
+        t = 1.0
+        if self.temperature is not None:
+            t = 1.0 + self.temperature[0] * math.log((p + 1) // self.temperature[1] + 1)
+        b = None
+        if self.bias is not None:
+            b = self.bias[h].float()[torch.clamp(p - see.to(self.bias.device), max=self.bias.shape[1] - 1)]
+        return t, b, 1.0 if self.gate is None else float(torch.sigmoid(self.gate[row, h].float()))
+
+
+def _attend(qrow, keys, vals, scale, softcap, sink=None, bias=None):
+    """qrow [hd], keys/vals [n, hd], fp32.  sink: a score without key or value that joins the denominator.  bias [n]: added
+    to the scores after the cap."""
     s = (keys @ qrow) * scale
     if softcap:
         s = softcap * torch.tanh(s / softcap)
+    if bias is not None:
+        s = s + bias
     if sink is not None:
         return torch.softmax(torch.cat([s, sink.reshape(1).float()]), dim=0)[:-1] @ vals
     p = torch.softmax(s, dim=0)
@@ -257,7 +293,8 @@ def _first_seen(p, window, chunk):
 
 
 def attention_prefill(q, k, v, H, KV, hd, cu_rows, max_count, scale, softcap, window, out_dtype, row_seq=None, row_pos=None,
-                      cached=None, shape=0, wide_weights=False, chunk=0, head_scale=None, sink=None, keep=0, pin=0):
+                      cached=None, shape=0, wide_weights=False, chunk=0, head_scale=None, sink=None, keep=0, pin=0,
+                      by_position=None):
     """k, v: the step's own rows.  cached None: every sequence starts at position 0.  Else cached = (new_len, table,
     k_pool, v_pool, rows_cap): sequence i's first row stands at new_len[i] - its count, and the positions before it are
     read from the cache as it is."""
@@ -285,9 +322,10 @@ def attention_prefill(q, k, v, H, KV, hd, cu_rows, max_count, scale, softcap, wi
             p = start + r - a
             see = _positions_seen(p, window, chunk, keep).to(q.device)
             for h in range(H):
-                out[r, h * hd:(h + 1) * hd] = _attend(qf[r, h], keys[see, h // g], vals[see, h // g],
-                                                      scale * (float(head_scale[h]) if head_scale is not None else 1.0), softcap,
-                                                      None if sink is None else sink[h])
+                t, b, f = by_position.of_query(p, see, r, h) if by_position is not None else (1.0, None, 1.0)
+                out[r, h * hd:(h + 1) * hd] = f * _attend(qf[r, h], keys[see, h // g], vals[see, h // g],
+                                                          t * scale * (float(head_scale[h]) if head_scale is not None else 1.0), softcap,
+                                                          None if sink is None else sink[h], b)
     return out.to(out_dtype)
 
 
@@ -296,7 +334,7 @@ def decode_splits(n, KV, hd, keys):
 
 
 def attention_decode(q, H, KV, hd, new_len, table, k_pool, v_pool, rows_cap, scale, softcap, window, out_dtype, max_keys=None, splits=None, head_groups=None,
-                     chunk=0, head_scale=None, sink=None, keep=0, pin=0):
+                     chunk=0, head_scale=None, sink=None, keep=0, pin=0, by_position=None):
     n = q.shape[0]
     page = k_pool.shape[2]
     out = torch.zeros((n, H * hd), dtype=torch.float32, device=q.device)
@@ -304,15 +342,17 @@ def attention_decode(q, H, KV, hd, new_len, table, k_pool, v_pool, rows_cap, sca
     g = H // KV
     for i in range(n):
         p = int(new_len[i]) - 1
-        rows = _rows_of(_positions_seen(p, window, chunk, keep), rows_cap, pin).to(q.device)
+        see = _positions_seen(p, window, chunk, keep)
+        rows = _rows_of(see, rows_cap, pin).to(q.device)
         pages = table[i].long()[rows // page]
         assert (pages >= 0).all()
         keys = k_pool[pages, :, rows % page, :].float()          # [n_keys, KV, hd]
         vals = v_pool[pages, :, rows % page, :].float()
         for h in range(H):
-            out[i, h * hd:(h + 1) * hd] = _attend(qf[i, h], keys[:, h // g], vals[:, h // g],
-                                                  scale * (float(head_scale[h]) if head_scale is not None else 1.0), softcap,
-                                                  None if sink is None else sink[h])
+            t, b, f = by_position.of_query(p, see, i, h) if by_position is not None else (1.0, None, 1.0)
+            out[i, h * hd:(h + 1) * hd] = f * _attend(qf[i, h], keys[:, h // g], vals[:, h // g],
+                                                      t * scale * (float(head_scale[h]) if head_scale is not None else 1.0), softcap,
+                                                      None if sink is None else sink[h], b)
     return out.to(out_dtype)
 
 
@@ -321,7 +361,8 @@ def fuses_decode_step(dtype, H, KV, hd, k_pool):
 
 
 def attention_decode_step(qkv, H, KV, hd, inv_freq, rotary_dim, new_len, table, k_pool, v_pool, rows_cap, scale, softcap,
-                          window, out_dtype, max_keys=None, write_kv=True, splits=None, sink=None, keep=0, pin=0):
+                          window, out_dtype, max_keys=None, write_kv=True, splits=None, sink=None, keep=0, pin=0,
+                          by_position=None):
     """The fused decode step as its three parts: qkv float32 [n, (H + 2 KV) hd] (already summed over K slices),
     rotated in float32 and rounded once to the cache's dtype."""
     n = qkv.shape[0]
@@ -329,7 +370,7 @@ def attention_decode_step(qkv, H, KV, hd, inv_freq, rotary_dim, new_len, table, 
     q = _rotate(qkv[:, :H * hd].float().reshape(n, H, hd), pos, inv_freq, rotary_dim).reshape(n, H * hd).to(k_pool.dtype)
     if write_kv:
         k = _rotate(qkv[:, H * hd:(H + KV) * hd].float().reshape(n, KV, hd), pos, inv_freq, rotary_dim).to(k_pool.dtype)
-        v = qkv[:, (H + KV) * hd:].reshape(n, KV, hd).to(k_pool.dtype)
+        v = qkv[:, (H + KV) * hd:(H + 2 * KV) * hd].reshape(n, KV, hd).to(k_pool.dtype)
         page = k_pool.shape[2]
         for i in range(n):
             row = _row_of(int(pos[i]), rows_cap, pin)
@@ -337,7 +378,10 @@ def attention_decode_step(qkv, H, KV, hd, inv_freq, rotary_dim, new_len, table, 
             assert pg >= 0
             k_pool[pg, :, row % page, :] = k[i]
             v_pool[pg, :, row % page, :] = v[i]
-    return attention_decode(q, H, KV, hd, new_len, table, k_pool, v_pool, rows_cap, scale, softcap, window, out_dtype, sink=sink, keep=keep, pin=pin)
+    if by_position is not None and by_position.gate is not None:          # there the number of the gates' first column
+        by_position = ByPosition(by_position.temperature, by_position.bias, qkv[:, by_position.gate:by_position.gate + H])
+    return attention_decode(q, H, KV, hd, new_len, table, k_pool, v_pool, rows_cap, scale, softcap, window, out_dtype, sink=sink, keep=keep, pin=pin,
+                            by_position=by_position)
 
 
 class SplitRows:
@@ -349,7 +393,18 @@ class SplitRows:
         self.dtype = torch.float32
 
 
+class WeightedRows:
+    """wa * a + wb * b, not added up yet."""
+
+    def __init__(self, a, wa, b, wb):
+        self.a, self.wa, self.b, self.wb = a, wa, b, wb
+        self.shape = tuple(a.shape)
+        self.dtype = torch.float32
+
+
 def rows(r, dtype):
+    if isinstance(r, WeightedRows):
+        return r.wa * rows(r.a, torch.float32).float() + r.wb * rows(r.b, torch.float32).float()
     if isinstance(r, SplitRows):
         return r.slices.sum(0).to(dtype)
     return r
@@ -491,6 +546,21 @@ def delta_scan(q, k, v, b, a, a_log, dt_bias, state, slot_ids, cu_rows, max_coun
             u = beta[t][:, None] * (vf[t] - (S * kf[t][:, :, None]).sum(1))
             S = S + kf[t][:, :, None] * u[:, None, :]
             y[t] = (S * qf[t][:, :, None]).sum(1)
+        state[slot] = S
+    return y.reshape(M, heads * dv).float()
+
+
+def linear_scan(q, k, v, decay, state, slot_ids, cu_rows, max_count, heads, dk, dv, chunks=None):
+    """S <- decay S + v k^T, o = S q, row after row of every sequence from state[slot] [heads, dv, dk], which is left updated."""
+    M, wide = q.shape[0], state.dtype
+    qf, kf, vf = q.to(wide).reshape(M, heads, dk), k.to(wide).reshape(M, heads, dk), v.to(wide).reshape(M, heads, dv)
+    y = torch.empty((M, heads, dv), dtype=wide, device=q.device)
+    for s in range(len(cu_rows) - 1):
+        slot = int(slot_ids[s])
+        S = state[slot].clone()
+        for t in range(int(cu_rows[s]), int(cu_rows[s + 1])):
+            S = decay.to(wide)[:, None, None] * S + vf[t][:, :, None] * kf[t][:, None, :]
+            y[t] = (S * qf[t][:, None, :]).sum(-1)
         state[slot] = S
     return y.reshape(M, heads * dv).float()
 

@@ -5,3 +5,4 @@ from .lutovik import LutovikConfig   # noqa: F401
 from .besulix import BesulixConfig   # noqa: F401
 from .vogunex import VogunexConfig   # noqa: F401
 from .solulix import SolulixConfig   # noqa: F401
+from .kaderax import KaderaxConfig   # noqa: F401

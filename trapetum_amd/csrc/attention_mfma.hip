@@ -10,6 +10,10 @@
 // Scores are computed transposed, S^T = K . Q^T with v_mfma_f32_16x16x32_bf16: key rows are the A operand (a
 // lane holds 8 consecutive elements of one key: one 16-byte load), queries the B operand, and a lane ends up
 // with 4 keys of ONE query, so the softmax statistics are per-lane scalars.
+//
+// Compiled with -DTP_BY_POSITION=1 the scores may depend on positions (TpPositional in common.h): the query's temperature is a
+// factor on its scale, and a lane fetches its four keys' biases with the round's keys; a gate per head multiplies the output
+// where it is normalised.
 #include "common.h"
 #include <type_traits>
 #include "error_channel.h"
@@ -21,7 +25,12 @@
 typedef __attribute__((__vector_size__(8 * sizeof(__bf16)))) __bf16 bf16x8;
 typedef __attribute__((__vector_size__(4 * sizeof(float)))) float f32x4;
 
+#ifndef TP_BY_POSITION
+#define TP_BY_POSITION 0
+#endif
+
 namespace {
+constexpr bool BY_POSITION = TP_BY_POSITION != 0;
 constexpr int HD = TP_HD;
 constexpr int HDP = (HD + 31) / 32 * 32;       // head size padded to the product's k step
 constexpr int KSTEPS = HDP / 32;
@@ -78,6 +87,7 @@ struct DecodeArgs {
     int chunk; const float* head_scale; const float* sink;
     // the first `keep` positions stay visible behind the window; in a ring they live in the `pin` rows in front of it
     int keep, pin;
+    TpPositional by_position;
 };
 
 namespace {
@@ -149,11 +159,19 @@ attn_decode_k(DecodeArgs a) {
     auto row_in_tile = [&](int tb, int t) {                        // a row of the tile that exists, for position t of it
         return t > p ? p : (t < lo && t >= a.keep ? (lo < tb + 15 ? lo : tb + 15) : t);
     };
+    const float* bias = nullptr;                                   // of query head c of the group
+    if constexpr (BY_POSITION)
+        if (a.by_position.bias) bias = a.by_position.bias + (size_t)(kvh * G + (c < G ? c : 0)) * (a.by_position.reach + 1);
+    float bs[4] = {0.f, 0.f, 0.f, 0.f};                            // the round's biases of the lane's keys
     auto load_round = [&](int ub, bf16x8 (&kf)[DSTEPS], Frag (&vf)[VPT]) {
         const int tb = ub < kept_al ? ub : ub + gap;
         const size_t tile = tile_offset(__builtin_amdgcn_readfirstlane(tb));
         const int tk = row_in_tile(tb, tb + c);
         const bf16_t* kp = a.k_pool + tile + (size_t)(tk - tb) * HD;
+        if constexpr (BY_POSITION)
+            if (bias)
+#pragma unroll
+                for (int i = 0; i < 4; i++) bs[i] = bias[min(max(p - (tb + g * 4 + i), 0), (int)a.by_position.reach)];
 #pragma unroll
         for (int ks = 0; ks < DSTEPS; ks++) {
             const int d0 = dofs(ks, g);
@@ -275,7 +293,8 @@ attn_decode_k(DecodeArgs a) {
 #pragma unroll
         for (int e = 0; e < 8; e++) acc[qi][e] = 0.f;
     float m_run = -INFINITY, l_run = 0.f;            // of query head c, over this wave's keys so far
-    const float scale_c = a.head_scale && c < G ? a.scale * a.head_scale[kvh * G + c] : a.scale;     // lane (c, g): query head c of the group
+    float scale_c = a.head_scale && c < G ? a.scale * a.head_scale[kvh * G + c] : a.scale;     // lane (c, g): query head c of the group
+    if constexpr (BY_POSITION) scale_c *= query_temperature(a.by_position, p);
     const float soc = a.cap > 0.f ? scale_c / a.cap : 0.f;
 
     for (int tb = tb0; tb < t_end; tb += ROUND) {
@@ -289,7 +308,7 @@ attn_decode_k(DecodeArgs a) {
         for (int i = 0; i < 4; i++) {
             const int u = tb + g * 4 + i, t = u < kept_al ? u : u + gap;
             const bool ok = (t >= lo || t < a.keep) && u < t_end;
-            s[i] = ok ? score_of(s[i], scale_c, a.cap, soc) : -INFINITY;
+            s[i] = ok ? score_of(s[i], scale_c, a.cap, soc) + (BY_POSITION ? bs[i] : 0.f) : -INFINITY;
             mx = fmaxf(mx, s[i]);
         }
         mx = fmaxf(mx, __shfl_xor(mx, 16, 64));
@@ -365,7 +384,9 @@ attn_decode_k(DecodeArgs a) {
             const int head = kvh * G + qi;
             if (a.nsplit == 1) {
                 if (a.sink) den += __expf(a.sink[head] - mx);                 // (the slice holds the query's own key: mx is finite)
-                a.out[((size_t)seq * a.H + head) * HD + tid] = f32_to_bf16(num / den);
+                float o = num / den;
+                if constexpr (BY_POSITION) if (a.by_position.gate) o *= head_gate(a.by_position, seq, head);
+                a.out[((size_t)seq * a.H + head) * HD + tid] = f32_to_bf16(o);
             } else {
                 const size_t at = ((size_t)seq * a.H + head) * a.nsplit + split;
                 a.ws_o[at * HD + tid] = num;
@@ -381,7 +402,7 @@ attn_decode_k(DecodeArgs a) {
 // unwritten: its weight is zero and the value is replaced by zero).
 __global__ void __launch_bounds__(256)
 attn_decode_combine_k(const float* __restrict__ ws_o, const float* __restrict__ ws_ml, int nsplit,
-                      bf16_t* __restrict__ out, const float* __restrict__ sink, int H) {
+                      bf16_t* __restrict__ out, const float* __restrict__ sink, int H, TpPositional by_position) {
     __shared__ float w_lds[128];
     const size_t at = (size_t)blockIdx.x * nsplit;               // blockIdx.x = sequence * heads + head
     const int tid = threadIdx.x;
@@ -409,6 +430,7 @@ attn_decode_combine_k(const float* __restrict__ ws_o, const float* __restrict__ 
         float den = 0.f;
         for (int s = 0; s < nsplit; s++) den += w_lds[s];
         if (sink) den += __expf(sink[blockIdx.x % H] - mx);       // (some slice holds the query's own key: mx is finite)
+        if constexpr (BY_POSITION) if (by_position.gate) den /= head_gate(by_position, blockIdx.x / H, blockIdx.x % H);
         __builtin_amdgcn_wave_barrier();
         w_lds[tid] = w0 / den;
         w_lds[tid + 64] = w1 / den;
@@ -467,20 +489,29 @@ static int decode_launch(DecodeArgs a, int n_seq, void* workspace, hipStream_t s
     else attn_decode_k<16><<<grid, DTH, 0, s>>>(a);
     if (int rc = tp_check_launch("attention decode")) return rc;
     if (a.nsplit > 1) {
-        attn_decode_combine_k<<<n_seq * a.H, HD < 64 ? 64 : HD, 0, s>>>(a.ws_o, a.ws_ml, a.nsplit, a.out, a.sink, a.H);
+        attn_decode_combine_k<<<n_seq * a.H, HD < 64 ? 64 : HD, 0, s>>>(a.ws_o, a.ws_ml, a.nsplit, a.out, a.sink, a.H, a.by_position);
         return tp_check_launch("attention decode (combine)");
     }
+    return 0;
+}
+
+static int take_positional(DecodeArgs& a, const TpPositional* by_position) {
+    if (!by_position) return 0;
+    TP_REQUIRE(BY_POSITION, "attention decode: this library's kernels know no scores by position");
+    TP_REQUIRE(tp_positional_ok(by_position), "attention decode: a bias, a temperature or a gate that does not fit");
+    a.by_position = *by_position;
     return 0;
 }
 
 extern "C" int tp_attn_decode(const void* q, long q_stride, int n_seq, int H, int KV, const int* new_len,
                               const int* table, int table_w, const void* k_pool, const void* v_pool, int page,
                               int rows_cap, float scale, float cap, int window, int chunk, const float* head_scale,
-                              const float* sink, int keep, int pin, void* out, void* workspace, int nsplit, void* stream) {
+                              const float* sink, int keep, int pin, const TpPositional* by_position, void* out, void* workspace, int nsplit, void* stream) {
     TP_REQUIRE(q_stride % 8 == 0 && (uintptr_t)q % 16 == 0, "attention decode: query rows must be 16-byte aligned");
     DecodeArgs a{(const bf16_t*)q, q_stride, H, KV, new_len, table, table_w, (bf16_t*)k_pool, (bf16_t*)v_pool,
                  page, rows_cap, scale, cap, window, (bf16_t*)out, nullptr, nullptr, nsplit,
-                 nullptr, 0, 1, 0, 0, nullptr, 0, 0, 0, chunk, head_scale, sink, keep, pin};
+                 nullptr, 0, 1, 0, 0, nullptr, 0, 0, 0, chunk, head_scale, sink, keep, pin, TpPositional{}};
+    if (int rc = take_positional(a, by_position)) return rc;
     return decode_launch(a, n_seq, workspace, (hipStream_t)stream);
 }
 
@@ -489,12 +520,12 @@ extern "C" int tp_attn_decode(const void* q, long q_stride, int n_seq, int H, in
 // block's worth of weighted sums, instead of one block forming all of them.
 extern "C" int tp_attn_decode_shared(const void* q, long q_stride, int n_seq, int H, int KV, int pool_kv, const int* new_len,
                                      const int* table, int table_w, const void* k_pool, const void* v_pool, int page,
-                                     int rows_cap, float scale, float cap, int window, void* out, void* workspace,
+                                     int rows_cap, float scale, float cap, int window, const float* sink, void* out, void* workspace,
                                      int nsplit, void* stream) {
     TP_REQUIRE(q_stride % 8 == 0 && (uintptr_t)q % 16 == 0, "attention decode: query rows must be 16-byte aligned");
     DecodeArgs a{(const bf16_t*)q, q_stride, H, KV, new_len, table, table_w, (bf16_t*)k_pool, (bf16_t*)v_pool,
                  page, rows_cap, scale, cap, window, (bf16_t*)out, nullptr, nullptr, nsplit,
-                 nullptr, 0, 1, 0, 0, nullptr, 0, 0, pool_kv};
+                 nullptr, 0, 1, 0, 0, nullptr, 0, 0, pool_kv, 0, nullptr, sink, 0, 0, TpPositional{}};
     return decode_launch(a, n_seq, workspace, (hipStream_t)stream);
 }
 
@@ -505,7 +536,7 @@ extern "C" int tp_attn_decode_fused(const void* qkv, int qkv_dtype, int n_slices
                                     const float* inv_freq, int rot, int write_kv,
                                     int n_seq, int H, int KV, const int* new_len, const int* table, int table_w,
                                     void* k_pool, void* v_pool, int page, int rows_cap, float scale, float cap,
-                                    int window, const float* sink, int keep, int pin, void* out, void* workspace, int nsplit, void* stream) {
+                                    int window, const float* sink, int keep, int pin, const TpPositional* by_position, void* out, void* workspace, int nsplit, void* stream) {
     TP_REQUIRE(qkv, "attention decode (fused): no projections");
     TP_REQUIRE(qkv_dtype == TP_BF16 || qkv_dtype == TP_F32, "attention decode (fused): projections of dtype %d", qkv_dtype);
     TP_REQUIRE(n_slices >= 1 && (n_slices == 1 || qkv_dtype == TP_F32), "attention decode (fused): %d slices must be float32", n_slices);
@@ -514,6 +545,7 @@ extern "C" int tp_attn_decode_fused(const void* qkv, int qkv_dtype, int n_slices
     TP_REQUIRE(row_stride >= (long)(H + (write_kv ? 2 * KV : 0)) * HD, "attention decode (fused): rows of %ld elements are too short", row_stride);
     DecodeArgs a{nullptr, 0, H, KV, new_len, table, table_w, (bf16_t*)k_pool, (bf16_t*)v_pool,
                  page, rows_cap, scale, cap, window, (bf16_t*)out, nullptr, nullptr, nsplit,
-                 qkv, qkv_dtype == TP_F32 ? 1 : 0, n_slices, slice_stride, row_stride, inv_freq, rot, write_kv, 0, 0, nullptr, sink, keep, pin};
+                 qkv, qkv_dtype == TP_F32 ? 1 : 0, n_slices, slice_stride, row_stride, inv_freq, rot, write_kv, 0, 0, nullptr, sink, keep, pin, TpPositional{}};
+    if (int rc = take_positional(a, by_position)) return rc;
     return decode_launch(a, n_seq, workspace, (hipStream_t)stream);
 }

@@ -31,6 +31,11 @@
 // changed nothing there: fragments three and four ahead instead of two, a second chain of score accumulation,
 // half or all of the queries in LDS, the block's upper waves running half a round behind the lower ones (slower:
 // the halves differ in length and every wave waits for the slowest at both barriers).
+//
+// Compiled with -DTP_BY_POSITION=1 the scores may depend on positions (TpPositional in common.h).  The query's temperature is
+// a factor on a lane's scale.  A tile whose every key is `reach` or more positions behind every query of the wave adds one
+// number per head; in the few tiles nearer than that a lane asks for its 16 keys' biases ahead of the round's first barrier,
+// while the V tile is on its way (neighbouring lanes read neighbouring entries of one table).
 #include "common.h"
 
 #ifndef TP_HD
@@ -57,9 +62,15 @@ struct PrefillArgs {
     const float* sink;                        // [H] or null: a score without key or value that joins every softmax's sum once
     int keep, pin;                            // the first `keep` positions stay visible behind the window; rows of the cache in front of its ring
     bf16_t* out;
+    TpPositional by_position;
 };
 
+#ifndef TP_BY_POSITION
+#define TP_BY_POSITION 0
+#endif
+
 namespace {
+constexpr bool BY_POSITION = TP_BY_POSITION != 0;
 constexpr int HD = TP_HD;
 static_assert(HD % 16 == 0 && HD >= 16 && HD <= 256, "head_dim must be a multiple of 16 up to 256");
 constexpr int KS16 = HD / 16;                 // k steps of the first product
@@ -243,7 +254,16 @@ attn_prefill_k(PrefillArgs a) {
 #pragma unroll
         for (int e = 0; e < 16; e++) o[dt][e] = 0.f;
     float m_ref = -INFINITY, l_i = 0.f;                            // in units of log 2; l_i: this lane's 16 keys of every tile
-    const float scale_h = a.head_scale ? a.scale * a.head_scale[h] : a.scale;
+    float scale_h = a.head_scale ? a.scale * a.head_scale[h] : a.scale;
+    const float* bias = nullptr;
+    float bias_far = 0.f;                                          // in units of log 2, like the scores
+    if constexpr (BY_POSITION) {
+        scale_h *= query_temperature(a.by_position, max(qpos, 0));
+        if (a.by_position.bias) {
+            bias = a.by_position.bias + (size_t)h * (a.by_position.reach + 1);
+            bias_far = bias[a.by_position.reach] * LOG2E;
+        }
+    }
     const float tanh_in = a.cap > 0.f ? 2.f * LOG2E * scale_h / a.cap : 0.f, cap2 = a.cap * LOG2E, scale2 = scale_h * LOG2E;
     // keys a query sees behind it, itself included: the window, and what its chunk holds up to it
     unsigned win = a.window > 0 ? (unsigned)a.window : 0x7fffffffu;
@@ -305,6 +325,20 @@ attn_prefill_k(PrefillArgs a) {
 #pragma unroll
                 for (int j = 0; j < 16; j++) sc[j] = s[j] * scale2;
             }
+            if constexpr (BY_POSITION)
+                if (bias) {
+                    if (qw0 - (kt + 31) < (int)a.by_position.reach) {      // (wave-uniform) some key is nearer than `reach` to some query
+                        const int d0 = qpos - kt - 4 * hi;
+                        float bs[16];
+#pragma unroll
+                        for (int j = 0; j < 16; j++) bs[j] = bias[min(max(d0 - 8 * (j >> 2) - (j & 3), 0), (int)a.by_position.reach)];
+#pragma unroll
+                        for (int j = 0; j < 16; j++) sc[j] = __builtin_fmaf(bs[j], LOG2E, sc[j]);
+                    } else {
+#pragma unroll
+                        for (int j = 0; j < 16; j++) sc[j] += bias_far;
+                    }
+                }
         }
         // The barrier stands in the middle of the softmax, so that both loads have about half a round to land: here
         // this round's V tile has landed and every wave has read the K tile, whose successor may come.
@@ -432,7 +466,8 @@ attn_prefill_k(PrefillArgs a) {
     if (!q_ok) return;
     float total = pair_sum(l_i);
     if (a.sink) total += exp2_fast(a.sink[h] * LOG2E - m_ref);       // (a query sees its own key at least: m_ref is finite)
-    const float inv = 1.f / total;
+    float inv = 1.f / total;
+    if constexpr (BY_POSITION) if (a.by_position.gate) inv *= head_gate(a.by_position, (size_t)(row0 + qpos - start), h);
     // lane: head elements dt * 32 + 8 (j / 4) + 4 hi + j % 4 of query `col`: four neighbours per store
     bf16_t* orow = a.out + ((size_t)(row0 + qpos - start) * a.H + h) * HD + 4 * hi;
 #pragma unroll
@@ -473,7 +508,7 @@ extern "C" int tp_attn_prefill(const void* q, long q_stride, const void* k, long
                                int M, int H, int KV, const int* cu_rows, int n_seq, int max_count,
                                const int* new_len, const int* table, int table_w, const void* k_pool, const void* v_pool,
                                int page, int rows_cap, float scale, float cap, int window, int chunk, const float* head_scale,
-                               const float* sink, int keep, int pin, void* out, int shape, void* stream) {
+                               const float* sink, int keep, int pin, const TpPositional* by_position, void* out, int shape, void* stream) {
     TP_REQUIRE(M > 0 && H > 0 && KV > 0 && n_seq > 0 && max_count > 0, "attention prefill: empty shape");
     TP_REQUIRE(H % KV == 0, "attention: %d query heads are no multiple of %d kv heads", H, KV);
     TP_REQUIRE(q_stride % 8 == 0 && k_stride % 8 == 0 && v_stride % 8 == 0 && (uintptr_t)q % 16 == 0 &&
@@ -491,8 +526,11 @@ extern "C" int tp_attn_prefill(const void* q, long q_stride, const void* k, long
         TP_REQUIRE(rows_cap == 0 || (reach > 0 && reach <= rows_cap - pin), "attention prefill: a reach of %d keys (window %d, chunk %d) does not fit a ring of %d rows", reach, window, chunk, rows_cap - pin);
         TP_REQUIRE((uintptr_t)k_pool % 16 == 0 && (uintptr_t)v_pool % 16 == 0, "attention prefill: the pools must be 16-byte aligned");
     }
+    TP_REQUIRE(BY_POSITION || !by_position, "attention prefill: this library's kernels know no scores by position");
+    TP_REQUIRE(tp_positional_ok(by_position), "attention prefill: a bias, a temperature or a gate that does not fit");
     const int G = H / KV;
     PrefillArgs a{};
+    if (by_position) a.by_position = *by_position;
     a.q = (const bf16_t*)q; a.q_stride = q_stride; a.k = (const bf16_t*)k; a.k_stride = k_stride; a.v = (const bf16_t*)v; a.v_stride = v_stride;
     a.cu_rows = cu_rows; a.new_len = new_len; a.table = table; a.table_w = table_w;
     a.k_pool = (const bf16_t*)k_pool; a.v_pool = (const bf16_t*)v_pool;

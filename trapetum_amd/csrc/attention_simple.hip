@@ -9,7 +9,8 @@
 // window W hides keys with p - t >= W (none there).  Beyond the reference: with chunks of C positions the query at p
 // sees only keys from floor(p / C) C on; a head may have a temperature that multiplies its scores and a sink, a score
 // without key or value whose exponential joins the denominator once, after the keys.  With `keep` the first keep positions
-// of a sequence stay visible behind the window; in a ring they live in the `pin` rows in front of it.
+// of a sequence stay visible behind the window; in a ring they live in the `pin` rows in front of it.  A temperature of the
+// query's position, a bias per distance and a gate per head come with TpPositional (common.h).
 #include "common.h"
 
 struct AttnSimpleArgs {
@@ -24,6 +25,7 @@ struct AttnSimpleArgs {
     void* out;
     int H, KV, hd; float scale, cap; int window; int paged;
     int chunk; const float* head_scale; const float* sink;        // 0 and null: none
+    TpPositional by_position;
     int keep, pin;                                       // positions seen beside the window; rows of the cache in front of its ring
 };
 
@@ -42,7 +44,8 @@ attn_simple_k(AttnSimpleArgs a) {
     }
     int lo = a.window > 0 ? max(0, p - a.window + 1) : 0;
     if (a.chunk > 0) lo = max(lo, p / a.chunk * a.chunk);
-    const float scale = a.head_scale ? a.scale * a.head_scale[h] : a.scale;
+    const float scale = (a.head_scale ? a.scale * a.head_scale[h] : a.scale) * query_temperature(a.by_position, p);
+    const float* bias = a.by_position.bias ? a.by_position.bias + (size_t)h * (a.by_position.reach + 1) : nullptr;
     const T* q = (const T*)a.q + (size_t)r * a.q_stride + (size_t)h * a.hd;
     float qv[NJ], o[NJ];
 #pragma unroll
@@ -80,12 +83,13 @@ attn_simple_k(AttnSimpleArgs a) {
             vv[j] = d < a.hd ? vx : 0.f;
         }
     };
-    auto use = [&](const float (&kk)[NJ], const float (&vv)[NJ]) {
+    auto use = [&](int i, const float (&kk)[NJ], const float (&vv)[NJ]) {
         float part = 0.f;
 #pragma unroll
         for (int j = 0; j < NJ; j++) part = fmaf(qv[j], kk[j], part);
         float s = wave_sum(part) * scale;
         if (a.cap > 0.f) s = softcap_f(s, a.cap);
+        if (bias) s += bias[min(p - at(i), (int)a.by_position.reach)];
         const float m_new = fmaxf(m, s);
         const float alpha = expf(m - m_new), pr = expf(s - m_new);
         l = l * alpha + pr;
@@ -98,13 +102,13 @@ attn_simple_k(AttnSimpleArgs a) {
     fetch(1, k1, v1);
     for (int i = 0; i < n_keys; i += 3) {
         fetch(i + 2, k2, v2);
-        use(k0, v0);
+        use(i, k0, v0);
         if (i + 1 >= n_keys) break;
         fetch(i + 3, k0, v0);
-        use(k1, v1);
+        use(i + 1, k1, v1);
         if (i + 2 >= n_keys) break;
         fetch(i + 4, k1, v1);
-        use(k2, v2);
+        use(i + 2, k2, v2);
     }
     if (a.sink) {
         const float sk = a.sink[h], m_new = fmaxf(m, sk);
@@ -114,7 +118,7 @@ attn_simple_k(AttnSimpleArgs a) {
         for (int j = 0; j < NJ; j++) o[j] *= alpha;
     }
     T* out = (T*)a.out + ((size_t)r * a.H + h) * a.hd;
-    const float inv = 1.f / l;
+    const float inv = (a.by_position.gate ? head_gate(a.by_position, r, h) : 1.f) / l;
 #pragma unroll
     for (int j = 0; j < NJ; j++) {
         const int d = lane + 64 * j;
@@ -146,7 +150,7 @@ extern "C" int tp_attn_simple_prefill(const void* q, long q_stride, const void* 
                                       const int* row_pos, const int* new_len, const int* table, int table_w,
                                       const void* k_pool, const void* v_pool, int page, int rows_cap,
                                       float scale, float cap, int window, int chunk, const float* head_scale, const float* sink,
-                                      int keep, int pin, void* out, void* stream) {
+                                      int keep, int pin, const TpPositional* by_position, void* out, void* stream) {
     TP_REQUIRE(chunk >= 0, "attention: chunks of %d positions", chunk);
     TP_REQUIRE(!new_len || (table && k_pool && v_pool && page > 0 && table_w > 0), "attention: cached positions need the page table and the pools");
     AttnSimpleArgs a{};
@@ -157,13 +161,15 @@ extern "C" int tp_attn_simple_prefill(const void* q, long q_stride, const void* 
     a.out = out; a.H = H; a.KV = KV; a.hd = hd; a.scale = scale; a.cap = cap; a.window = window; a.paged = 0;
     a.chunk = chunk; a.head_scale = head_scale; a.sink = sink;
     a.keep = keep; a.pin = pin;
+    TP_REQUIRE(tp_positional_ok(by_position), "attention: a bias, a temperature or a gate that does not fit");
+    if (by_position) a.by_position = *by_position;
     return launch(a, dtype, M, (hipStream_t)stream);
 }
 
 extern "C" int tp_attn_simple_decode(const void* q, long q_stride, int dtype, int n_seq, int H, int KV, int hd,
                                      const int* new_len, const int* table, int table_w, const void* k_pool,
                                      const void* v_pool, int page, int rows_cap, float scale, float cap, int window,
-                                     int chunk, const float* head_scale, const float* sink, int keep, int pin, void* out, void* stream) {
+                                     int chunk, const float* head_scale, const float* sink, int keep, int pin, const TpPositional* by_position, void* out, void* stream) {
     TP_REQUIRE(chunk >= 0, "attention: chunks of %d positions", chunk);
     TP_REQUIRE(page > 0 && table_w > 0, "attention: page size %d, table width %d", page, table_w);
     AttnSimpleArgs a{};
@@ -172,5 +178,7 @@ extern "C" int tp_attn_simple_decode(const void* q, long q_stride, int dtype, in
     a.out = out; a.H = H; a.KV = KV; a.hd = hd; a.scale = scale; a.cap = cap; a.window = window; a.paged = 1;
     a.chunk = chunk; a.head_scale = head_scale; a.sink = sink;
     a.keep = keep; a.pin = pin;
+    TP_REQUIRE(tp_positional_ok(by_position), "attention: a bias, a temperature or a gate that does not fit");
+    if (by_position) a.by_position = *by_position;
     return launch(a, dtype, n_seq, (hipStream_t)stream);
 }

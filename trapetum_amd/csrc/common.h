@@ -83,6 +83,30 @@ __device__ __forceinline__ float gelu_tanh_fast(float g) {
     return g * __builtin_amdgcn_rcpf(1.f + __builtin_amdgcn_exp2f(g * __builtin_fmaf(C3, g * g, C1)));
 }
 
+// ---- attention whose scores and outputs depend on positions and gates ------------------------------------------------------
+// Handed to the attention kernels by pointer (null: none of it).  The scores of the query at position p are multiplied by
+// 1 + temp_coef ln(floor((p + 1) / temp_every) + 1) (temp_every 0: not at all); after the cap, head h's score on the key at
+// distance n gets bias[h][min(n, reach)] added; head h's output of row r is multiplied by sigmoid(gate[r][h]), gate being
+// rows of either dtype, float32 ones possibly in K slices of a product that are added in slice order.
+struct TpPositional {
+    const float* bias; long reach;
+    const void* gate; long gate_f32, gate_slices, gate_slice_stride, gate_stride;
+    float temp_coef; int temp_every;
+};
+__device__ __forceinline__ float query_temperature(const TpPositional& s, int p) {
+    return s.temp_every > 0 ? 1.f + s.temp_coef * logf((float)((p + 1) / s.temp_every + 1)) : 1.f;
+}
+__device__ __forceinline__ float head_gate(const TpPositional& s, size_t row, int h) {
+    const size_t at = row * s.gate_stride + h;
+    float g = 0.f;
+    if (s.gate_f32) for (int i = 0; i < (int)s.gate_slices; i++) g += ((const float*)s.gate)[i * s.gate_slice_stride + at];
+    else g = bf16_to_f32(((const bf16_t*)s.gate)[at]);
+    return 1.f / (1.f + expf(-g));
+}
+static inline bool tp_positional_ok(const TpPositional* s) {
+    return !s || ((!s->bias || s->reach >= 0) && s->temp_every >= 0 && (!s->gate || (s->gate_slices >= 1 && (s->gate_f32 || s->gate_slices == 1))));
+}
+
 // ---- gate activations of a gated product -----------------------------------------------------------------------
 // The activations offered are of one form, act(g) = g / (1 + 2^(g (c1 + c3 g^2))): gelu-tanh (above) with
 // c1 = -2 * 0.7978845608 * log2(e), c3 = c1 * 0.044715, and SiLU, g / (1 + e^-g), with c1 = -log2(e), c3 = 0.  The

@@ -33,12 +33,13 @@ extern "C" int tp_embed_rows(const int* tokens, const void* table, int dtype, fl
 // A norm over `groups` equal consecutive parts of a row is the same norm over rows of the part's length, `groups`
 // times as many, part g of a row taking the g-th stretch of the gain: a block's row is blockIdx.x, its stretch
 // blockIdx.x % groups, and D is the part's length.
+// x_stride: elements from one row of x to the next (a view of wider rows; the output is contiguous).
 template <typename TI, typename TO>
-__global__ void rms_norm_k(const TI* __restrict__ x, const float* __restrict__ gain, float eps,
+__global__ void rms_norm_k(const TI* __restrict__ x, long x_stride, const float* __restrict__ gain, float eps,
                            TO* __restrict__ out, int D, int groups) {
     __shared__ float red[16];
     gain += (size_t)(blockIdx.x % groups) * D;
-    const TI* xr = x + (size_t)blockIdx.x * D;
+    const TI* xr = x + (size_t)(blockIdx.x / groups) * x_stride + (size_t)(blockIdx.x % groups) * D;
     TO* orow = out + (size_t)blockIdx.x * D;
     float ss = 0.f;
     for (int i = threadIdx.x; i < D; i += blockDim.x) { float v = ld_f32(xr + i); ss += v * v; }
@@ -50,10 +51,10 @@ __global__ void rms_norm_k(const TI* __restrict__ x, const float* __restrict__ g
 // the same for rows of at most 256 * EPT elements: every element is read once and kept in registers
 template <typename TI, typename TO, int EPT, int NTH>
 __global__ void __launch_bounds__(NTH)
-rms_norm_reg_k(const TI* __restrict__ x, const float* __restrict__ gain, float eps, TO* __restrict__ out, int D, int groups) {
+rms_norm_reg_k(const TI* __restrict__ x, long x_stride, const float* __restrict__ gain, float eps, TO* __restrict__ out, int D, int groups) {
     __shared__ float red[16];
     gain += (size_t)(blockIdx.x % groups) * D;
-    const TI* xr = x + (size_t)blockIdx.x * D;
+    const TI* xr = x + (size_t)(blockIdx.x / groups) * x_stride + (size_t)(blockIdx.x % groups) * D;
     TO* orow = out + (size_t)blockIdx.x * D;
     float v[EPT], gn[EPT];
     float ss = 0.f;
@@ -75,25 +76,26 @@ rms_norm_reg_k(const TI* __restrict__ x, const float* __restrict__ gain, float e
 }
 
 template <typename TI, typename TO>
-static void rms_norm_launch(const void* x, const float* gain, float eps, void* out, int M, int D, int groups, hipStream_t s) {
-    if (D <= 256 * 2) rms_norm_reg_k<TI, TO, 2, 256><<<M, 256, 0, s>>>((const TI*)x, gain, eps, (TO*)out, D, groups);
-    else if (M <= 128 && D <= 1024 * 4) rms_norm_reg_k<TI, TO, 4, 1024><<<M, 1024, 0, s>>>((const TI*)x, gain, eps, (TO*)out, D, groups);
-    else if (D <= 256 * 4) rms_norm_reg_k<TI, TO, 4, 256><<<M, 256, 0, s>>>((const TI*)x, gain, eps, (TO*)out, D, groups);
-    else if (D <= 256 * 12) rms_norm_reg_k<TI, TO, 12, 256><<<M, 256, 0, s>>>((const TI*)x, gain, eps, (TO*)out, D, groups);
-    else if (D <= 1024 * 8) rms_norm_reg_k<TI, TO, 8, 1024><<<M, 1024, 0, s>>>((const TI*)x, gain, eps, (TO*)out, D, groups);
-    else rms_norm_k<TI, TO><<<M, 256, 0, s>>>((const TI*)x, gain, eps, (TO*)out, D, groups);
+static void rms_norm_launch(const void* x, long xs, const float* gain, float eps, void* out, int M, int D, int groups, hipStream_t s) {
+    if (D <= 256 * 2) rms_norm_reg_k<TI, TO, 2, 256><<<M, 256, 0, s>>>((const TI*)x, xs, gain, eps, (TO*)out, D, groups);
+    else if (M <= 128 && D <= 1024 * 4) rms_norm_reg_k<TI, TO, 4, 1024><<<M, 1024, 0, s>>>((const TI*)x, xs, gain, eps, (TO*)out, D, groups);
+    else if (D <= 256 * 4) rms_norm_reg_k<TI, TO, 4, 256><<<M, 256, 0, s>>>((const TI*)x, xs, gain, eps, (TO*)out, D, groups);
+    else if (D <= 256 * 12) rms_norm_reg_k<TI, TO, 12, 256><<<M, 256, 0, s>>>((const TI*)x, xs, gain, eps, (TO*)out, D, groups);
+    else if (D <= 1024 * 8) rms_norm_reg_k<TI, TO, 8, 1024><<<M, 1024, 0, s>>>((const TI*)x, xs, gain, eps, (TO*)out, D, groups);
+    else rms_norm_k<TI, TO><<<M, 256, 0, s>>>((const TI*)x, xs, gain, eps, (TO*)out, D, groups);
 }
 
-extern "C" int tp_rms_norm(const void* x, int in_dtype, const float* gain, float eps, void* out, int out_dtype,
+extern "C" int tp_rms_norm(const void* x, long x_stride, int in_dtype, const float* gain, float eps, void* out, int out_dtype,
                            int M, int D, int groups, void* stream) {
     TP_REQUIRE(M > 0 && D > 0, "rms_norm: empty shape M=%d D=%d", M, D);
     TP_REQUIRE(groups > 0 && D % groups == 0, "rms_norm: rows of %d elements cannot be cut into %d equal groups", D, groups);
+    TP_REQUIRE(x_stride >= D, "rms_norm: rows of %d elements, %ld apart", D, x_stride);
     M *= groups; D /= groups;
     hipStream_t s = (hipStream_t)stream;
-    if (in_dtype == TP_F32 && out_dtype == TP_F32) rms_norm_launch<float, float>(x, gain, eps, out, M, D, groups, s);
-    else if (in_dtype == TP_F32 && out_dtype == TP_BF16) rms_norm_launch<float, bf16_t>(x, gain, eps, out, M, D, groups, s);
-    else if (in_dtype == TP_BF16 && out_dtype == TP_F32) rms_norm_launch<bf16_t, float>(x, gain, eps, out, M, D, groups, s);
-    else if (in_dtype == TP_BF16 && out_dtype == TP_BF16) rms_norm_launch<bf16_t, bf16_t>(x, gain, eps, out, M, D, groups, s);
+    if (in_dtype == TP_F32 && out_dtype == TP_F32) rms_norm_launch<float, float>(x, x_stride, gain, eps, out, M, D, groups, s);
+    else if (in_dtype == TP_F32 && out_dtype == TP_BF16) rms_norm_launch<float, bf16_t>(x, x_stride, gain, eps, out, M, D, groups, s);
+    else if (in_dtype == TP_BF16 && out_dtype == TP_F32) rms_norm_launch<bf16_t, float>(x, x_stride, gain, eps, out, M, D, groups, s);
+    else if (in_dtype == TP_BF16 && out_dtype == TP_BF16) rms_norm_launch<bf16_t, bf16_t>(x, x_stride, gain, eps, out, M, D, groups, s);
     else return tp_fail("rms_norm: unknown dtypes %d -> %d", in_dtype, out_dtype);
     return tp_check_launch("rms_norm");
 }
@@ -356,15 +358,20 @@ extern "C" int tp_add_rms_norm(float* stream, const void* rows, int rows_dtype, 
     return tp_check_launch("add_rms_norm");
 }
 
-// ---- stream += a + b + vec + origin; out = norm(stream) --------------------------------------------------------------
+// ---- stream += wa a + wb b + vec + origin; out = norm(stream) --------------------------------------------------------------
 // For a block whose two sub-layers read one norm: their rows are added to the stream together.  a and b: rows of either
 // dtype, or float32 K slices of a product (added in slice order); b may be null, and a too (then only what follows is
 // added).  vec [D] and origin [M, D] (float32, or null) are what stands between two layers of a model: a vector that
-// every row gets, and earlier rows of the stream.  The sums are float32.  One block a row; PC: elements a lane takes at a
-// time (4 where every operand allows it).
+// every row gets, and earlier rows of the stream.  The sums are float32.  wa and wb are constants of the model (1: the rows as
+// they are).  With `fresh` the stream's own values are replaced, not added to.  With `stack` there is no norm: what leaves,
+// beside the stream, are the operand rows of a product over [stream | origin]: float32 [v | o] of 2 D elements, or bfloat16
+// [v1 | v2 | o1 (| o2)] with v1 = bf16(v) and v2 = bf16(v - v1) (likewise o), which keep 16 bits of the float32 values
+// through a product whose matrix stands as often side by side; origin is not added then.  One block a row; PC: elements a
+// lane takes at a time (4 where every operand allows it).
 struct JoinArgs {
     float* stream; const void* a; int a_f32, a_slices; long a_stride; const void* b; int b_f32, b_slices; long b_stride;
     const float* vec; const float* origin; const float* gain; float eps; void* out; int D;
+    float wa, wb; int fresh; void* stack; int origin_terms;
 };
 
 template <int PC>
@@ -404,16 +411,46 @@ join_rms_norm_k(JoinArgs x) {
         const int i = (threadIdx.x + j * NTH) * PC;
         const bool ok = i < D;
         const int ic = ok ? i : 0;
-        ld_piece<PC>(x.stream + row + ic, v[j]);
+        if (x.fresh) {
+#pragma unroll
+            for (int e = 0; e < PC; e++) v[j][e] = 0.f;
+        } else ld_piece<PC>(x.stream + row + ic, v[j]);
         if (x.gain) ld_piece<PC>(x.gain + ic, gn[j]);
         float more[PC];
 #pragma unroll
         for (int e = 0; e < PC; e++) more[e] = 0.f;
         if (x.a) add_rows_piece<PC>(x.a, x.a_f32, x.a_slices, x.a_stride, row + ic, more);
-        if (x.b) add_rows_piece<PC>(x.b, x.b_f32, x.b_slices, x.b_stride, row + ic, more);
+        if (x.wa == 1.f && x.wb == 1.f) {
+            if (x.b) add_rows_piece<PC>(x.b, x.b_f32, x.b_slices, x.b_stride, row + ic, more);
+        } else {
+            float other[PC];
+#pragma unroll
+            for (int e = 0; e < PC; e++) other[e] = 0.f;
+            if (x.b) add_rows_piece<PC>(x.b, x.b_f32, x.b_slices, x.b_stride, row + ic, other);
+#pragma unroll
+            for (int e = 0; e < PC; e++) more[e] = __builtin_fmaf(x.wb, other[e], x.wa * more[e]);
+        }
 #pragma unroll
         for (int e = 0; e < PC; e++) v[j][e] += more[e];
-        if (x.origin) {
+        if (x.stack) {
+            if (!ok) continue;
+            float o[PC];
+            ld_piece<PC>(x.origin + row + ic, o);
+            if constexpr (std::is_same<T, float>::value) {
+                T* at = (T*)x.stack + 2 * row + i;
+                if constexpr (PC == 4) { st4(at, v[j]); st4(at + D, o); } else { at[0] = v[j][0]; at[D] = o[0]; }
+            } else {
+                T* at = (T*)x.stack + (size_t)blockIdx.x * (2 + x.origin_terms) * D + i;
+                float lo[PC], ol[PC];
+#pragma unroll
+                for (int e = 0; e < PC; e++) {
+                    lo[e] = v[j][e] - bf16_to_f32(f32_to_bf16(v[j][e]));
+                    ol[e] = o[e] - bf16_to_f32(f32_to_bf16(o[e]));
+                }
+                if constexpr (PC == 4) { st4(at, v[j]); st4(at + D, lo); st4(at + 2 * D, o); if (x.origin_terms > 1) st4(at + 3 * D, ol); }
+                else { st_f32(at, v[j][0]); st_f32(at + D, lo[0]); st_f32(at + 2 * D, o[0]); if (x.origin_terms > 1) st_f32(at + 3 * D, ol[0]); }
+            }
+        } else if (x.origin) {
             float t[PC];
             ld_piece<PC>(x.origin + row + ic, t);
 #pragma unroll
@@ -448,7 +485,7 @@ join_rms_norm_k(JoinArgs x) {
 template <typename T>
 static int join_launch(const JoinArgs& x, int M, hipStream_t s) {
     const auto al = [](const void* p) { return (uintptr_t)p % 16 == 0; };
-    const bool wide = x.D % 4 == 0 && x.a_stride % 4 == 0 && x.b_stride % 4 == 0 && al(x.stream) && al(x.a) && al(x.b) && al(x.vec) && al(x.origin) && al(x.gain) && al(x.out);
+    const bool wide = x.D % 4 == 0 && x.a_stride % 4 == 0 && x.b_stride % 4 == 0 && al(x.stream) && al(x.a) && al(x.b) && al(x.vec) && al(x.origin) && al(x.gain) && al(x.out) && al(x.stack);
     const int D = x.D;
 #define TP_JOIN(PC, CPT, NTH) join_rms_norm_k<T, PC, CPT, NTH><<<M, NTH, 0, s>>>(x)
     if (wide) {
@@ -470,16 +507,19 @@ static int join_launch(const JoinArgs& x, int M, hipStream_t s) {
     return tp_check_launch("join_rms_norm");
 }
 
-// gain null: no norm, no output.  a, b: [M, D] of a_dtype, b_dtype, float32 ones in a_slices, b_slices slices a stride apart
+// gain null: no norm, no output.  a, b: [M, D] of a_dtype, b_dtype, float32 ones in a_slices, b_slices slices a stride apart,
+// times wa and wb.  stack: rows of (2 + origin_terms) D bfloat16 or 2 D float32 elements (out_dtype), in place of a norm
 extern "C" int tp_join_rms_norm(float* stream, const void* a, int a_dtype, int a_slices, long a_stride, const void* b, int b_dtype, int b_slices,
                                 long b_stride, const float* vec, const float* origin, const float* gain, float eps, void* out, int out_dtype,
-                                int M, int D, void* stream_) {
+                                float wa, float wb, int fresh, void* stack, int origin_terms, int M, int D, void* stream_) {
+    TP_REQUIRE(!stack || (origin && !gain && !vec && (origin_terms == 1 || origin_terms == 2)), "join_rms_norm: operand rows need earlier rows (in one or two terms) and leave no norm");
+    TP_REQUIRE(!fresh || a, "join_rms_norm: rows that replace the stream are missing");
     TP_REQUIRE(M > 0 && D > 0 && stream, "join_rms_norm: empty shape M=%d D=%d", M, D);
     TP_REQUIRE(!gain || out, "join_rms_norm: a norm needs an output buffer");
     TP_REQUIRE(a || !b, "join_rms_norm: a second operand without a first");
     TP_REQUIRE(!a || ((a_dtype == TP_F32 || a_dtype == TP_BF16) && a_slices >= 1 && (a_slices == 1 || a_dtype == TP_F32)), "join_rms_norm: rows in %d slices of dtype %d", a_slices, a_dtype);
     TP_REQUIRE(!b || ((b_dtype == TP_F32 || b_dtype == TP_BF16) && b_slices >= 1 && (b_slices == 1 || b_dtype == TP_F32)), "join_rms_norm: rows in %d slices of dtype %d", b_slices, b_dtype);
-    JoinArgs x{stream, a, a_dtype == TP_F32, a_slices, a_stride, b, b_dtype == TP_F32, b_slices, b_stride, vec, origin, gain, eps, out, D};
+    JoinArgs x{stream, a, a_dtype == TP_F32, a_slices, a_stride, b, b_dtype == TP_F32, b_slices, b_stride, vec, origin, gain, eps, out, D, wa, wb, fresh, stack, origin_terms};
     if (out_dtype == TP_BF16) return join_launch<bf16_t>(x, M, (hipStream_t)stream_);
     if (out_dtype == TP_F32) return join_launch<float>(x, M, (hipStream_t)stream_);
     return tp_fail("join_rms_norm: unknown output dtype %d", out_dtype);

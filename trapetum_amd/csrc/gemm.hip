@@ -48,7 +48,8 @@ gemm_simple_k(const TI* __restrict__ X, const TI* __restrict__ W, TO* __restrict
         for (int j = 0; j < R; j++) {
             const int n = n0 + tx * R + j;
             if (n >= N) continue;
-            st_f32(Y + (size_t)m * N + n, plain_epilogue(epilogue, acc[i][j], epi));
+            st_f32(Y + (size_t)m * N + n, epilogue == TP_EPI_SILU ? ((float)n < epi.z ? gate_act_exact(acc[i][j], TP_ACT_SILU) : acc[i][j])
+                                                                      : plain_epilogue(epilogue, acc[i][j], epi, n));
         }
     }
 }
@@ -57,7 +58,7 @@ extern "C" int tp_gated_act(const float* y, void* out, int dtype, int M, int I, 
 
 template <typename TI>
 static int simple_typed(const GemmArgs& a, void* y, int out_dtype, int epilogue) {
-    const float4 epi = make_float4(a.cap, 0.f, 0.f, 0.f);
+    const float4 epi = make_float4(a.cap, 0.f, (float)a.units, 0.f);
     if (a.M <= 16) {
         dim3 grid(tp_cdiv(a.N, 16), 1);
         if (out_dtype == TP_F32)
@@ -95,6 +96,7 @@ static int check_args(const GemmArgs& a) {
     TP_REQUIRE(a.out_dtype == TP_F32 || a.out_dtype == TP_BF16, "linear: unknown output dtype %d", a.out_dtype);
     TP_REQUIRE(!(a.in_dtype == TP_F32 && a.out_dtype == TP_BF16), "linear: float32 rows give float32 output");
     TP_REQUIRE(a.epilogue != TP_EPI_SOFTCAP || a.cap > 0.f, "linear: a soft cap must be positive");
+    TP_REQUIRE(a.epilogue != TP_EPI_SILU || (a.units > 0 && a.units <= a.N && a.N < (1 << 24)), "linear: SiLU on the first %d of %d columns", a.units, a.N);
     TP_REQUIRE(!a.defer || a.epilogue == TP_EPI_NONE, "linear: K slices can be left to the consumer only without an epilogue (found %d)", a.epilogue);
     if (a.epilogue == TP_EPI_GATED) {
         const int padded = 2 * ((a.units + 15) / 16) * 16;

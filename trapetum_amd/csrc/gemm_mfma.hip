@@ -56,7 +56,7 @@ __device__ __forceinline__ void store_tile(const f32x4 (&acc)[TM][TN], void* __r
             } else {
                 col = n0 + wn * 16 * TN + j * 16 + g * 4;
 #pragma unroll
-                for (int v = 0; v < 4; v++) o[v] = plain_epilogue(EPI, acc[i][j][v], epi);
+                for (int v = 0; v < 4; v++) o[v] = plain_epilogue(EPI, acc[i][j][v], epi, col + v);
             }
             if (col >= width) continue;
             const size_t at = (size_t)m * width + col;
@@ -484,12 +484,14 @@ int gemm_mfma_launch(const GemmArgs& a) {
         if (a.epilogue == TP_EPI_GATED) mfma_launch_direct<TP_EPI_GATED>(a, t, a.y, a.out_dtype, 1, a.K);
         else if (a.epilogue == TP_EPI_SOFTCAP) mfma_launch_direct<TP_EPI_SOFTCAP>(a, t, a.y, a.out_dtype, 1, a.K);
         else if (a.epilogue == TP_EPI_RELU2) mfma_launch_direct<TP_EPI_RELU2>(a, t, a.y, a.out_dtype, 1, a.K);
+        else if (a.epilogue == TP_EPI_SILU) mfma_launch_direct<TP_EPI_SILU>(a, t, a.y, a.out_dtype, 1, a.K);
         else mfma_launch_direct<TP_EPI_NONE>(a, t, a.y, a.out_dtype, 1, a.K);
         return tp_check_launch("linear (tiled kernel, loads into LDS)");
     }
     if (a.epilogue == TP_EPI_GATED) mfma_launch_tile<TP_EPI_GATED>(a, t, a.y, a.out_dtype, 1, a.K);
     else if (a.epilogue == TP_EPI_SOFTCAP) mfma_launch_tile<TP_EPI_SOFTCAP>(a, t, a.y, a.out_dtype, 1, a.K);
     else if (a.epilogue == TP_EPI_RELU2) mfma_launch_tile<TP_EPI_RELU2>(a, t, a.y, a.out_dtype, 1, a.K);
+    else if (a.epilogue == TP_EPI_SILU) mfma_launch_tile<TP_EPI_SILU>(a, t, a.y, a.out_dtype, 1, a.K);
     else mfma_launch_tile<TP_EPI_NONE>(a, t, a.y, a.out_dtype, 1, a.K);
     return tp_check_launch("linear (tiled kernel)");
 }

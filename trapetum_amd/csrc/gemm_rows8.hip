@@ -121,7 +121,7 @@ gemm_rows8_k(const bf16_t* __restrict__ X, const bf16_t* __restrict__ W, void* _
             const int n = row0[t] + wr;
             if (n >= N) continue;
             float o = v[t];
-            o = plain_epilogue(epilogue, o, epi);
+            o = plain_epilogue(epilogue, o, epi, n);
             if (out_dtype == TP_F32) ((float*)Y)[(size_t)m * N + n] = o;
             else ((bf16_t*)Y)[(size_t)m * N + n] = f32_to_bf16(o);
         }

@@ -156,7 +156,7 @@ gemm_skinny_k(const bf16_t* __restrict__ X, const bf16_t* __restrict__ W, void* 
                 const int n = n0 + s * 16 + nl;
                 if (n >= N) continue;
                 float o = v[t][s];
-                o = plain_epilogue(epilogue, o, epi);
+                o = plain_epilogue(epilogue, o, epi, n);
                 store_out(Y, out_dtype, (size_t)m * N + n, o);
             }
         }
@@ -182,7 +182,7 @@ __global__ void skinny_reduce_k(const float* __restrict__ part, void* __restrict
         } else {
             float sum = 0.f;
             for (int s = 0; s < n_splits; s++) sum += part[((size_t)s * M + m) * N + c];
-            sum = plain_epilogue(epilogue, sum, epi);
+            sum = plain_epilogue(epilogue, sum, epi, c);
             store_out(Y, out_dtype, idx, sum);
         }
     }

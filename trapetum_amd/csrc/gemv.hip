@@ -100,7 +100,7 @@ gemv_k(const bf16_t* __restrict__ X, const bf16_t* __restrict__ W, void* __restr
             for (int j = 0; j < GV_ROWS; j++) {
                 if (row[j] >= N) continue;
                 float o = acc[j][m];
-                o = plain_epilogue(epilogue, o, epi);
+                o = plain_epilogue(epilogue, o, epi, row[j]);
                 if (out_dtype == TP_F32) ((float*)Y)[(size_t)m * N + row[j]] = o;
                 else ((bf16_t*)Y)[(size_t)m * N + row[j]] = f32_to_bf16(o);
             }

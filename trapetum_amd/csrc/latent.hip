@@ -100,11 +100,15 @@ extern "C" int tp_latent_prepare(const void* proj, long proj_stride, int dtype, 
 
 // ---- per-head products: out[m, h, n] = sum_k x[m, h, k] * w[h, n, k] ----------------------------------------------
 // x and out are views of wider rows (strides in elements: row, head; elements of a head contiguous); w is contiguous.
+// gate (or null): rows of H N elements of the same type; out[m, h, n] is multiplied by sigmoid(gate[m][h N + n]) before it is
+// rounded.
+__device__ __forceinline__ float gated_by(float x, float g) { return x / (1.f + expf(-g)); }
+
 // grid (column tiles, row tiles, heads)
 template <typename T, int TM>
 __global__ void __launch_bounds__(256)
 head_linear_k(const T* __restrict__ x, long x_row, long x_head, const T* __restrict__ w, T* __restrict__ out, long o_row, long o_head,
-              int M, int N, int K) {
+              int M, int N, int K, const T* __restrict__ gate, long gate_row) {
     constexpr int TN = 64, BK = 16;
     __shared__ TileShared<TM, TN, BK> sh;
     const int h = blockIdx.z, m0 = blockIdx.y * TM, n0 = blockIdx.x * TN;
@@ -120,7 +124,7 @@ head_linear_k(const T* __restrict__ x, long x_row, long x_head, const T* __restr
 #pragma unroll
         for (int j = 0; j < TN / 16; j++) {
             const int m = m0 + ty + 16 * i, n = n0 + tx + 16 * j;
-            if (m < M && n < N) st_f32(out + (size_t)m * o_row + (size_t)h * o_head + n, acc[i][j]);
+            if (m < M && n < N) st_f32(out + (size_t)m * o_row + (size_t)h * o_head + n, gate ? gated_by(acc[i][j], ld_f32(gate + (size_t)m * gate_row + (size_t)h * N + n)) : acc[i][j]);
         }
 }
 
@@ -128,7 +132,7 @@ head_linear_k(const T* __restrict__ x, long x_row, long x_head, const T* __restr
 template <int TM>
 __global__ void __launch_bounds__(256)
 head_linear_mfma_k(const bf16_t* __restrict__ x, long x_row, long x_head, const bf16_t* __restrict__ w, bf16_t* __restrict__ out,
-                   long o_row, long o_head, int M, int N, int K) {
+                   long o_row, long o_head, int M, int N, int K, const bf16_t* __restrict__ gate, long gate_row) {
     using Tile = MfmaTile<TM, false>;
     __shared__ typename Tile::Shared sh;
     const int h = blockIdx.z, m0 = blockIdx.y * TM, n0 = blockIdx.x * 64;
@@ -145,8 +149,13 @@ head_linear_mfma_k(const bf16_t* __restrict__ x, long x_row, long x_head, const 
 #pragma unroll
         for (int j = 0; j < Tile::NJ; j++) {
             const int m = m0 + Tile::m_of(i), n = n0 + Tile::n_of(j);
-            if (m >= M) continue;
+            if (m >= M || n >= N) continue;
             bf16_t* dst = out + (size_t)m * o_row + (size_t)h * o_head + n;
+            if (gate) {
+                const bf16_t* gp = gate + (size_t)m * gate_row + (size_t)h * N + n;
+#pragma unroll
+                for (int v = 0; v < 4; v++) t.acc[0][i][j][v] = gated_by(t.acc[0][i][j][v], bf16_to_f32(gp[n + v < N ? v : 0]));
+            }
             if (wide && n + 3 < N) {                      // the lane's four neighbours in one store
                 uint2 o;
                 o.x = (uint32_t)f32_to_bf16(t.acc[0][i][j][0]) | ((uint32_t)f32_to_bf16(t.acc[0][i][j][1]) << 16);
@@ -161,7 +170,8 @@ head_linear_mfma_k(const bf16_t* __restrict__ x, long x_row, long x_head, const 
 }
 
 extern "C" int tp_head_linear(const void* x, long x_row, long x_head, const void* w, void* out, long o_row, long o_head,
-                              int dtype, int M, int H, int N, int K, int plain, void* stream) {
+                              int dtype, int M, int H, int N, int K, const void* gate, long gate_row, int plain, void* stream) {
+    TP_REQUIRE(!gate || gate_row >= (long)H * N, "head_linear: gates of %ld elements a row do not cover %d heads of %d", gate_row, H, N);
     TP_REQUIRE(M > 0 && H > 0 && N > 0 && K > 0, "head_linear: empty shape M=%d H=%d N=%d K=%d", M, H, N, K);
     TP_REQUIRE(x && w && out, "head_linear: a null operand");
     TP_REQUIRE(x_head >= K && o_head >= N && x_row >= (long)(H - 1) * x_head + K && o_row >= (long)(H - 1) * o_head + N,
@@ -174,15 +184,15 @@ extern "C" int tp_head_linear(const void* x, long x_row, long x_head, const void
     TP_REQUIRE(grid.y <= 65535, "head_linear: %d rows exceed one launch", M);
     if (dtype == TP_BF16 && !plain && M >= 512 && K % 8 == 0 && x_row % 8 == 0 && x_head % 8 == 0 && (uintptr_t)x % 16 == 0 && (uintptr_t)w % 16 == 0) {
         grid.y = tp_cdiv(M, 128);
-        head_linear_mfma_k<128><<<grid, 256, 0, s>>>((const bf16_t*)x, x_row, x_head, (const bf16_t*)w, (bf16_t*)out, o_row, o_head, M, N, K);
+        head_linear_mfma_k<128><<<grid, 256, 0, s>>>((const bf16_t*)x, x_row, x_head, (const bf16_t*)w, (bf16_t*)out, o_row, o_head, M, N, K, (const bf16_t*)gate, gate_row);
         return tp_check_launch("head_linear (matrix cores)");
     }
     if (dtype == TP_BF16 && !plain && K % 8 == 0 && x_row % 8 == 0 && x_head % 8 == 0 && (uintptr_t)x % 16 == 0 && (uintptr_t)w % 16 == 0) {
-        if (few) head_linear_mfma_k<16><<<grid, 256, 0, s>>>((const bf16_t*)x, x_row, x_head, (const bf16_t*)w, (bf16_t*)out, o_row, o_head, M, N, K);
-        else head_linear_mfma_k<64><<<grid, 256, 0, s>>>((const bf16_t*)x, x_row, x_head, (const bf16_t*)w, (bf16_t*)out, o_row, o_head, M, N, K);
+        if (few) head_linear_mfma_k<16><<<grid, 256, 0, s>>>((const bf16_t*)x, x_row, x_head, (const bf16_t*)w, (bf16_t*)out, o_row, o_head, M, N, K, (const bf16_t*)gate, gate_row);
+        else head_linear_mfma_k<64><<<grid, 256, 0, s>>>((const bf16_t*)x, x_row, x_head, (const bf16_t*)w, (bf16_t*)out, o_row, o_head, M, N, K, (const bf16_t*)gate, gate_row);
         return tp_check_launch("head_linear (matrix cores)");
     }
-#define TP_HEAD_LINEAR(T, TMv) head_linear_k<T, TMv><<<grid, 256, 0, s>>>((const T*)x, x_row, x_head, (const T*)w, (T*)out, o_row, o_head, M, N, K)
+#define TP_HEAD_LINEAR(T, TMv) head_linear_k<T, TMv><<<grid, 256, 0, s>>>((const T*)x, x_row, x_head, (const T*)w, (T*)out, o_row, o_head, M, N, K, (const T*)gate, gate_row)
     if (dtype == TP_BF16) { if (few) TP_HEAD_LINEAR(bf16_t, 16); else TP_HEAD_LINEAR(bf16_t, 64); }
     else if (dtype == TP_F32) { if (few) TP_HEAD_LINEAR(float, 16); else TP_HEAD_LINEAR(float, 64); }
     else return tp_fail("head_linear: unknown dtype %d", dtype);

@@ -123,6 +123,55 @@ head_norm_gate_k(const float* __restrict__ y, const float* __restrict__ gain, co
     }
 }
 
+// The same for long parts (a whole row normed together): a block of 256 lanes each, quads of elements held in registers.
+template <typename TG, typename TO, int Q>
+__global__ void __launch_bounds__(256)
+long_norm_gate_k(const float* __restrict__ y, const float* __restrict__ gain, const TG* __restrict__ g, long g_stride, float eps,
+                 TO* __restrict__ out, int H, int hs, int act) {
+    __shared__ float red[16];
+    const int r = blockIdx.x, h = blockIdx.y, tid = threadIdx.x;
+    const float* yr = y + ((size_t)r * H + h) * hs;
+    const TG* gr = g + (size_t)r * g_stride + (size_t)h * hs;
+    struct alignas(4 * sizeof(TG)) G4 { TG v[4]; };
+    struct alignas(4 * sizeof(TO)) O4 { TO v[4]; };
+    float4 a[Q], w[Q];
+    G4 gq[Q];
+    float ss = 0.f;
+#pragma unroll
+    for (int j = 0; j < Q; j++) {
+        const int d = (tid + 256 * j) * 4, dc = d < hs ? d : 0;
+        a[j] = *reinterpret_cast<const float4*>(yr + dc);
+        w[j] = *reinterpret_cast<const float4*>(gain + (size_t)h * hs + dc);
+        gq[j] = *reinterpret_cast<const G4*>(gr + dc);
+        if (d < hs) ss += a[j].x * a[j].x + a[j].y * a[j].y + a[j].z * a[j].z + a[j].w * a[j].w;
+    }
+    const float inv = rsqrtf(block_sum_once(ss, red) / (float)hs + eps);
+#pragma unroll
+    for (int j = 0; j < Q; j++) {
+        const int d = (tid + 256 * j) * 4;
+        const float v[4] = {a[j].x * inv * w[j].x, a[j].y * inv * w[j].y, a[j].z * inv * w[j].z, a[j].w * inv * w[j].w};
+        O4 o;
+#pragma unroll
+        for (int e = 0; e < 4; e++) {
+            const float gv = ld_f32(&gq[j].v[e]), sg = 1.f / (1.f + expf(-gv));
+            st_f32(&o.v[e], v[e] * (act == TP_GATE_SILU ? gv * sg : sg));
+        }
+        if (d < hs) *reinterpret_cast<O4*>(out + ((size_t)r * H + h) * hs + d) = o;
+    }
+}
+template <typename TG, typename TO>
+static bool long_norm_gate(const float* y, const float* gain, const void* g, long g_stride, float eps, void* out, int M, int H, int hs, int act, hipStream_t s) {
+    if (hs <= 256 || hs > 8192 || hs % 4 || g_stride % 4 || (uintptr_t)g % (4 * sizeof(TG)) || (uintptr_t)y % 16 || (uintptr_t)gain % 16 || (uintptr_t)out % (4 * sizeof(TO))) return false;
+    dim3 grid(M, H);
+#define TP_LONG(Q) long_norm_gate_k<TG, TO, Q><<<grid, 256, 0, s>>>(y, gain, (const TG*)g, g_stride, eps, (TO*)out, H, hs, act)
+    if (hs <= 1024) TP_LONG(1);
+    else if (hs <= 3072) TP_LONG(3);
+    else if (hs <= 5120) TP_LONG(5);
+    else TP_LONG(8);
+#undef TP_LONG
+    return true;
+}
+
 extern "C" int tp_head_norm_gate(const float* y, const float* gain, const void* g, long g_stride, int g_dtype, float eps, void* out,
                                  int out_dtype, int M, int H, int hs, int act, void* stream) {
     TP_REQUIRE(M > 0 && H > 0 && hs > 0 && y && gain && g && out, "head_norm_gate: empty shape or null operand (M=%d H=%d size=%d)", M, H, hs);
@@ -130,6 +179,9 @@ extern "C" int tp_head_norm_gate(const float* y, const float* gain, const void* 
     TP_REQUIRE(H <= 65535, "head_norm_gate: %d heads exceed one launch", H);
     hipStream_t s = (hipStream_t)stream;
     dim3 grid(M, H);
+    if (g_dtype == TP_BF16 && out_dtype == TP_BF16 ? long_norm_gate<bf16_t, bf16_t>(y, gain, g, g_stride, eps, out, M, H, hs, act, s)
+        : g_dtype == TP_F32 && out_dtype == TP_F32 && long_norm_gate<float, float>(y, gain, g, g_stride, eps, out, M, H, hs, act, s))
+        return tp_check_launch("head_norm_gate (long rows)");
     if (g_dtype == TP_BF16 && out_dtype == TP_BF16) head_norm_gate_k<bf16_t, bf16_t><<<grid, 64, 0, s>>>(y, gain, (const bf16_t*)g, g_stride, eps, (bf16_t*)out, H, hs, act);
     else if (g_dtype == TP_F32 && out_dtype == TP_F32) head_norm_gate_k<float, float><<<grid, 64, 0, s>>>(y, gain, (const float*)g, g_stride, eps, (float*)out, H, hs, act);
     else return tp_fail("head_norm_gate: gate dtype %d with output dtype %d has no kernel", g_dtype, out_dtype);

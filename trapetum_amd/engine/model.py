@@ -55,8 +55,14 @@ class Model:
         for layer in self.layers:
             self.places.extend(layer.places)
         # what the model adds to the stream before a run of a layer, by schedule entry
-        self.added = [build_part("stream_add", e.before) if e.before is not None else None for e in spec.schedule]
-        self.places.extend((p, e.before_prefix) for p, e in zip(self.added, spec.schedule) if p is not None)
+        # (runs that name the same part with the same tensors share it)
+        self.added, built = [], {}
+        for e in spec.schedule:
+            key = (repr(e.before), e.before_prefix)
+            if e.before is not None and key not in built:
+                built[key] = build_part("stream_add", e.before)
+                self.places.append((built[key], e.before_prefix))
+            self.added.append(built[key] if e.before is not None else None)
         self.places.append((self.final_norm, spec.final_norm_prefix))
         self.places.append((self.head, spec.head_prefix))
         self.schedule = spec.schedule

@@ -19,7 +19,7 @@ ARCH = "gfx950"
 FLAGS = ["--offload-arch=" + ARCH, "-O3", "-fPIC", "-std=c++17",
          "-Xclang", "-target-feature", "-Xclang", "-packed-fp32-ops", "-Wno-unused-result"]
 CORE_SOURCES = ["elementwise.hip", "gemm.hip", "gemm_skinny.hip", "gemm_mfma.hip", "gemv.hip", "gemm_rows8.hip", "attention_simple.hip", "sampling.hip", "probes.hip",
-                "conv.hip", "latent.hip", "moe.hip", "ssd.hip", "recurrent.hip", "delta.hip", "attention_pooled.hip"]
+                "conv.hip", "latent.hip", "moe.hip", "ssd.hip", "recurrent.hip", "delta.hip", "linear_scan.hip", "attention_pooled.hip"]
 ATTN_SOURCES = ["attention_mfma.hip", "attention_prefill.hip", "attention_pooled_mfma.hip"]      # decode steps; steps of many queries; a window with pooled blocks
 _NOISE = "is not a recognized feature for this target"
 
@@ -142,12 +142,14 @@ def build_core(force=False):
     return build_library("trapetum_core", CORE_SOURCES, force=force)
 
 
-def attn_name(head_dim, wide=False):
-    return f"trapetum_attn_hd{head_dim}" + ("w" if wide else "")
+def attn_name(head_dim, wide=False, by_position=False):
+    return f"trapetum_attn_hd{head_dim}" + ("w" if wide else "") + ("p" if by_position else "")
 
 
-def build_attention(head_dim, force=False, wide=False):
+def build_attention(head_dim, force=False, wide=False, by_position=False):
     """wide: the variant whose kernel of many queries carries the softmax weights into the second product as two bf16
-    terms (see attention_prefill.hip)."""
-    defines = [f"-DTP_HD={head_dim}"] + (["-DTP_WIDE_WEIGHTS=1"] if wide else [])
-    return build_library(attn_name(head_dim, wide), ATTN_SOURCES, defines, force=force)
+    terms (see attention_prefill.hip).  by_position: the variant whose kernels know scores that depend on positions and a
+    gate per head (TpPositional in common.h)."""
+    defines = [f"-DTP_HD={head_dim}"] + (["-DTP_WIDE_WEIGHTS=1"] if wide else []) + (["-DTP_BY_POSITION=1"] if by_position else [])
+    sources = ATTN_SOURCES[:2] if by_position else ATTN_SOURCES
+    return build_library(attn_name(head_dim, wide, by_position), sources, defines, force=force)

@@ -15,13 +15,13 @@ _P, _I, _L, _F = _c.c_void_p, _c.c_int, _c.c_long, _c.c_float
 
 _CORE_SIGS = {
     "tp_embed_rows": [_P, _P, _I, _F, _P, _I, _I, _I, _P],
-    "tp_rms_norm": [_P, _I, _P, _F, _P, _I, _I, _I, _I, _P],
+    "tp_rms_norm": [_P, _L, _I, _P, _F, _P, _I, _I, _I, _I, _P],
     "tp_add_rms_norm": [_P, _P, _I, _I, _L, _P, _F, _P, _F, _P, _I, _I, _I, _I, _P],
-    "tp_join_rms_norm": [_P, _P, _I, _I, _L, _P, _I, _I, _L, _P, _P, _P, _F, _P, _I, _I, _I, _P],
+    "tp_join_rms_norm": [_P, _P, _I, _I, _L, _P, _I, _I, _L, _P, _P, _P, _F, _P, _I, _F, _F, _I, _P, _I, _I, _I, _P],
     "tp_scale_rows": [_P, _L, _F, _P],
     "tp_causal_conv": [_P, _P, _P, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _I, _P],
     "tp_latent_prepare": [_P, _L, _I, _I, _I, _I, _I, _I, _P, _F, _P, _I, _P, _P, _P, _P, _I, _P, _I, _I, _P, _P, _I, _P, _L, _P],
-    "tp_head_linear": [_P, _L, _L, _P, _P, _L, _L, _I, _I, _I, _I, _I, _I, _P],
+    "tp_head_linear": [_P, _L, _L, _P, _P, _L, _L, _I, _I, _I, _I, _I, _P, _L, _I, _P],
     "tp_route_top": [_P, _I, _I, _I, _I, _I, _P, _F, _P, _P, _P],
     "tp_expert_ffn_workspace_bytes": [_I, _I, _I, _I, _I, _I],
     "tp_expert_ffn": [_P, _I, _I, _I, _P, _P, _I, _I, _I, _P, _P, _I, _F, _F, _F, _I, _P, _L, _P, _I, _P],
@@ -52,11 +52,13 @@ _CORE_SIGS = {
     "tp_matrix_memory_scan": [_P, _L, _P, _L, _P, _L, _I, _P, _F, _F, _P, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _P, _P],
     "tp_delta_scan": [_P, _L, _P, _L, _P, _L, _P, _P, _L, _I, _P, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _F, _I, _P, _L, _P],
     "tp_delta_scan_workspace_bytes": [_I, _I, _I, _I, _I],
+    "tp_linear_scan": [_P, _L, _P, _L, _P, _L, _I, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _P, _L, _P],
+    "tp_linear_scan_workspace_bytes": [_I, _I, _I, _I, _I],
     "tp_time_mix_scan_workspace_floats": [_I, _I, _I, _I],
     "tp_matrix_memory_scan_workspace_floats": [_I, _I, _I, _I, _I],
     "tp_linear_workspace_bytes": [_I, _I, _I, _I, _I, _I, _I, _I, _I],
-    "tp_attn_simple_prefill": [_P, _L, _P, _L, _P, _L, _I, _I, _I, _I, _I, _P, _P, _P, _P, _P, _I, _P, _P, _I, _I, _F, _F, _I, _I, _P, _P, _I, _I, _P, _P],
-    "tp_attn_simple_decode": [_P, _L, _I, _I, _I, _I, _I, _P, _P, _I, _P, _P, _I, _I, _F, _F, _I, _I, _P, _P, _I, _I, _P, _P],
+    "tp_attn_simple_prefill": [_P, _L, _P, _L, _P, _L, _I, _I, _I, _I, _I, _P, _P, _P, _P, _P, _I, _P, _P, _I, _I, _F, _F, _I, _I, _P, _P, _I, _I, _P, _P, _P],
+    "tp_attn_simple_decode": [_P, _L, _I, _I, _I, _I, _I, _P, _P, _I, _P, _P, _I, _I, _F, _F, _I, _I, _P, _P, _I, _I, _P, _P, _P],
     "tp_argmax": [_P, _I, _I, _P, _P, _P],
     "tp_argmax_workspace_bytes": [_I, _I],
     "tp_repetition_penalty": [_P, _I, _I, _P, _I, _F, _P],
@@ -68,16 +70,16 @@ _CORE_SIGS = {
     "tp_probe_mfma": [_I, _I, _I, _P, _P, _P],
 }
 _ATTN_SIGS = {
-    "tp_attn_prefill": [_P, _L, _P, _L, _P, _L, _I, _I, _I, _P, _I, _I, _P, _P, _I, _P, _P, _I, _I, _F, _F, _I, _I, _P, _P, _I, _I, _P, _I, _P],
-    "tp_attn_decode": [_P, _L, _I, _I, _I, _P, _P, _I, _P, _P, _I, _I, _F, _F, _I, _I, _P, _P, _I, _I, _P, _P, _I, _P],
-    "tp_attn_decode_shared": [_P, _L, _I, _I, _I, _I, _P, _P, _I, _P, _P, _I, _I, _F, _F, _I, _P, _P, _I, _P],
+    "tp_attn_prefill": [_P, _L, _P, _L, _P, _L, _I, _I, _I, _P, _I, _I, _P, _P, _I, _P, _P, _I, _I, _F, _F, _I, _I, _P, _P, _I, _I, _P, _P, _I, _P],
+    "tp_attn_decode": [_P, _L, _I, _I, _I, _P, _P, _I, _P, _P, _I, _I, _F, _F, _I, _I, _P, _P, _I, _I, _P, _P, _P, _I, _P],
+    "tp_attn_decode_shared": [_P, _L, _I, _I, _I, _I, _P, _P, _I, _P, _P, _I, _I, _F, _F, _I, _P, _P, _P, _I, _P],
     "tp_attn_decode_workspace_floats": [_I, _I, _I],
     "tp_attn_pooled_tile": [_P, _L, _P, _L, _P, _L, _I, _I, _I, _I, _P, _P, _P, _I, _P, _P, _I, _I, _P, _I, _P, _P, _I, _F, _F, _I, _I, _P, _P],
-    "tp_attn_decode_fused": [_P, _I, _I, _L, _L, _P, _I, _I, _I, _I, _I, _P, _P, _I, _P, _P, _I, _I, _F, _F, _I, _P, _I, _I, _P, _P, _I, _P],
+    "tp_attn_decode_fused": [_P, _I, _I, _L, _L, _P, _I, _I, _I, _I, _I, _P, _P, _I, _P, _P, _I, _I, _F, _F, _I, _P, _I, _I, _P, _P, _P, _I, _P],
 }
 
-EPI_NONE, EPI_SOFTCAP, EPI_GATED, EPI_RELU2 = 0, 1, 2, 3
-PLAIN_ACTIVATIONS = {"relu2": EPI_RELU2}              # what a product without a gate can apply to its sums: max(z, 0)^2
+EPI_NONE, EPI_SOFTCAP, EPI_GATED, EPI_RELU2, EPI_SILU = 0, 1, 2, 3, 4
+PLAIN_ACTIVATIONS = {"relu2": EPI_RELU2, "silu": EPI_SILU}     # what a product without a gate can apply to its sums: max(z, 0)^2, z sigmoid(z)
 ROPE_PAIRINGS = {"halves": 0, "neighbours": 1}          # the kernel library's TP_ROPE_* enumerators
 GATE_ACTIVATIONS = {"gelu_tanh": 0, "silu": 1, "relu": 2, "quick_gelu": 3}       # what a gated product's epilogue can apply to the gate
 HEAD_GATES = {"sigmoid": 0, "silu": 1}               # what `head_norm_gate` multiplies a normed head by: act(g)
@@ -102,6 +104,36 @@ class SplitRows:
         self.dtype = torch.float32
 
 
+class _PositionalStruct(_c.Structure):
+    """The kernel library's TpPositional (common.h)."""
+    _fields_ = [("bias", _P), ("reach", _L), ("gate", _P), ("gate_f32", _L), ("gate_slices", _L), ("gate_slice_stride", _L),
+                ("gate_stride", _L), ("temp_coef", _F), ("temp_every", _I)]
+
+
+class ByPosition:
+    """What of an attention's scores and outputs depends on positions, and its heads' gates (each may be absent):
+    temperature (coef, every): scores of the query at p times 1 + coef ln(floor((p + 1) / every) + 1);
+    bias float32 [H, reach + 1]: added to head h's score on the key at distance n, entry min(n, reach), after the cap;
+    gate: head h's output of row r is multiplied by sigmoid(gate[r, h]): a view [rows, H] of wider rows or, in a fused
+    decode step, the number of the first of H columns of the step's projections."""
+
+    def __init__(self, temperature=None, bias=None, gate=None):
+        self.temperature, self.bias, self.gate = temperature, bias, gate
+
+    def with_gate(self, gate):
+        return ByPosition(self.temperature, self.bias, gate)
+
+
+class WeightedRows:
+    """wa * a + wb * b of two sub-mixers' rows (tensors or SplitRows), not added up yet: the kernel that adds them to the
+    stream (`join_rms_norm`) takes both with their constants.  `HipOps.rows()` forms the sum otherwise."""
+
+    def __init__(self, a, wa, b, wb):
+        self.a, self.wa, self.b, self.wb = a, float(wa), b, float(wb)
+        self.shape = tuple(a.shape)
+        self.dtype = torch.float32
+
+
 def _code(dtype):
     if dtype == torch.float32:
         return 0
@@ -120,6 +152,8 @@ def _bind(lib, sigs):
 
 class HipOps:
     SplitRows = SplitRows
+    WeightedRows = WeightedRows
+    ByPosition = ByPosition
 
     def __init__(self, device):
         if device.type != "cuda" or not torch.cuda.is_available():
@@ -201,14 +235,17 @@ class HipOps:
             raise KernelError(f"{what}: expected rows with contiguous elements, found shape {tuple(t.shape)} strides {t.stride()}")
         return t.stride(0)
 
-    def attn_lib(self, head_dim, wide=False):
-        key = (head_dim, bool(wide))
+    def attn_lib(self, head_dim, wide=False, by_position=False):
+        """The library of a head size; by_position: the variant whose kernels know `ByPosition` (its kernel of many queries
+        carries its weights in two terms)."""
+        wide = bool(wide or by_position)
+        key = (head_dim, wide, bool(by_position))
         if key not in self._attn:
             try:
-                lib = _c.CDLL(_build.build_attention(head_dim, wide=wide))
+                lib = _c.CDLL(_build.build_attention(head_dim, wide=wide, by_position=by_position))
             except (OSError, _build.BuildError) as e:
                 raise KernelError(f"the attention kernels for head_dim {head_dim} could not be built or loaded: {e}") from None
-            _bind(lib, _ATTN_SIGS)
+            _bind(lib, {k: v for k, v in _ATTN_SIGS.items() if not (by_position and k == "tp_attn_pooled_tile")})     # (that variant is decode and prefill)
             self._attn[key] = lib
         return self._attn[key]
 
@@ -238,15 +275,14 @@ class HipOps:
     def rms_norm(self, x, gain, eps, out_dtype, groups=1):
         """groups: the row is cut into that many equal consecutive parts, each over its own root mean square."""
         self._dev(x, gain)
-        if not x.is_contiguous() or x.dim() != 2:
-            raise KernelError("rms_norm: rows must be a contiguous matrix")
+        stride = self._rows(x, "rms_norm rows")              # a view of wider rows may do
         m, d = x.shape
         if gain.dtype != torch.float32 or gain.numel() != d or not gain.is_contiguous():
             raise KernelError(f"rms_norm: gain must be float32 [{d}]")
         out = torch.empty((m, d), dtype=out_dtype, device=self.device)
         if groups < 1 or d % groups:
             raise KernelError(f"rms_norm: rows of {d} elements cannot be cut into {groups} equal groups")
-        self._call(self.lib, "tp_rms_norm", x.data_ptr(), _code(x.dtype), gain.data_ptr(), float(eps), out.data_ptr(),
+        self._call(self.lib, "tp_rms_norm", x.data_ptr(), stride, _code(x.dtype), gain.data_ptr(), float(eps), out.data_ptr(),
                    _code(out_dtype), m, d, int(groups), self._stream())
         return out
 
@@ -277,10 +313,17 @@ class HipOps:
                    out.data_ptr() if out is not None else None, _code(out_dtype), m, d, int(groups), self._stream())
         return out
 
-    def join_rms_norm(self, stream, a, b, gain, eps, out_dtype, vec=None, origin=None):
-        """stream += a + b (+ vec) (+ origin); returns norm(stream), or None without a gain.  a, b: rows [M, D] (a tensor of
-        either dtype, or SplitRows), b or both may be None; vec float32 [D] goes to every row, origin float32 [M, D]."""
+    def join_rms_norm(self, stream, a, b, gain, eps, out_dtype, vec=None, origin=None, wa=1.0, wb=1.0, fresh=False, stack=0):
+        """stream += wa a + wb b (+ vec) (+ origin); returns norm(stream), or None without a gain.  a, b: rows [M, D] (a tensor
+        of either dtype, or SplitRows), b or both may be None; vec float32 [D] goes to every row, origin float32 [M, D].
+        fresh: the stream becomes that sum instead of taking it up.  stack (1 or 2): returns the operand rows of a product
+        over [stream | origin] instead of a norm, and origin is not added: float32 [M, 2 D] as they are, or bfloat16
+        [M, (2 + stack) D], the stream in two terms (its rounding and the remainder's) and origin in `stack` terms."""
         m, d = stream.shape
+        if stack and (origin is None or gain is not None or vec is not None or stack not in (1, 2)):
+            raise KernelError("join_rms_norm: operand rows come of the stream and earlier rows in one or two terms, without a norm or a vector")
+        if fresh and a is None:
+            raise KernelError("join_rms_norm: the rows that replace the stream are missing")
         self._dev(stream, gain, vec, origin)
         if stream.dtype != torch.float32 or not stream.is_contiguous():
             raise KernelError("join_rms_norm: the stream must be contiguous float32")
@@ -301,10 +344,13 @@ class HipOps:
             if t is not None and (t.dtype != torch.float32 or t.numel() != n or not t.is_contiguous()):
                 raise KernelError(f"join_rms_norm: the {what} must be contiguous float32 of {n} elements")
         out = torch.empty((m, d), dtype=out_dtype, device=self.device) if gain is not None else None
+        stacked = None
+        if stack:
+            stacked = torch.empty((m, (2 if out_dtype == torch.float32 else 2 + stack) * d), dtype=out_dtype, device=self.device)
         ptr = lambda t: t.data_ptr() if t is not None else None
         self._call(self.lib, "tp_join_rms_norm", stream.data_ptr(), *args, ptr(vec), ptr(origin), ptr(gain), float(eps), ptr(out),
-                   _code(out_dtype), m, d, self._stream())
-        return out
+                   _code(out_dtype), float(wa), float(wb), 1 if fresh else 0, ptr(stacked), int(stack) or 1, m, d, self._stream())
+        return stacked if stack else out
 
     def scale_rows(self, x, scale):
         """x *= scale, in place (float32)."""
@@ -384,10 +430,11 @@ class HipOps:
                    self._stream())
         return q, mine
 
-    def head_linear(self, x, w, out=None):
+    def head_linear(self, x, w, out=None, gate=None):
         """out[m, h, :] = w[h] @ x[m, h, :].  x: a view [M, H, K] of wider rows (a head's elements contiguous), w
-        contiguous [H, N, K]; out: a view [M, H, N] to fill, or None for a new contiguous tensor."""
-        self._dev(x, w, out)
+        contiguous [H, N, K]; out: a view [M, H, N] to fill, or None for a new contiguous tensor.  gate [M, H N] of x's dtype
+        (possibly a view of wider rows): out[m, h, n] times sigmoid(gate[m, h N + n]), before the rounding."""
+        self._dev(x, w, out, gate)
         if x.dim() != 3 or w.dim() != 3 or w.shape[0] != x.shape[1] or w.shape[2] != x.shape[2] or not w.is_contiguous() or x.dtype != w.dtype:
             raise KernelError(f"head_linear: rows {tuple(x.shape)} and matrices {tuple(w.shape)} do not fit, or differ in dtype")
         m, H, K = x.shape
@@ -399,8 +446,13 @@ class HipOps:
         for t, what in ((x, "rows"), (out, "output")):
             if t.shape[2] > 1 and t.stride(2) != 1:
                 raise KernelError(f"head_linear: a head's elements must be contiguous in the {what}")
+        gate_row = 0
+        if gate is not None:
+            gate_row = self._rows(gate, "head_linear gates")
+            if tuple(gate.shape) != (m, H * N) or gate.dtype != x.dtype:
+                raise KernelError(f"head_linear: gates must be {(m, H * N)} of {x.dtype}")
         self._call(self.lib, "tp_head_linear", x.data_ptr(), x.stride(0), x.stride(1), w.data_ptr(), out.data_ptr(),
-                   out.stride(0), out.stride(1), _code(x.dtype), m, H, N, K, 1 if self.force_linear == 1 else 0, self._stream())
+                   out.stride(0), out.stride(1), _code(x.dtype), m, H, N, K, gate.data_ptr() if gate is not None else None, gate_row, 1 if self.force_linear == 1 else 0, self._stream())
         return out
 
     # ---- mixture of experts ------------------------------------------------------------------------------------
@@ -743,6 +795,40 @@ class HipOps:
                    kv_heads, dk, dv, float(q_scale), n_chunks, ws.data_ptr() if ws is not None else None, nbytes, self._stream())
         return y
 
+    LINEAR_CHUNK = 64              # tokens of a chunk (the kernel library's)
+    LINEAR_CHUNKS_FROM = 16        # rows of the longest sequence from which a bfloat16 step runs in chunks
+    MAX_LINEAR_VALUES = 512
+
+    def linear_scan(self, q, k, v, decay, state, slot_ids, cu_rows, max_count, heads, dk, dv, chunks=None):
+        """S <- decay S + v k^T, o = S q, row after row of every sequence from state[slot] (float32 [slots, heads, dv, dk]),
+        which is left updated.  q, k [M, heads dk], v [M, heads dv]: views of wider rows of one dtype; decay float32 [heads].
+        Returns float32 [M, heads dv].  chunks: as in `delta_scan`."""
+        self._dev(q, k, v, decay, state, slot_ids, cu_rows)
+        m = q.shape[0]
+        qs, ks, vs = self._rows(q, "linear_scan q"), self._rows(k, "linear_scan k"), self._rows(v, "linear_scan v")
+        if tuple(q.shape) != (m, heads * dk) or tuple(k.shape) != (m, heads * dk) or tuple(v.shape) != (m, heads * dv) or not (q.dtype == k.dtype == v.dtype):
+            raise KernelError(f"linear_scan: q, k {(m, heads * dk)} and v {(m, heads * dv)} of one dtype")
+        if dk > self.MAX_SCAN_DIM or dv > self.MAX_LINEAR_VALUES:
+            raise KernelError(f"linear_scan: heads of {dk} x {dv} exceed {self.MAX_SCAN_DIM} x {self.MAX_LINEAR_VALUES}")
+        if decay.dtype != torch.float32 or decay.numel() != heads or not decay.is_contiguous():
+            raise KernelError(f"linear_scan: the decays must be contiguous float32 [{heads}]")
+        if state.dtype != torch.float32 or state.dim() != 4 or tuple(state.shape[1:]) != (heads, dv, dk) or not state.is_contiguous():
+            raise KernelError(f"linear_scan: the state must be contiguous float32 [slots, {heads}, {dv}, {dk}]")
+        n_seq = self._geometry("linear_scan", m, slot_ids, cu_rows)
+        can = q.dtype == torch.bfloat16 and dk % 8 == 0 and dv % 8 == 0 and all(t.data_ptr() % 16 == 0 and st % 8 == 0 for t, st in ((q, qs), (k, ks), (v, vs)))
+        if chunks is None:
+            chunks = can and int(max_count) >= self.LINEAR_CHUNKS_FROM
+        elif chunks and not can:
+            raise KernelError("linear_scan: chunks need bfloat16 rows of whole 16-byte pieces")
+        n_chunks = -(-int(max_count) // self.LINEAR_CHUNK) if chunks else 0
+        nbytes = self.lib.tp_linear_scan_workspace_bytes(n_seq, n_chunks, heads, dk, dv) if chunks else 0
+        ws = torch.empty(nbytes, dtype=torch.uint8, device=self.device) if nbytes else None
+        y = torch.empty((m, heads * dv), dtype=torch.float32, device=self.device)
+        self._call(self.lib, "tp_linear_scan", q.data_ptr(), qs, k.data_ptr(), ks, v.data_ptr(), vs, _code(q.dtype), decay.data_ptr(),
+                   state.data_ptr(), slot_ids.data_ptr(), cu_rows.data_ptr(), y.data_ptr(), n_seq, heads, dk, dv, n_chunks,
+                   ws.data_ptr() if ws is not None else None, nbytes, self._stream())
+        return y
+
     def pair_norm_mean(self, a, b, gain_a, gain_b, eps):
         """float32 [M, D]: 0.5 (a / rms(a) * gain_a + b / rms(b) * gain_b), each row over its own root mean square."""
         self._dev(a, b, gain_a, gain_b)
@@ -796,7 +882,10 @@ class HipOps:
     MAX_SLICED_WIDTH = 8192        # widest row `add_rms_norm` takes in K slices
 
     def rows(self, rows, dtype):
-        """A tensor of `dtype` from what `linear` returned: K slices are added in slice order."""
+        """A tensor of `dtype` from what `linear` returned: K slices are added in slice order.  (Of WeightedRows: their sum,
+        float32.)"""
+        if isinstance(rows, WeightedRows):
+            return self.weighted_sum(self.rows(rows.a, torch.float32).float(), rows.wa, self.rows(rows.b, torch.float32).float(), rows.wb)
         if not isinstance(rows, SplitRows):
             return rows
         sl = rows.slices
@@ -1008,11 +1097,14 @@ class HipOps:
                    ws.data_ptr() if ws is not None else None, nbytes, 0, algo, self._stream())
         return out
 
-    def linear_act(self, x, w, out_dtype, activation):
-        """act(x @ w^T), the activation applied to the float32 sums before they are rounded; one of PLAIN_ACTIVATIONS."""
+    def linear_act(self, x, w, out_dtype, activation, columns=None):
+        """act(x @ w^T), the activation applied to the float32 sums before they are rounded; one of PLAIN_ACTIVATIONS.
+        columns: only the first so many columns pass it (silu alone knows this), the others are the product's."""
+        if columns is not None and activation != "silu":
+            raise KernelError(f"linear_act: '{activation}' is applied to every column")
         if activation not in PLAIN_ACTIVATIONS:
             raise KernelError(f"linear_act: activation '{activation}' has no kernel ({', '.join(PLAIN_ACTIVATIONS)})")
-        return self._linear(x, w, out_dtype, PLAIN_ACTIVATIONS[activation], 0.0, 0)
+        return self._linear(x, w, out_dtype, PLAIN_ACTIVATIONS[activation], 0.0, w.shape[0] if columns is None else int(columns))
 
     def linear(self, x, w, out_dtype, softcap=None, defer=False, bias=None, out=None):
         """x @ w^T (+ bias).  defer: the caller hands the result to `add_rms_norm` (or through `rows()`), so a product
@@ -1050,6 +1142,34 @@ class HipOps:
     # ---- attention -------------------------------------------------------------------------------------
     DECODE_GROUP = 16              # query heads per kv head the matrix-core decode kernel takes
 
+    def _positional(self, what, by_position, H, rows, step=None):
+        """The kernel library's form of a `ByPosition` (None: none of it).  step: (rows, dtype, slices, slice stride, row
+        stride) of a fused decode step's projections, which hold the gates as columns."""
+        if by_position is None:
+            return None
+        b, s = by_position, _PositionalStruct(gate_slices=1)
+        if b.temperature is not None:
+            s.temp_coef, s.temp_every = float(b.temperature[0]), int(b.temperature[1])
+            if s.temp_every < 1:
+                raise KernelError(f"{what}: a query temperature that changes every {s.temp_every} positions")
+        if b.bias is not None:
+            self._dev(b.bias)
+            if b.bias.dtype != torch.float32 or b.bias.dim() != 2 or b.bias.shape[0] != H or not b.bias.is_contiguous():
+                raise KernelError(f"{what}: the biases must be contiguous float32 [{H}, distances]")
+            s.bias, s.reach = b.bias.data_ptr(), b.bias.shape[1] - 1
+        if b.gate is not None:
+            if step is not None:
+                base, dtype, slices, slice_stride, row_stride = step
+                s.gate = base + int(b.gate) * (4 if dtype == torch.float32 else 2)
+                s.gate_f32, s.gate_slices, s.gate_slice_stride, s.gate_stride = int(dtype == torch.float32), slices, slice_stride, row_stride
+            else:
+                self._dev(b.gate)
+                s.gate_stride = self._rows(b.gate, what + " gates")
+                if tuple(b.gate.shape) != (rows, H):
+                    raise KernelError(f"{what}: gates must be {(rows, H)}")
+                s.gate, s.gate_f32 = b.gate.data_ptr(), 1 - _code(b.gate.dtype)
+        return s
+
     def _fast_attention(self, dtype, H, KV, hd, decode=True):
         """Whether the matrix-core kernels take this geometry; the kernel of many queries takes any number of query
         heads per kv head, the decode kernel up to DECODE_GROUP."""
@@ -1058,7 +1178,7 @@ class HipOps:
 
     def attention_prefill(self, q, k, v, H, KV, hd, cu_rows, max_count, scale, softcap, window, out_dtype,
                           row_seq=None, row_pos=None, cached=None, shape=0, wide_weights=False, chunk=0, head_scale=None, sink=None,
-                          keep=0, pin=0):
+                          keep=0, pin=0, by_position=None):
         """Causal attention of the step's queries over the step's own rows of keys and values and, with
         `cached` = (new_len, table, k_pool, v_pool, rows_cap), over the positions before them, read in place from the
         cache as earlier steps left it (the step's own rows are not looked for there).  Without `cached` every sequence
@@ -1068,7 +1188,8 @@ class HipOps:
         terms) instead of 8; the plain kernel's weights are float32 in any case.
         chunk C: a query at position p sees keys from floor(p / C) C on only.  head_scale, sink: float32 [H], a factor on
         every head's scores and a score without key or value in every head's softmax.  keep: the first keep positions are
-        seen beside the window; pin: the rows of the cache in front of its ring that hold them (`CacheSite.pinned`)."""
+        seen beside the window; pin: the rows of the cache in front of its ring that hold them (`CacheSite.pinned`).
+        by_position: a `ByPosition`."""
         self._dev(q, k, v, cu_rows, head_scale, sink)
         self._head_vectors("attention_prefill", H, chunk, head_scale, sink)
         m = q.shape[0]
@@ -1086,13 +1207,15 @@ class HipOps:
             self._check_pools("attention_prefill", q.dtype, n_seq, KV, hd, new_len, table, k_pool, v_pool)
             page, table_w, rows_cap = k_pool.shape[2], table.shape[1], rows_cap or 0
         ptr = lambda t: t.data_ptr() if t is not None else None
+        pos = self._positional("attention_prefill", by_position, H, m)
+        pos_ref = _c.byref(pos) if pos is not None else None
         out = torch.empty((m, H * hd), dtype=out_dtype, device=self.device)
         if self._fast_attention(q.dtype, H, KV, hd, decode=False) and (cached is None or (page >= 16 and page & (page - 1) == 0)):
-            lib = self.attn_lib(hd, wide=wide_weights)
+            lib = self.attn_lib(hd, wide=wide_weights, by_position=pos is not None)
             self._call(lib, "tp_attn_prefill", q.data_ptr(), qs, k.data_ptr(), ks, v.data_ptr(), vs,
                        m, H, KV, cu_rows.data_ptr(), n_seq, int(max_count), ptr(new_len), ptr(table), table_w,
                        ptr(k_pool), ptr(v_pool), page, rows_cap,
-                       float(scale), float(softcap), int(window), int(chunk), ptr(head_scale), ptr(sink), int(keep), int(pin), out.data_ptr(), int(shape),
+                       float(scale), float(softcap), int(window), int(chunk), ptr(head_scale), ptr(sink), int(keep), int(pin), pos_ref, out.data_ptr(), int(shape),
                        self._stream())
             return out
         if cached is not None and (row_seq is None or row_pos is None):
@@ -1104,7 +1227,8 @@ class HipOps:
         self._call(self.lib, "tp_attn_simple_prefill", q.data_ptr(), qs, k.data_ptr(), ks, v.data_ptr(), vs, _code(q.dtype),
                    m, H, KV, hd, cu_rows.data_ptr(), row_seq.data_ptr(), row_pos.data_ptr(), ptr(new_len), ptr(table), table_w,
                    ptr(k_pool), ptr(v_pool), page, rows_cap, float(scale), float(softcap),
-                   int(window), int(chunk), ptr(head_scale), ptr(sink), int(keep), int(pin) if cached is not None else 0, out.data_ptr(), self._stream())
+                   int(window), int(chunk), ptr(head_scale), ptr(sink), int(keep), int(pin) if cached is not None else 0, pos_ref,
+                   out.data_ptr(), self._stream())
         return out
 
     def _head_vectors(self, what, H, chunk, head_scale, sink):
@@ -1137,13 +1261,14 @@ class HipOps:
 
     def attention_decode(self, q, H, KV, hd, new_len, table, k_pool, v_pool, rows_cap, scale, softcap, window,
                          out_dtype, max_keys=None, splits=None, head_groups=None, chunk=0, head_scale=None, sink=None,
-                         keep=0, pin=0):
+                         keep=0, pin=0, by_position=None):
         """head_groups: cut the query heads into that many groups (a multiple of KV), each read the pool head
         `group % KV` by a block of its own: for caches whose one kv head serves many heads, where one block would
         otherwise form all their weighted sums.  The plain kernel takes any grouping as it is.
-        chunk, head_scale, sink, keep, pin: as in `attention_prefill`."""
+        chunk, head_scale, sink, keep, pin, by_position: as in `attention_prefill`."""
         self._dev(q, new_len, table, k_pool, v_pool, head_scale, sink)
-        per_head = self._head_vectors("attention_decode", H, chunk, head_scale, sink) or keep > 0
+        self._head_vectors("attention_decode", H, chunk, head_scale, sink)
+        own_groups = bool(chunk) or head_scale is not None or keep > 0 or by_position is not None     # what groups of heads on one pool head have no kernel for
         n = q.shape[0]
         qs = self._rows(q, "attention q")
         if q.shape[1] != H * hd:
@@ -1152,10 +1277,12 @@ class HipOps:
         out = torch.empty((n, H * hd), dtype=out_dtype, device=self.device)
         page = k_pool.shape[2]
         groups = int(head_groups) if head_groups else KV
+        pos = self._positional("attention_decode", by_position, H, n)
+        pos_ref = _c.byref(pos) if pos is not None else None
         if groups % KV or H % groups:
             raise KernelError(f"attention_decode: {H} heads in {groups} groups on {KV} kv heads")
-        if self._fast_attention(q.dtype, H, groups, hd) and page >= 16 and page & (page - 1) == 0 and not (per_head and groups != KV):
-            lib = self.attn_lib(hd)
+        if self._fast_attention(q.dtype, H, groups, hd) and page >= 16 and page & (page - 1) == 0 and not (own_groups and groups != KV):
+            lib = self.attn_lib(hd, by_position=pos is not None)
             keys = int(max_keys) if max_keys else k_pool.shape[0] * k_pool.shape[2]
             nsplit = int(splits) if splits else self.decode_splits(n, groups, hd, keys)
             floats = lib.tp_attn_decode_workspace_floats(n, H, nsplit)
@@ -1163,19 +1290,19 @@ class HipOps:
             if groups != KV:
                 self._call(lib, "tp_attn_decode_shared", q.data_ptr(), qs, n, H, groups, KV, new_len.data_ptr(), table.data_ptr(),
                            table.shape[1], k_pool.data_ptr(), v_pool.data_ptr(), k_pool.shape[2], rows_cap, float(scale),
-                           float(softcap), int(window), out.data_ptr(), ws.data_ptr() if ws is not None else None, nsplit,
-                           self._stream())
+                           float(softcap), int(window), sink.data_ptr() if sink is not None else None, out.data_ptr(),
+                           ws.data_ptr() if ws is not None else None, nsplit, self._stream())
                 return out
             self._call(lib, "tp_attn_decode", q.data_ptr(), qs, n, H, KV, new_len.data_ptr(), table.data_ptr(),
                        table.shape[1], k_pool.data_ptr(), v_pool.data_ptr(), k_pool.shape[2], rows_cap, float(scale),
                        float(softcap), int(window), int(chunk), head_scale.data_ptr() if head_scale is not None else None,
-                       sink.data_ptr() if sink is not None else None, int(keep), int(pin), out.data_ptr(), ws.data_ptr() if ws is not None else None, nsplit,
-                       self._stream())
+                       sink.data_ptr() if sink is not None else None, int(keep), int(pin), pos_ref, out.data_ptr(),
+                       ws.data_ptr() if ws is not None else None, nsplit, self._stream())
             return out
         self._call(self.lib, "tp_attn_simple_decode", q.data_ptr(), qs, _code(q.dtype), n, H, KV, hd, new_len.data_ptr(),
                    table.data_ptr(), table.shape[1], k_pool.data_ptr(), v_pool.data_ptr(), k_pool.shape[2], rows_cap,
                    float(scale), float(softcap), int(window), int(chunk), head_scale.data_ptr() if head_scale is not None else None,
-                   sink.data_ptr() if sink is not None else None, int(keep), int(pin), out.data_ptr(), self._stream())
+                   sink.data_ptr() if sink is not None else None, int(keep), int(pin), pos_ref, out.data_ptr(), self._stream())
         return out
 
     def fuses_decode_step(self, dtype, H, KV, hd, k_pool):
@@ -1184,17 +1311,21 @@ class HipOps:
         return self._fast_attention(dtype, H, KV, hd) and page >= 16 and page & (page - 1) == 0
 
     def attention_decode_step(self, qkv, H, KV, hd, inv_freq, rotary_dim, new_len, table, k_pool, v_pool, rows_cap,
-                              scale, softcap, window, out_dtype, max_keys=None, write_kv=True, splits=None, sink=None, keep=0, pin=0):
+                              scale, softcap, window, out_dtype, max_keys=None, write_kv=True, splits=None, sink=None, keep=0, pin=0,
+                              by_position=None):
         """A decode step's rotation, cache write and attention in one launch.  qkv: each sequence's projections
         [queries | keys | values] (queries only when write_kv is false), a bf16 tensor or what
-        `linear(..., defer=True)` returned; sequence i's token has position new_len[i] - 1.  sink, keep, pin: as in `attention_prefill`."""
+        `linear(..., defer=True)` returned; sequence i's token has position new_len[i] - 1.  sink, keep, pin, by_position: as in
+        `attention_prefill` (its gate: the first of H further columns of the rows)."""
         self._head_vectors("attention_decode_step", H, 0, None, sink)
         self._dev(sink)
         split = isinstance(qkv, SplitRows)
         rows = qkv.slices if split else qkv
         self._dev(rows, inv_freq, new_len, table, k_pool, v_pool)
         n, width = rows.shape[-2], rows.shape[-1]
-        if width != (H + (2 * KV if write_kv else 0)) * hd:
+        gated = by_position is not None and by_position.gate is not None
+        need = (H + (2 * KV if write_kv else 0)) * hd
+        if (not gated and width != need) or (gated and not need <= by_position.gate <= width - H):
             raise KernelError(f"attention_decode_step: rows of {width} columns, {H} heads and {KV} kv heads of {hd} need "
                               f"{(H + (2 * KV if write_kv else 0)) * hd}")
         if out_dtype != torch.bfloat16 or not self.fuses_decode_step(out_dtype, H, KV, hd, k_pool):
@@ -1210,7 +1341,8 @@ class HipOps:
         if rotary_dim and (inv_freq is None or inv_freq.dtype != torch.float32 or inv_freq.numel() != rotary_dim // 2):
             raise KernelError(f"attention_decode_step: a rotation over {rotary_dim} needs float32 inv_freq [{rotary_dim // 2}]")
         self._check_pools("attention_decode_step", torch.bfloat16, n, KV, hd, new_len, table, k_pool, v_pool)
-        lib = self.attn_lib(hd)
+        pos = self._positional("attention_decode_step", by_position, H, n, step=(rows.data_ptr(), rows.dtype, n_slices, slice_stride, row_stride))
+        lib = self.attn_lib(hd, by_position=pos is not None)
         keys = int(max_keys) if max_keys else k_pool.shape[0] * k_pool.shape[2]
         nsplit = int(splits) if splits else self.decode_splits(n, KV, hd, keys)
         floats = lib.tp_attn_decode_workspace_floats(n, H, nsplit)
@@ -1220,7 +1352,8 @@ class HipOps:
                    inv_freq.data_ptr() if rotary_dim else None, int(rotary_dim), 1 if write_kv else 0,
                    n, H, KV, new_len.data_ptr(), table.data_ptr(), table.shape[1], k_pool.data_ptr(), v_pool.data_ptr(),
                    k_pool.shape[2], rows_cap, float(scale), float(softcap), int(window), sink.data_ptr() if sink is not None else None,
-                   int(keep), int(pin), out.data_ptr(), ws.data_ptr() if ws is not None else None, nsplit, self._stream())
+                   int(keep), int(pin), _c.byref(pos) if pos is not None else None, out.data_ptr(), ws.data_ptr() if ws is not None else None,
+                   nsplit, self._stream())
         return out
 
     # ---- token choice -------------------------------------------------------------------------------------

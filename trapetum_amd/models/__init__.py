@@ -1,2 +1,2 @@
 """Architectures; importing this package registers the built-in ones."""
-from . import besulix, gemma2, golepel, lutovik, solulix, vogunex   # noqa: F401
+from . import besulix, gemma2, golepel, kaderax, lutovik, solulix, vogunex   # noqa: F401

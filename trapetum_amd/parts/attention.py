@@ -49,6 +49,13 @@ values (y_t = sum_j w[:, j] u_(t - taps + 1 + j), zeros before the sequence; the
 state), before the rotation and the cache; `keep_first` F: beside the window the first F positions of the sequence stay
 visible, and the cache keeps them in rows in front of its ring; and a `sink` given as a number, the same score for
 every head (0: softmax with one added to its denominator).
+
+And three that make scores depend on positions without a rotation: `query_temperature` (coef, every): the query at p is
+multiplied by 1 + coef ln(floor((p + 1) / every) + 1); `distance_bias`: a table [B, heads] whose row bucket(n) is added to
+the scores, after the cap, of keys at distance n, with bucket(n) = n below B/2 and B/2 + floor(ln(n / (B/2)) / ln(D / (B/2)) (B - B/2)),
+at most B - 1, from there on (D = `bias_reach`; from D on the bias is one number, so the kernels get a table by distance of
+D + 1 entries per head); `output_gate="head"`: a head's output is multiplied by sigmoid(W_g x)_h, one number per head, whose
+product rides with the projections' as further columns.  All three are applied inside the attention kernels (`ops.ByPosition`).
 """
 from ..cache.store import TokenSpec
 from ..models.spec import TensorSpec
@@ -62,9 +69,10 @@ class Attention(Mixer):
                  precise_weights=False,
                  tensors=("q_proj.weight", "k_proj.weight", "v_proj.weight", "o_proj.weight", "g_proj.weight"),
                  bias_suffix=None, chunk=None, head_temperature=None, sink=None, value_rotation=None,
-                 unit_norm_eps=None, pool=None, talk=None, conv=None, conv_suffix=".conv", keep_first=0):
+                 unit_norm_eps=None, pool=None, talk=None, conv=None, conv_suffix=".conv", keep_first=0,
+                 query_temperature=None, distance_bias=None, bias_reach=None, bias_rows=32):
         """value_dim: elements of a value head when they differ from a key's head_dim.  output_gate: the heads' outputs
-        are multiplied by sigmoid(W_g x) before the output projection.  own_kv False: the layer has no key and value
+        are multiplied by sigmoid(W_g x) before the output projection, element by element (True) or each head by one number ("head").  own_kv False: the layer has no key and value
         projections; its schedule entry names the run whose cache it reads.  precise_weights: the softmax weights meet
         the values with 16 bits of mantissa or more in every kernel (the kernel of many queries rounds them to bfloat16
         otherwise; a decode step's are float32 anyway).  tensors: local names of W_q, W_k, W_v, W_o (and W_g).
@@ -74,7 +82,8 @@ class Attention(Mixer):
         no such norm).  pool: positions per pooled block before the window.  talk: local name of the matrix
         [heads, heads] that mixes the heads' softmax weights.  conv: taps of the convolutions over time on q, k and v, named
         like their matrices with conv_suffix (None: none).  keep_first: positions at a sequence's start that stay visible
-        beside the window."""
+        beside the window.  query_temperature: (coef, every).  distance_bias: local name of the table [B, heads], whose number
+        of rows the checkpoint gives (bias_rows is what a random model takes); bias_reach: the distance D it reaches to."""
         if num_heads % num_kv_heads:
             raise ValueError(f"{num_heads} query heads are no multiple of {num_kv_heads} kv heads")
         self.hidden_size = hidden_size
@@ -89,7 +98,10 @@ class Attention(Mixer):
         self.query_scale = float(query_scale)
         self.softcap = float(softcap) if softcap else 0.0
         self.window = int(window) if window else 0
-        self.output_gate = bool(output_gate)
+        if output_gate not in (False, True, "head"):
+            raise ValueError(f"an output gate is per element (True) or per head ('head'), not {output_gate!r}")
+        self.output_gate = output_gate is True
+        self.head_gate = output_gate == "head"
         self.own_kv = bool(own_kv)
         self.precise_weights = bool(precise_weights)
         self.names = dict(zip(("q", "k", "v", "o", "g"), tuple(tensors) + ("g_proj.weight",) * (5 - len(tensors))))
@@ -121,6 +133,16 @@ class Attention(Mixer):
             raise ValueError("first positions are kept beside a window, by an attention on its own cache, without chunks or pooled blocks")
         if self.taps and (self.pooled or not self.own_kv or bias_suffix):
             raise ValueError("convolutions go with an attention on its own cache, without biases, unit norms, pooled blocks or talking heads")
+        self.query_temperature = None if query_temperature is None else (float(query_temperature[0]), int(query_temperature[1]))
+        self.bias_name, self.bias_reach, self.bias_rows = distance_bias, None if bias_reach is None else int(bias_reach), int(bias_rows)
+        self.by_position = self.query_temperature is not None or self.bias_name is not None or self.head_gate
+        if self.query_temperature is not None and self.query_temperature[1] < 1:
+            raise ValueError(f"a query temperature changes every so many positions, not every {self.query_temperature[1]}")
+        if self.bias_name is not None and not (self.bias_reach and self.bias_reach > 0):
+            raise ValueError("a bias by distance needs the distance it reaches to")
+        if self.by_position and (self.pooled or not self.own_kv or self.taps or bias_suffix or value_rotation is not None):
+            raise ValueError("temperatures by position, biases by distance and gates per head go with an attention on its own cache, "
+                             "without convolutions, projection biases, rotated values, unit norms, pooled blocks or talking heads")
         if self.pool and not self.window:
             raise ValueError("pooled blocks stand before a window: the layer needs one")
 
@@ -138,6 +160,10 @@ class Attention(Mixer):
             specs[n["v"]] = TensorSpec((self.num_kv_heads * self.value_dim, d))
         if self.output_gate:
             specs[n["g"]] = TensorSpec((self.num_heads * self.value_dim, d))
+        if self.head_gate:
+            specs[n["g"]] = TensorSpec((self.num_heads, d))
+        if self.bias_name:
+            specs[self.bias_name] = TensorSpec((self.bias_rows, self.num_heads), init="norm", free=(0,))
         if self.bias_suffix:
             for s in ("q", "k", "v") if self.own_kv else ("q",):
                 specs[n[s] + self.bias_suffix] = TensorSpec((specs[n[s]].shape[0],), init="norm")
@@ -195,7 +221,14 @@ class Attention(Mixer):
         parts = [self._heads(tensors[n["q"]], H, self.head_dim, turned=True)]
         if self.own_kv:
             parts += [self._heads(tensors[n["k"]], KV, self.head_dim, turned=True), self._heads(tensors[n["v"]], KV, self.value_dim)]
+        self.gate_column = sum(p.shape[0] for p in parts)
+        if self.head_gate:                                   # further columns of the product, which ends on whole 16-byte pieces
+            parts.append(tensors[n["g"]])
+            spare = -sum(p.shape[0] for p in parts) % 8
+            if spare:
+                parts.append(parts[-1].new_zeros((spare, self.hidden_size)))
         self.w_qkv = rt.matrix(torch.cat(parts, dim=0)).contiguous()
+        self.distance_table = self._table_by_distance(tensors[self.bias_name]) if self.bias_name else None
         self.w_g = rt.matrix(self._heads(tensors[n["g"]], H, self.value_dim).contiguous()) if self.output_gate else None
         w_o = tensors[n["o"]]
         if self.value_dim < self.row:
@@ -224,6 +257,28 @@ class Attention(Mixer):
         if self.value_position is not None:
             self.value_freq = self.value_position.inv_freq(rt.device)
             self.value_back = (-self.value_freq).contiguous()            # the same angles the other way round
+
+    @staticmethod
+    def bucket_of_distance(n, rows, reach):
+        """The row of a table of `rows` that a key at distance n >= 0 reads."""
+        import math
+        half = rows // 2
+        if n < half:
+            return n
+        return min(rows - 1, half + math.floor(math.log(n / half) / math.log(reach / half) * (rows - half)))
+
+    def _table_by_distance(self, table):
+        """[B, heads] -> float32 [heads, D + 1]: the bias of every distance; the last entry's is that of all farther keys."""
+        rows, D = table.shape[0], self.bias_reach
+        if rows < 2 or D <= rows // 2:
+            raise ValueError(f"a bias table of {rows} rows does not reach to a distance of {D}")
+        index = [self.bucket_of_distance(n, rows, D) for n in range(D + 1)]
+        return table.float()[index].t().contiguous()
+
+    def _positional(self, ctx, gate):
+        if not self.by_position:
+            return {}
+        return {"by_position": ctx.ops.ByPosition(self.query_temperature, self.distance_table, gate if self.head_gate else None)}
 
     def _project_out(self, ctx, x, out):
         if self.output_gate:
@@ -285,6 +340,8 @@ class Attention(Mixer):
         owns_cache = ctx.cache_owner == ctx.entry
         if self.taps and not owns_cache:
             raise ValueError("an attention with convolutions runs on its own cache")
+        if self.by_position and not owns_cache:
+            raise ValueError("an attention with scores by position or gates per head runs on its own cache")
         if owns_cache and not self.own_kv:
             raise ValueError("an attention without key and value projections must read another run's cache")
         w_in = self.w_qkv if owns_cache else self.w_qkv[:Q]          # a run on another run's cache projects its queries only
@@ -307,16 +364,18 @@ class Attention(Mixer):
             out = ops.attention_decode_step(qkv, H, KV, hd, self.inv_freq, self.position.rotary_dim, ctx.new_len,
                                             table, k_pool, v_pool, rows_cap, self.query_scale, self.softcap,
                                             self.window, ctx.dtype, max_keys=ctx.max_rows_visible(site), write_kv=owns_cache,
-                                            **(dict(sink=self.sink) if self.sink is not None else {}), **kept)
+                                            **(dict(sink=self.sink) if self.sink is not None else {}), **kept,
+                                            **self._positional(ctx, self.gate_column))
             return self._project_out(ctx, x, out)
         if self.taps:
             qkv = self._convolved(ctx, x, w_in)
         else:
             qkv = ops.linear(x, w_in, ctx.dtype, bias=bias) if bias is not None else ops.linear(x, w_in, ctx.dtype)
         if owns_cache:
-            q, k, v = qkv[:, :Q], qkv[:, Q:Q + KVD], qkv[:, Q + KVD:]
+            q, k, v = qkv[:, :Q], qkv[:, Q:Q + KVD], qkv[:, Q + KVD:Q + 2 * KVD]
         else:
             q, k, v = qkv, None, None
+        more.update(self._positional(ctx, qkv[:, self.gate_column:self.gate_column + H]))
         if self.value_freq is not None:
             self._turn(ctx, v, KV, self.value_freq)
         # Sequences that go on by several tokens (or some start while others go on) see cached positions and the

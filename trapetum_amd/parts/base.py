@@ -26,7 +26,9 @@ step (`forward`).  Interfaces:
                of the fp32 stream when a short causal convolution over time stands in front of it.
   StreamAdd    operands(ctx) -> (vec, origin): what a model adds to the stream before a run of a layer, a float32 vector
                [hidden] for every row and float32 rows [M, hidden] (either may be None); `needs_origin` asks the engine
-               to keep the embedding's rows for the step (`ctx.origin`).
+               to keep the embedding's rows for the step (`ctx.origin`).  With `replaces` it makes the stream anew instead:
+               forward(ctx, stream, a, b, wa, wb, gain, eps, dtype) brings stream + wa a + wb b to its new values, in
+               place, and returns their norm.
   Embedding    forward(ctx, tokens) -> fp32 stream;  Head  forward(ctx, rows) -> fp32 logits.
 
 `ctx` is the step's StepContext: batch geometry on the device, the kernels
@@ -126,6 +128,7 @@ class Conv(Part):
 
 class StreamAdd(Part):
     needs_origin = False
+    replaces = False
 
     def operands(self, ctx):
         raise NotImplementedError

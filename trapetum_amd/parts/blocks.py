@@ -5,7 +5,8 @@ sandwich  x += post_mixer_norm(mixer(pre_mixer_norm(x)));
 pre_norm  x += mixer(pre_mixer_norm(x));  x += ff(pre_ff_norm(x)); the feed-forward may be absent
           (the reference's other layer type, runtime/src/lib.rs:721-730).  With `token_shift` the mixer reads
           h + (h' - h) * w instead of h = pre_mixer_norm(x), h' being the h of the token before (zeros before the
-          sequence) and w a vector of the layer; the last token's h is a state of the sequence.
+          sequence) and w a vector of the layer; the last token's h is a state of the sequence.  With `residual_scale` m
+          a sub-layer's output is multiplied by m before it is added.
 post_norm x += post_mixer_norm(mixer(c1(x)));  x += post_ff_norm(ff(c2(x))): no norm in front of a sub-layer; c1
           and c2 are what it reads of the stream, the stream itself or (input_conv) the stream through a short
           causal convolution whose last rows are a state of the sequence.  The feed-forward may be absent.
@@ -22,9 +23,17 @@ from ..registry import register_part
 from .base import Block
 
 
-def add_then_norm(ctx, stream, rows, post, nxt):
-    """stream += post(rows) (or rows); returns nxt(stream) (or None).  One kernel when both norms
+def add_then_norm(ctx, stream, rows, post, nxt, scale=1.0):
+    """stream += scale * post(rows) (or rows); returns nxt(stream) (or None).  One kernel when both norms
     expose an RMS gain, else the norms' own forward around a plain add."""
+    pair = isinstance(rows, ctx.ops.WeightedRows)
+    if post is None and (pair or scale != 1.0):          # constants on the rows: the kernel that adds two operands takes them
+        a, wa, b, wb = (rows.a, rows.wa, rows.b, rows.wb) if pair else (rows, 1.0, None, 1.0)
+        return join_then_norm(ctx, stream, a, b, nxt, wa * scale, wb * scale)
+    if scale != 1.0:
+        raise ValueError("a residual scale goes with blocks that do not norm a sub-layer's output")
+    if pair:
+        rows = ctx.ops.rows(rows, ctx.dtype)
     if isinstance(nxt, NormAfterAdd):
         if post is None:
             return join_then_norm(ctx, stream, rows, None, nxt)
@@ -56,17 +65,18 @@ class NormAfterAdd:
         return join_then_norm(ctx, stream, None, None, self)
 
 
-def join_then_norm(ctx, stream, a, b, nxt):
-    """stream += a + b (either may be None) and what `nxt` adds before its norm; returns its norm of the stream (or None)."""
-    vec = origin = None
-    norm = nxt
-    if isinstance(nxt, NormAfterAdd):
-        norm = nxt.norm
-        vec, origin = nxt.added.operands(ctx)
+def join_then_norm(ctx, stream, a, b, nxt, wa=1.0, wb=1.0):
+    """stream += wa a + wb b (either may be None) and what `nxt` does to the stream before its norm; returns its norm of the
+    stream (or None)."""
+    norm = nxt.norm if isinstance(nxt, NormAfterAdd) else nxt
     plain = norm is None or (norm.gain is not None and getattr(norm, "groups", 1) == 1)
     dtype = getattr(norm, "reader_dtype", None) or ctx.dtype
     gain, eps = (norm.gain, norm.eps) if plain and norm is not None else (None, 0.0)
-    out = ctx.ops.join_rms_norm(stream, a, b, gain, eps, dtype, vec=vec, origin=origin)
+    if isinstance(nxt, NormAfterAdd) and nxt.added.replaces:
+        out = nxt.added.forward(ctx, stream, a, b, wa, wb, gain, eps, dtype)
+    else:
+        vec, origin = nxt.added.operands(ctx) if isinstance(nxt, NormAfterAdd) else (None, None)
+        out = ctx.ops.join_rms_norm(stream, a, b, gain, eps, dtype, vec=vec, origin=origin, wa=wa, wb=wb)
     return out if plain else norm.forward(ctx, stream, getattr(norm, "reader_dtype", None))
 
 
@@ -104,8 +114,10 @@ class SandwichBlock(Block):
 
 
 class PreNormBlock(Block):
-    def __init__(self, mixer, feed_forward, make_norm, token_shift=None):
-        """token_shift: the local name of the mixing vector [hidden] (None: the mixer reads the normed rows as they are)."""
+    def __init__(self, mixer, feed_forward, make_norm, token_shift=None, residual_scale=1.0):
+        """token_shift: the local name of the mixing vector [hidden] (None: the mixer reads the normed rows as they are).
+        residual_scale: the constant a sub-layer's output is multiplied by."""
+        self.residual_scale = float(residual_scale)
         self.mixer = mixer
         self.feed_forward = feed_forward                 # None: the layer is its mixer behind its norm
         sites = self.norm_sites() if feed_forward is not None else self.norm_sites()[:1]
@@ -152,14 +164,14 @@ class PreNormBlock(Block):
         a = self.mixer.forward(ctx, x, site)
         ctx.dump("mixer_out", a)
         if self.feed_forward is None:
-            normed_next = add_then_norm(ctx, stream, a, None, next_norm)
+            normed_next = add_then_norm(ctx, stream, a, None, next_norm, self.residual_scale)
             ctx.dump("layer_out", stream)
             return stream, normed_next
-        x = add_then_norm(ctx, stream, a, None, n["pre_ff_norm"])
+        x = add_then_norm(ctx, stream, a, None, n["pre_ff_norm"], self.residual_scale)
         ctx.dump("after_mixer", stream)
         m = self.feed_forward.forward(ctx, x)
         ctx.dump("ff_out", m)
-        normed_next = add_then_norm(ctx, stream, m, None, next_norm)
+        normed_next = add_then_norm(ctx, stream, m, None, next_norm, self.residual_scale)
         ctx.dump("layer_out", stream)
         return stream, normed_next
 

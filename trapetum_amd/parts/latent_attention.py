@@ -14,7 +14,10 @@ token for all heads, instead of heads * (dim + vdim).
 
 Further parameters: `query_rank` (the queries go through a latent of their own, q = W_uq rmsnorm(W_dq h) * w_qnorm,
 instead of one product), `window` W (the query at p sees the positions p - W + 1 .. p; the cache then keeps a ring),
-`output_gate` (head h's output is multiplied by sigmoid(W_g h)_h, one number per head and token) and a rotation of
+`output_gate` (head h's output is multiplied by sigmoid(W_g h)_h, one number
+per head and token, or with `gate_per="element"` element by element with sigmoid(W_g h), W_g [H vdim, hidden], in the per-head
+product that forms the values' sums), a `sink` per head (a learned score without key or value that joins the softmax's
+denominator once), `joint_input` (W_dq, W_dkv and W_g are one product of the layer's input) and a rotation of
 neighbouring pairs (2f, 2f + 1), carried out as the rotation of halves on projection rows reordered at bind (queries
 and key part alike: every score is the same sum in another order).
 
@@ -33,11 +36,13 @@ class LatentAttention(Mixer):
     def __init__(self, hidden_size, num_heads, nope_dim, rope_dim, value_dim, latent_rank, scale, latent_eps,
                  position=("none", {}), own_latent=True,
                  tensors=("q", "dkv", "dkv.norm", "uk", "uv", "o"), query_rank=None, query_tensors=("dq", "dq.norm", "uq"),
-                 window=None, output_gate=None, precise_weights=False):
+                 window=None, output_gate=None, precise_weights=False, gate_per="head", sink=None, joint_input=False):
         """query_rank: size of the queries' latent (None: queries are one product, tensor `q`); query_tensors: local
         names of W_dq, the latent's gain and W_uq.  window: positions back a query sees, its own included (None: all).
         output_gate: local name of W_g [heads, hidden] (None: no gate).  precise_weights: softmax weights of 16 bits of
-        mantissa in the matrix-core kernel of many queries."""
+        mantissa in the matrix-core kernel of many queries.  gate_per: "head", or "element" with W_g [heads vdim, hidden].
+        sink: local name of a float vector [heads].  joint_input: one product for the queries' latent, the cached row and the
+        gate (needs a query latent, a latent of its own and a gate per element)."""
         self.hidden_size, self.num_heads = int(hidden_size), int(num_heads)
         self.nope_dim, self.rope_dim, self.value_dim, self.rank = int(nope_dim), int(rope_dim), int(value_dim), int(latent_rank)
         self.scale = float(scale)
@@ -50,7 +55,13 @@ class LatentAttention(Mixer):
         self.query_rank = int(query_rank) if query_rank else 0
         self.names.update(zip(("dq", "dq_norm", "uq"), query_tensors))
         self.window = int(window) if window else 0
-        self.gate_name = output_gate
+        self.gate_name, self.gate_per = output_gate, gate_per
+        self.sink_name = sink
+        self.joint_input = bool(joint_input)
+        if gate_per not in ("head", "element"):
+            raise ValueError(f"a gate is per head or per element, not per '{gate_per}'")
+        if self.joint_input and not (self.query_rank and self.own_latent and self.gate_name and gate_per == "element"):
+            raise ValueError("one input product needs a query latent, a latent of its own and a gate per element")
         self.precise_weights = bool(precise_weights)
 
     @property
@@ -67,7 +78,9 @@ class LatentAttention(Mixer):
         else:
             specs = {n["q"]: TensorSpec((qd, d))}
         if self.gate_name:
-            specs[self.gate_name] = TensorSpec((H, d))
+            specs[self.gate_name] = TensorSpec((H if self.gate_per == "head" else H * self.value_dim, d))
+        if self.sink_name:
+            specs[self.sink_name] = TensorSpec((H,), init="norm")
         specs.update({n["uk"]: TensorSpec((H * self.nope_dim, self.rank)), n["uv"]: TensorSpec((H * self.value_dim, self.rank)),
                  n["o"]: TensorSpec((d, H * self.value_dim))})
         if self.own_latent:
@@ -98,11 +111,18 @@ class LatentAttention(Mixer):
             self.w_dq = rt.matrix(tensors[n["dq"]].contiguous())
             self.query_gain = tensors[n["dq_norm"]].float().contiguous()
             self.w_uq = rt.matrix(wq.contiguous())
-            if self.own_latent:
+            if self.joint_input:                         # rows of whole 16-byte pieces: [cached row | gate | queries' latent]
+                parts = [tail, tensors[self.gate_name], tensors[n["dq"]]]
+                spare = -sum(p.shape[0] for p in parts) % 8
+                if spare:
+                    parts.append(tail.new_zeros((spare, tail.shape[1])))
+                self.w_joint, self.w_dq = rt.matrix(torch.cat(parts, dim=0).contiguous()), None
+            elif self.own_latent:
                 self.w_tail = rt.matrix(tail.contiguous())
         else:
             self.w_in = rt.matrix((torch.cat([wq, tail], dim=0) if self.own_latent else wq).contiguous())
-        self.w_gate = rt.matrix(tensors[self.gate_name].contiguous()) if self.gate_name else None
+        self.w_gate = rt.matrix(tensors[self.gate_name].contiguous()) if self.gate_name and not self.joint_input else None
+        self.sink = tensors[self.sink_name].float().contiguous() if self.sink_name else None
         self.w_absorb = rt.matrix(tensors[n["uk"]].reshape(H, dn, R).transpose(1, 2).contiguous())     # [H, rank, dim]
         self.w_up = rt.matrix(tensors[n["uv"]].reshape(H, dv, R).contiguous())                         # [H, vdim, rank]
         self.w_o = rt.matrix(tensors[n["o"]])
@@ -121,8 +141,12 @@ class LatentAttention(Mixer):
         rows_cap = site.rows_cap or 0
         m = x.shape[0]
         import torch
-        tail = None
-        if self.query_rank:
+        tail = gate = None
+        if self.joint_input:
+            joint = ops.linear(x, self.w_joint, ctx.dtype)
+            tail, gate, dq = joint[:, :row], joint[:, row:row + H * dv], joint[:, row + H * dv:row + H * dv + self.query_rank]
+            proj = ops.linear(ops.rms_norm(dq, self.query_gain, self.latent_eps, ctx.dtype), self.w_uq, ctx.dtype)
+        elif self.query_rank:
             cq = ops.rms_norm(ops.linear(x, self.w_dq, torch.float32), self.query_gain, self.latent_eps, ctx.dtype)
             proj = ops.linear(cq, self.w_uq, ctx.dtype)           # [M, H (dr + dn)]
             if owns:
@@ -131,6 +155,7 @@ class LatentAttention(Mixer):
             proj = ops.linear(x, self.w_in, ctx.dtype)            # [M, H (dr + dn) (+ dr + rank)]
         # A step that continues sequences by several tokens reads the ring as earlier steps left it, so its rows are
         # cached after the attention: in a ring they may take the places of positions that its first queries still see.
+        more = dict(sink=self.sink) if self.sink is not None else {}
         late = owns and ctx.mode == "extend" and bool(rows_cap)
         # rotations, the latent's norm and the cache write in one launch: the queries' rotated parts go to their
         # places in q, the step's rows [r | c] to `mine` and into the cache
@@ -149,7 +174,7 @@ class LatentAttention(Mixer):
             per = next(g for g in (self.DECODE_GROUP_LONG if keys >= self.LONG_KEYS else self.DECODE_GROUP, 4, 2, 1) if H % g == 0)
             out = ops.attention_decode(q, H, 1, row, ctx.new_len, table, pool, pool, rows_cap, self.scale, 0.0, self.window,
                                        ctx.dtype, max_keys=keys, head_groups=H // per,
-                                       splits=ops.decode_splits(m * (H // per), 1, row, keys))
+                                       splits=ops.decode_splits(m * (H // per), 1, row, keys), **more)
         else:
             if owns:
                 ctx.offer_step_rows(latent=mine)
@@ -159,12 +184,14 @@ class LatentAttention(Mixer):
             out = ops.attention_prefill(q, mine, mine, H, 1, row, ctx.cu_rows, ctx.max_count, self.scale, 0.0, self.window, ctx.dtype,
                                         row_seq=ctx.row_seq, row_pos=ctx.row_pos,
                                         cached=(ctx.new_len, table, pool, pool, rows_cap) if extend else None,
-                                        wide_weights=self.precise_weights)
+                                        wide_weights=self.precise_weights, **more)
             if late:
                 row_seq, row_pos, new_len = ctx.row_seq, ctx.row_pos, ctx.new_len
                 ctx.after_readers(lambda: ops.kv_write(mine, mine, 1, row, row_seq, row_pos, new_len, table, pool, pool, rows_cap))
-        heads = ops.head_linear(out.view(m, H, row)[:, :, dr:], self.w_up, None)      # [M, H, vdim]
-        if self.w_gate is not None:
+        if self.w_gate is not None and self.gate_per == "element":
+            gate = ops.linear(x, self.w_gate, ctx.dtype)
+        heads = ops.head_linear(out.view(m, H, row)[:, :, dr:], self.w_up, None, **(dict(gate=gate) if gate is not None else {}))      # [M, H, vdim]
+        if self.w_gate is not None and self.gate_per == "head":
             ops.mul_sigmoid_heads(heads.view(m, H * dv), ops.linear(x, self.w_gate, torch.float32), H)
         return ops.linear(heads.view(m, H * dv), self.w_o, ctx.dtype, defer=True)
 

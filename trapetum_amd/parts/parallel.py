@@ -2,7 +2,8 @@
 
 combine "norm_mean": each output is divided by its root mean square over the model width and multiplied by a gain of
 its own (used as stored), in float32, before the two are averaged.  combine "weighted_sum": the outputs are added as
-they are, in float32, each times a constant of the model (`weights`); there are no gains.  The two mixers are any registered mixers; at most one of them may
+they are, in float32, each times a constant of the model (`weights`); there are no gains.  With `deferred` that sum is left
+to the block's add (`ops.WeightedRows`), each side's last product in the form it has (K slices too).  The two mixers are any registered mixers; at most one of them may
 keep tensors per token (it becomes this mixer's cache, so that another layer's run can read it), and the states they
 declare by name are kept under "left." and "right.".
 """
@@ -14,7 +15,7 @@ from .base import Mixer
 
 class ParallelMixers(Mixer):
     def __init__(self, hidden_size, left, right, eps=0.0, prefixes=("left.", "right."), tensors=("left.out", "right.out"),
-                 combine="norm_mean", weights=(1.0, 1.0)):
+                 combine="norm_mean", weights=(1.0, 1.0), deferred=False):
         if combine not in ("norm_mean", "weighted_sum"):
             raise ValueError(f"two mixers side by side are combined by norm_mean or weighted_sum, not '{combine}'")
         self.hidden_size, self.eps = int(hidden_size), float(eps)
@@ -22,7 +23,10 @@ class ParallelMixers(Mixer):
         self.prefixes = tuple(prefixes)
         self.combine, self.weights = combine, tuple(float(w) for w in weights)
         self.names = tuple(tensors) if combine == "norm_mean" else ()
-        if combine == "weighted_sum":
+        self.deferred = bool(deferred)
+        if self.deferred and combine != "weighted_sum":
+            raise ValueError("only a weighted sum can be left to the block's add")
+        if combine == "weighted_sum" and not self.deferred:
             import torch
             for m in self.sides:                     # the sum is formed in float32 from float32 products where a side can give them
                 if hasattr(m, "output_dtype"):
@@ -60,6 +64,9 @@ class ParallelMixers(Mixer):
 
     def forward(self, ctx, x, site):
         ops = ctx.ops
+        if self.deferred:
+            a, b = (m.forward(ctx, x, site) for m in self.sides)
+            return ops.WeightedRows(a, self.weights[0], b, self.weights[1])
         if self.combine == "weighted_sum":
             import torch
             a, b = (ops.rows(m.forward(ctx, x, site), torch.float32) for m in self.sides)
