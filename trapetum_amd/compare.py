@@ -1,7 +1,7 @@
 """Two designs side by side at equal layer sizes: Golepel or Lutovik next to Gemma-2, Besulix, Vogunex or Solulix next to
-Lutovik, random weights, one MI355X.
+Lutovik, Kaderax next to Vogunex and Lutovik, random weights, one MI355X.
 
-    python bench.py --compare golepel|lutovik|besulix|vogunex|solulix [--sizes 2b|9b] [--layers L] [--steps K] [--warmup W]
+    python bench.py --compare golepel|lutovik|besulix|vogunex|solulix|kaderax [--sizes 2b|9b] [--layers L] [--steps K] [--warmup W]
 
 For each design: tokens per second of a prefill of 2,048 tokens and of the generation loop's decode steps at batch 8
 and 1 (HIP graphs, greedy choice on the device), and the time of the kernels a step spends its time in, one by one at
@@ -33,6 +33,11 @@ four layers the first and third are attention layers (Gemma-2's heads; a window 
 width and half as many kv heads, 4 taps); the second and third have 8 squared-ReLU experts of half the dense width and 2
 identity outputs, 2 chosen, and a shared expert of a quarter of it, the others a dense feed-forward
 (`time_solulix_kernels`).
+The Kaderax sizes: the same width and vocabulary and as many runs of a layer (three layers in the middle run twice), each with a
+dense feed-forward of Gemma's width; of every three layers two are attentions through a latent of Vogunex's sizes (without a
+window, a sink per head, a gate per element), the third runs Gemma-2's attention heads (a cap, a temperature that changes every
+256 positions, biases that reach to a distance of 128, a gate per head) beside linear attention heads of 128 x 128 filling the
+width (`time_kaderax_kernels`).
 """
 import json
 import sys
@@ -140,6 +145,157 @@ def solulix_config(which, layers=0):
         start = (n // 2) // 4 * 4
         d["loop"] = {"start": start, "stop": start + looped, "times": 2}
     return SolulixConfig.from_dict(d)
+
+
+def kaderax_config(which, layers=0):
+    from .config import KaderaxConfig
+    g = dict(SIZES, **OTHER_SIZES[which])
+    runs = layers or g["num_hidden_layers"]
+    looped = 3 if runs >= 9 else 0
+    n = runs - looped
+    D, I, H, KV, hd = g["hidden_size"], g["intermediate_size"], g["num_attention_heads"], g["num_key_value_heads"], g["head_dim"]
+    lat = {"heads": 16, "dim": 128, "rot_dim": 64, "vdim": 128, "kv_rank": 192, "q_rank": 768, "scale": 192 ** -0.5,
+           "rot": {"base": 10000.0, "dims": 64}}
+    heads = D // 128
+    par = {"left": {"heads": H, "kv_heads": KV, "dim": hd, "vdim": hd, "scale": hd ** -0.5, "softcap": 50.0, "bias_max": 128,
+                    "q_temp": {"coef": 0.1, "every": 256}}, "left_scale": 0.7,
+           "right": {"heads": heads, "dim": 128, "vdim": 128, "decay": [1.0 - 2.0 ** (-1.0 - 8.0 * i / heads) for i in range(heads)]}, "right_scale": 0.6}
+    out = [{"type": "parallel" if i % 3 == 2 else "latent_attention", "mixer": par if i % 3 == 2 else lat, "mlp": {"kind": "dense", "ff": I}} for i in range(n)]
+    d = {"architecture": "Kaderax", "vocab": g["vocab_size"], "width": D, "norm": {"eps": 1e-6}, "residual_mult": 0.5, "layers": out}
+    if looped:
+        start = (n // 2) // 3 * 3
+        d["loop"] = {"start": start, "stop": start + looped, "times": 2}
+    return KaderaxConfig.from_dict(d)
+
+
+def time_kaderax_kernels(engine, cfg, batch, context, prefill_tokens):
+    """Microseconds of Kaderax's kernels at a decode step of `batch` sequences over `context` cached tokens and at a
+    prefill of `prefill_tokens`, each called once per layer on that layer's own weights, replayed from a HIP graph.
+    Products are priced by their weights' bytes (decode) or their flops against the bf16 matrix peak (prefill); the linear
+    attention's scan by its state's bytes (decode) or by the flops of its rows taken one by one, 5 key_dim value_dim a head
+    (a decay, an outer product, a product with the query), against the float32 peak (prefill); the attentions by the keys and
+    values a query sees (decode) or by their flops (prefill)."""
+    import torch
+    from .engine.batch import StepContext
+    model, ops, dev = engine.model, engine.model.rt.ops, engine.model.rt.device
+    bf, f32 = torch.bfloat16, torch.float32
+    blocks = [l.block for l in model.layers]
+    par = [b for b in blocks if hasattr(b.mixer, "sides")]
+    lat = [b for b in blocks if hasattr(b.mixer, "w_absorb")]
+    D = cfg.hidden_size
+    out = {}
+    timed = _timer(dev, out)
+    cache = engine.cache
+    entry = lambda group: next(i for i, e in enumerate(model.schedule) if model.layers[e.layer].block is group[0])
+    elems = lambda w: float(w.numel())
+    for rows, tag in ((batch, f"decode_b{batch}"), (prefill_tokens, f"prefill_{prefill_tokens}")):
+        decode = rows == batch
+        slots = [cache.acquire() for _ in range(batch if decode else 1)]
+        try:
+            for s in slots:
+                cache.grow(s, context if decode else rows)
+            counts = [1] * batch if decode else [rows]
+            starts = [context - 1] * batch if decode else [0]
+            ctx = StepContext(model.rt, cache, slots, counts, starts, [])
+            x = torch.randn((rows, D), device=dev).to(bf)
+            pairs = rows * (rows + 1) / 2.0
+            one = lambda f, **kw: timed(f"{tag}.{kw.pop('name')}", f, **kw)
+            prod = (lambda name, calls, w, m=rows: one(calls, name=name, bytes_each=2.0 * elems(w)) if decode
+                    else one(calls, name=name, flops_each=2.0 * m * elems(w)))
+            if lat:
+                mx = lat[0].mixer
+                H, dn, dr, dv, R, lrow = mx.num_heads, mx.nope_dim, mx.rope_dim, mx.value_dim, mx.rank, mx.row
+                site = cache.site(entry(lat))
+                table, pool, cap = ctx.page_table(site.group_index), site.tensor("latent"), 0
+                prod("latent_in", [(lambda b=b: ops.linear(x, b.mixer.w_joint, bf)) for b in lat], mx.w_joint)
+                joint = ops.linear(x, mx.w_joint, bf)
+                tail, gate, dq = joint[:, :lrow], joint[:, lrow:lrow + H * dv], joint[:, lrow + H * dv:lrow + H * dv + mx.query_rank]
+                one([lambda: ops.rms_norm(dq, mx.query_gain, 1e-6, bf)] * 16, name="latent_query_norm", bytes_each=rows * mx.query_rank * 4.0)
+                cq = torch.randn((rows, mx.query_rank), device=dev).to(bf)
+                prod("latent_uq", [(lambda b=b: ops.linear(cq, b.mixer.w_uq, bf)) for b in lat], mx.w_uq)
+                proj = ops.linear(cq, mx.w_uq, bf)
+                prep = lambda: ops.latent_prepare(proj, H, dn, dr, R, mx.latent_gain, 1e-6, mx.inv_freq, mx.position.rotary_dim, ctx.row_seq,
+                                                  ctx.row_pos, ctx.new_len, table, pool, cap, own=True, out_dtype=bf, tail=tail)
+                one([prep] * 16, name="latent_prepare", bytes_each=rows * (proj.shape[1] + H * dr + 3 * lrow) * 2.0)
+                q, mine = prep()
+                xq = proj.view(rows, H, dr + dn)[:, :, dr:]
+                qv = q.view(rows, H, lrow)[:, :, dr:]
+                one([(lambda b=b: ops.head_linear(xq, b.mixer.w_absorb, qv)) for b in lat], name="latent_absorb",
+                    bytes_each=2.0 * (elems(mx.w_absorb) + rows * H * (dn + R)))
+                if decode:
+                    per = next(g for g in (mx.DECODE_GROUP_LONG if context >= mx.LONG_KEYS else mx.DECODE_GROUP, 4, 2, 1) if H % g == 0)
+                    one([lambda: ops.attention_decode(q, H, 1, lrow, ctx.new_len, table, pool, pool, cap, mx.scale, 0.0, 0, bf,
+                                                      max_keys=ctx.max_rows_visible(site), head_groups=H // per,
+                                                      splits=ops.decode_splits(batch * (H // per), 1, lrow, context), sink=mx.sink)] * 8,
+                        name=f"latent_attention_{context}_keys", bytes_each=2.0 * batch * context * lrow)
+                else:
+                    one([lambda: ops.attention_prefill(q, mine, mine, H, 1, lrow, ctx.cu_rows, rows, mx.scale, 0.0, 0, bf, row_seq=ctx.row_seq,
+                                                       row_pos=ctx.row_pos, wide_weights=True, sink=mx.sink)] * 4,
+                        name="latent_attention", flops_each=4.0 * pairs * H * lrow)
+                o_lat = torch.randn((rows, H * lrow), device=dev).to(bf)
+                ov = o_lat.view(rows, H, lrow)[:, :, dr:]
+                one([(lambda b=b: ops.head_linear(ov, b.mixer.w_up, None, gate=gate)) for b in lat], name="latent_up_gated",
+                    bytes_each=2.0 * (elems(mx.w_up) + rows * H * (R + 2 * dv)))
+                hv = torch.randn((rows, H * dv), device=dev).to(bf)
+                prod("latent_o", [(lambda b=b: ops.linear(hv, b.mixer.w_o, bf, defer=True)) for b in lat], mx.w_o)
+            if par:
+                e = entry(par)
+                a, r = par[0].mixer.sides
+                H, KV, row = a.num_heads, a.num_kv_heads, a.row
+                site = cache.site(e)
+                table, kp, vp = ctx.page_table(site.group_index), site.tensor("k"), site.tensor("v")
+                prod("left_qkvg", [(lambda b=b: ops.linear(x, b.mixer.sides[0].w_qkv, bf, defer=decode)) for b in par], a.w_qkv)
+                qkv = ops.linear(x, a.w_qkv, bf, defer=decode)
+                by = lambda gate: ops.ByPosition(a.query_temperature, a.distance_table, gate)
+                if decode:
+                    one([lambda: ops.attention_decode_step(qkv, H, KV, row, None, 0, ctx.new_len, table, kp, vp, 0, a.query_scale, a.softcap, 0, bf,
+                                                           max_keys=ctx.max_rows_visible(site), by_position=by(a.gate_column))] * 8,
+                        name=f"left_attention_ctx{context}", bytes_each=2.0 * batch * context * 2 * KV * row)
+                else:
+                    q, k, v = qkv[:, :H * row], qkv[:, H * row:(H + KV) * row], qkv[:, (H + KV) * row:(H + 2 * KV) * row]
+                    one([lambda: ops.kv_write(k, v, KV, row, ctx.row_seq, ctx.row_pos, ctx.new_len, table, kp, vp, 0)] * 16,
+                        name="kv_write", bytes_each=rows * 2 * KV * row * 4.0)
+                    gate = qkv[:, a.gate_column:a.gate_column + H]
+                    one([lambda: ops.attention_prefill(q, k, v, H, KV, row, ctx.cu_rows, rows, a.query_scale, a.softcap, 0, bf, wide_weights=True,
+                                                       by_position=by(gate))] * 4,
+                        name="left_attention", flops_each=4.0 * pairs * H * row)
+                xa = torch.randn((rows, H * row), device=dev).to(bf)
+                prod("left_o", [(lambda b=b: ops.linear(xa, b.mixer.sides[0].w_o, bf, defer=True)) for b in par], a.w_o)
+                H, dk, dv = r.num_heads, r.key_dim, r.value_dim
+                qk, vv = H * dk, H * dv
+                prod("right_in_silu", [(lambda b=b: ops.linear_act(x, b.mixer.sides[1].w_in, bf, "silu", columns=2 * qk + vv)) for b in par], r.w_in)
+                u = ops.linear_act(x, r.w_in, bf, "silu", columns=2 * qk + vv)
+                state = cache.entry_state(e, "mixer.right.memory")
+                scan = lambda: ops.linear_scan(u[:, :qk], u[:, qk:2 * qk], u[:, 2 * qk:2 * qk + vv], r.decay, state, ctx.slot_ids, ctx.cu_rows,
+                                               ctx.max_count, H, dk, dv)
+                if decode:
+                    one([scan] * 8, name="linear_scan", bytes_each=batch * H * dk * dv * 8.0)
+                else:
+                    one([scan] * 4, name="linear_scan", flops_each=5.0 * rows * H * dk * dv, peak=PEAK_FLOPS["float32"])
+                y = torch.randn((rows, vv), device=dev)
+                one([lambda: ops.head_norm_gate(y, r.norm_gain, u[:, 2 * qk + vv:2 * (qk + vv)], 1e-6, 1, "sigmoid", bf)] * 16, name="norm_gate",
+                    bytes_each=rows * vv * 8.0)
+                xo = torch.randn((rows, vv), device=dev).to(bf)
+                prod("right_o", [(lambda b=b: ops.linear(xo, b.mixer.sides[1].w_o, bf, defer=True)) for b in par], r.w_o)
+            ff = blocks[0].feed_forward
+            prod("gate_up_gelu", [(lambda b=b: ops.gated_linear(x, b.feed_forward.w_gate_up, ff.intermediate_size, "gelu_tanh", bf)) for b in blocks],
+                 ff.w_gate_up[:2 * ff.intermediate_size])
+            xi = torch.randn((rows, ff.intermediate_size), device=dev).to(bf)
+            prod("down", [(lambda b=b: ops.linear(xi, b.feed_forward.w_down, bf, defer=True)) for b in blocks], ff.w_down)
+            stream, origin = torch.randn((rows, D), device=dev), torch.randn((rows, D), device=dev)
+            rows_a, rows_b, g = torch.randn((rows, D), device=dev).to(bf), torch.randn((rows, D), device=dev).to(bf), torch.ones(D, device=dev)
+            one([lambda: ops.join_rms_norm(stream, rows_a, rows_b, g, 1e-6, bf, wa=0.3, wb=0.4)] * 16, name="join_rms_norm",
+                bytes_each=rows * D * (4 + 4 + 2 + 2 + 2) + 4.0 * D)
+            mix = next((p for p in model.added if p is not None), None)
+            if mix is not None:
+                one([lambda: ops.join_rms_norm(stream, rows_a, None, None, 0.0, bf, origin=origin, wa=0.3, stack=1)] * 16, name="loop_operands",
+                    bytes_each=rows * D * (4 + 4 + 2 + 4 + 6))
+                xs = ops.join_rms_norm(stream, rows_a, None, None, 0.0, bf, origin=origin, stack=1)
+                prod("loop_in", [lambda: ops.linear(xs, mix.w, f32, defer=True)] * 4, mix.w)
+        finally:
+            for s in slots:
+                cache.release(s)
+    return out
 
 
 def time_solulix_kernels(engine, cfg, batch, context, prefill_tokens):
@@ -896,16 +1052,18 @@ def main(args):
     design = args.compare
     build, time_design = {"golepel": (golepel_config, time_golepel_kernels), "lutovik": (lutovik_config, time_lutovik_kernels),
                           "besulix": (besulix_config, time_besulix_kernels), "vogunex": (vogunex_config, time_vogunex_kernels),
-                          "solulix": (solulix_config, time_solulix_kernels)}[design]
-    # the design it stands next to: the closest of the others
-    beside_lutovik = ("lutovik", lutovik_config, time_lutovik_kernels, "Lutovik")
-    other, build_other, time_other, title = {"besulix": beside_lutovik, "vogunex": beside_lutovik, "solulix": beside_lutovik}.get(
-        design, ("gemma2", gemma_config, time_kernels, "Gemma-2"))
-    line = {"metric": f"{design.capitalize()} next to {title} at {which} layer sizes: prefill and decode tok/s", "unit": "tok/s", "n_gpus": 1,
+                          "solulix": (solulix_config, time_solulix_kernels), "kaderax": (kaderax_config, time_kaderax_kernels)}[design]
+    # the designs it stands next to: the closest of the others
+    lutovik = ("lutovik", lutovik_config, time_lutovik_kernels, "Lutovik")
+    vogunex = ("vogunex", vogunex_config, time_vogunex_kernels, "Vogunex")
+    others = {"besulix": [lutovik], "vogunex": [lutovik], "solulix": [lutovik], "kaderax": [vogunex, lutovik]}.get(
+        design, [("gemma2", gemma_config, time_kernels, "Gemma-2")])
+    line = {"metric": f"{design.capitalize()} next to {' and '.join(o[3] for o in others)} at {which} layer sizes: prefill and decode tok/s", "unit": "tok/s", "n_gpus": 1,
             "steps": steps, "warmup": warmup, "dtype": "bf16", "data": "synthetic: seeded random weights N(0, 0.02) and uniform-random token ids",
             "sizes": which, "designs": {}, "kernels": {}}
     most = max(PREFILL_TOKENS, batch * (prompt + steps + warmup + 128)) + 1024
-    for name, cfg in ((design, build(which, args.layers)), (other, build_other(which, args.layers))):
+    for name, make, time_kernels_of in [(design, build, time_design)] + [o[:3] for o in others]:
+        cfg = make(which, args.layers)
         run = Run(cfg, max(batch, 8), most, name)
         pre = run.prefill()
         d = {"layers": len(cfg.layers) if hasattr(cfg, "layers") else cfg.num_hidden_layers, "runs": len(run.model.schedule), "weights_GB": round(run.weight_bytes / 1e9, 2),
@@ -915,17 +1073,16 @@ def main(args):
             d[f"decode_b{b}_tok_s"] = round(b * steps / dt, 1)
             d[f"decode_b{b}_ms_per_step"] = round(dt / steps * 1e3, 4)
         print(f"[compare] {name}: {d}", file=sys.stderr, flush=True)
-        if name == design:
-            k = time_design(run.engine, cfg, batch, prompt + 40, PREFILL_TOKENS)
-        else:
-            k = time_other(run.engine, cfg, batch, prompt + 40, PREFILL_TOKENS)
+        k = time_kernels_of(run.engine, cfg, batch, prompt + 40, PREFILL_TOKENS)
         for kn, row in k.items():
             print(f"[compare] {name} kernel {kn}: {row}", file=sys.stderr, flush=True)
         line["designs"][name] = d
         line["kernels"][name] = k
         run.close()
-    g, m = line["designs"][design], line["designs"][other]
+    g = line["designs"][design]
     line["value"] = g[f"decode_b{batch}_tok_s"]
-    line[f"ratio_to_{other}"] = {k: round(g[k] / m[k], 3) for k in g if k.endswith("tok_s")}
+    for other in others:
+        m = line["designs"][other[0]]
+        line[f"ratio_to_{other[0]}"] = {k: round(g[k] / m[k], 3) for k in g if k.endswith("tok_s")}
     print(json.dumps(line), flush=True)
     return 0
