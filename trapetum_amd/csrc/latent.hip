@@ -139,6 +139,7 @@ head_linear_mfma_k(const bf16_t* __restrict__ x, long x_row, long x_head, const 
     const bf16_t* xh = x + (size_t)h * x_head;
     const bf16_t* wh = w + (size_t)h * N * K;
     const uint4 zero = make_uint4(0, 0, 0, 0);
+    const bool quads = gate && gate_row % 4 == 0 && N % 4 == 0 && (uintptr_t)gate % 8 == 0;
     const bool wide = o_row % 4 == 0 && o_head % 4 == 0 && (uintptr_t)out % 8 == 0;
     Tile t;
     t.run(K,
@@ -153,8 +154,11 @@ head_linear_mfma_k(const bf16_t* __restrict__ x, long x_row, long x_head, const 
             bf16_t* dst = out + (size_t)m * o_row + (size_t)h * o_head + n;
             if (gate) {
                 const bf16_t* gp = gate + (size_t)m * gate_row + (size_t)h * N + n;
+                union { uint2 u; bf16_t h[4]; } g4;
+                if (quads) g4.u = *reinterpret_cast<const uint2*>(gp);
+                else for (int v = 0; v < 4; v++) g4.h[v] = gp[n + v < N ? v : 0];
 #pragma unroll
-                for (int v = 0; v < 4; v++) t.acc[0][i][j][v] = gated_by(t.acc[0][i][j][v], bf16_to_f32(gp[n + v < N ? v : 0]));
+                for (int v = 0; v < 4; v++) t.acc[0][i][j][v] = gated_by(t.acc[0][i][j][v], bf16_to_f32(g4.h[v]));
             }
             if (wide && n + 3 < N) {                      // the lane's four neighbours in one store
                 uint2 o;

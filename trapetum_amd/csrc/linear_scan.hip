@@ -27,8 +27,7 @@ struct LinearScanArgs {
     const int* slot_ids; const int* cu_rows; float* y;   // y [M, H dv]
     int n_seq, H, dk, dv;
     int n_chunks;                                        // chunks of the longest sequence
-    float* ends;                                         // [sequence x chunk, H, dv, dk]: E
-    bf16_t* starts;                                      // [sequence x chunk, H, 3 terms, dv, dk]: S_0
+    float* chunks;                                       // [sequence x chunk, H, dv, dk]: E, which gives way to S_0
 };
 
 namespace {
@@ -36,7 +35,7 @@ constexpr int LC = 64;                           // tokens of a chunk
 constexpr int LCP = LC + 8;                      // a row of 64 tokens in LDS
 constexpr int EB = 64;                           // value elements a block of scan_ends_k takes
 template <typename T> struct alignas(sizeof(T) * 4) Four { T v[4]; };
-union LFrag { uint4 u; ls_bf16x8 v; uint32_t w[4]; uint2 half[2]; };
+union LFrag { uint4 u; ls_bf16x8 v; uint32_t w[4]; };
 
 // a and b as sums of three bfloat16 numbers: word n holds their nth terms
 __device__ __forceinline__ void split_two(float a, float b, uint32_t (&word)[3]) {
@@ -183,7 +182,7 @@ scan_ends_k(LinearScanArgs x) {
     for (int m = 0; m < 3; m++)
 #pragma unroll
         for (int s = 0; s < 2; s++) vf[m][s].u = *reinterpret_cast<const uint4*>(Vt + (m * EB + wave * 16 + r) * LCP + s * 32 + g * 8);
-    float* out = x.ends + ((size_t)blockIdx.x * x.H + h) * dv * dk;
+    float* out = x.chunks + ((size_t)blockIdx.x * x.H + h) * dv * dk;
     for (int j = 0; j < dkp / 16; j++) {
         ls_f32x4 acc = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
@@ -210,23 +209,18 @@ scan_carry_k(LinearScanArgs x) {
     const int chunks = (count + LC - 1) / LC;
     const float dec = x.decay[h], whole = power(dec, LC), last = power(dec, count - (chunks - 1) * LC);
     float4* st = reinterpret_cast<float4*>(x.state + ((size_t)x.slot_ids[seq] * x.H + h) * size + at);
-    const float* ends = x.ends + ((size_t)seq * x.n_chunks * x.H + h) * size + at;
-    bf16_t* starts = x.starts + ((size_t)seq * x.n_chunks * x.H + h) * 3 * size + at;
+    float* mine = x.chunks + ((size_t)seq * x.n_chunks * x.H + h) * size + at;
     const size_t apart = (size_t)x.H * size;
     float4 s = *st;
     for (int c0 = 0; c0 < chunks; c0 += AHEAD) {
         float4 E[AHEAD];
 #pragma unroll
-        for (int u = 0; u < AHEAD; u++) E[u] = *reinterpret_cast<const float4*>(ends + (size_t)min(c0 + u, chunks - 1) * apart);
+        for (int u = 0; u < AHEAD; u++) E[u] = *reinterpret_cast<const float4*>(mine + (size_t)min(c0 + u, chunks - 1) * apart);
 #pragma unroll
         for (int u = 0; u < AHEAD; u++) {
             const int c = c0 + u;
             if (c >= chunks) break;
-            uint32_t lo[3], hi[3];
-            split_two(s.x, s.y, lo);
-            split_two(s.z, s.w, hi);
-#pragma unroll
-            for (int m = 0; m < 3; m++) *reinterpret_cast<uint2*>(starts + (size_t)c * 3 * apart + (size_t)m * size) = make_uint2(lo[m], hi[m]);
+            *reinterpret_cast<float4*>(mine + (size_t)c * apart) = s;
             const float f = c + 1 < chunks ? whole : last;
             s.x = __builtin_fmaf(f, s.x, E[u].x);
             s.y = __builtin_fmaf(f, s.y, E[u].y);
@@ -237,39 +231,48 @@ scan_carry_k(LinearScanArgs x) {
     *st = s;
 }
 
-// The outputs of one chunk.  grid (sequences x chunks, heads), four waves: wave w takes the tokens 16 w .. 16 w + 15, a lane
-// one of them (column r).  Weights are formed turned, (k_s . q_t) with the keys as rows, so that a lane's sums are, as they
-// lie, its operand of the product with the values: k place 8 g + i of step u is key 32 u + 4 g + i for i < 4 and key
-// 32 u + 16 + 4 g + i - 4 for the others, and the values are read from LDS in that order.
+// The outputs of one chunk.  grid (sequences x chunks, heads), four waves.  Wave w first forms the weights of the tokens
+// 16 w .. 16 w + 15, turned (keys as rows), so that a lane's four sums are neighbours of one token's row of weights; they meet
+// in LDS in three terms.  Then wave w takes the value elements 16 w .. 16 w + 15, + 64, .. of all 64 tokens: its rows of S_0
+// come from memory once, asked for before anything else, and are split into their terms in registers.
 template <int KS>
 __global__ void __launch_bounds__(256)
 scan_outputs_k(LinearScanArgs x) {
     extern __shared__ __attribute__((aligned(16))) bf16_t ls_lds[];
     constexpr int KP = KS * 32 + 8;
-    bf16_t* const Kr = ls_lds;                             // [LC][KP]
-    bf16_t* const Vt = ls_lds + LC * KP;                   // [dv up to a multiple of 16][LCP]
+    bf16_t* const Kr = ls_lds;                             // [LC][KP] keys by rows
+    bf16_t* const Qr = Kr + LC * KP;                       // [LC][KP] queries by rows
+    bf16_t* const P = Qr + LC * KP;                        // [3][LC tokens][LCP keys]
+    bf16_t* const Vt = P + 3 * LC * LCP;                   // [dv up to a multiple of 16][LCP]: values turned
     __shared__ float pow_s[LC + 1];
     const int seq = blockIdx.x / x.n_chunks, chunk = blockIdx.x % x.n_chunks, h = blockIdx.y;
     const int begin = x.cu_rows[seq] + chunk * LC, n = min(LC, x.cu_rows[seq + 1] - begin);
     if (n <= 0) return;
-    const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, r = lane & 15, g = lane >> 4, dk = x.dk, dv = x.dv;
+    const int tid = threadIdx.x, wave = __builtin_amdgcn_readfirstlane(tid >> 6), lane = tid & 63, r = lane & 15, g = lane >> 4, dk = x.dk, dv = x.dv;
     const uint4 zero = make_uint4(0, 0, 0, 0);
-    if (tid <= LC) pow_s[tid] = power(x.decay[h], tid);
-    LFrag qf[KS];
-    {
-        const bf16_t* qp = (const bf16_t*)x.q + (size_t)(begin + min(wave * 16 + r, n - 1)) * x.q_stride + (size_t)h * dk;
+    const float* const S = x.chunks + ((size_t)blockIdx.x * x.H + h) * dv * dk;
+    float4 sr[KS][2];                                      // eight neighbouring elements of row e0 + r of S_0 by k step
+    auto rows_of = [&](int e0) {
+        const float* p = S + (size_t)min(e0 + r, dv - 1) * dk;
 #pragma unroll
         for (int s = 0; s < KS; s++) {
-            const int d = s * 32 + g * 8;
-            qf[s].u = *reinterpret_cast<const uint4*>(qp + (d < dk ? d : 0));
+            const int d = s * 32 + g * 8, dc = d < dk ? d : 0;           // (past dk: the queries' elements are zero)
+            sr[s][0] = *reinterpret_cast<const float4*>(p + dc);
+            sr[s][1] = *reinterpret_cast<const float4*>(p + dc + 4);
         }
-    }
+    };
+    rows_of(min(wave * 16, dv - 1));
+    if (tid <= LC) pow_s[tid] = power(x.decay[h], tid);
     {
         const bf16_t* kb = (const bf16_t*)x.k + (size_t)begin * x.k_stride + (size_t)h * dk;
-        for (int i = tid; i < LC * KS * 4; i += 256) {     // keys by rows, zeros past a row's end
-            const int t = i / (KS * 4), d = (i - t * (KS * 4)) * 8;
-            const uint4 f = *reinterpret_cast<const uint4*>(kb + (size_t)min(t, n - 1) * x.k_stride + (d < dk ? d : 0));
-            *reinterpret_cast<uint4*>(Kr + t * KP + d) = d < dk ? f : zero;
+        const bf16_t* qb = (const bf16_t*)x.q + (size_t)begin * x.q_stride + (size_t)h * dk;
+#pragma unroll
+        for (int i0 = 0; i0 < LC * KS * 4; i0 += 256) {    // (past the chunk's end: its last row; past a row's end: zeros)
+            const int i = i0 + tid, t = i / (KS * 4), d = (i - t * (KS * 4)) * 8, dc = d < dk ? d : 0;
+            const uint4 kf = *reinterpret_cast<const uint4*>(kb + (size_t)min(t, n - 1) * x.k_stride + dc);
+            const uint4 qf = *reinterpret_cast<const uint4*>(qb + (size_t)min(t, n - 1) * x.q_stride + dc);
+            *reinterpret_cast<uint4*>(Kr + t * KP + d) = d < dk ? kf : zero;
+            *reinterpret_cast<uint4*>(Qr + t * KP + d) = d < dk ? qf : zero;
         }
         const int pair = tid & 31, t0 = pair * 2, ta = min(t0, n - 1), tb = min(t0 + 1, n - 1);
         union Eight { uint4 u; bf16_t h[8]; };
@@ -284,18 +287,14 @@ scan_outputs_k(LinearScanArgs x) {
             for (int i = 0; i < 8; i++) *reinterpret_cast<uint32_t*>(Vt + (c * 8 + i) * LCP + t0) = (uint32_t)a.h[i] | ((uint32_t)b.h[i] << 16);
         }
     }
-    if (dk < KS * 32) {
-#pragma unroll
-        for (int s = 0; s < KS; s++) if (s * 32 + g * 8 >= dk) qf[s].u = zero;
-    }
     __syncthreads();
-    const int t = wave * 16 + r;
-    LFrag pf[2][3];                                        // the weights' terms by k step
+    {
+        const int t = wave * 16 + r;
+        LFrag qf[KS];
 #pragma unroll
-    for (int u = 0; u < 2; u++)
+        for (int s = 0; s < KS; s++) qf[s].u = *reinterpret_cast<const uint4*>(Qr + t * KP + s * 32 + g * 8);
 #pragma unroll
-        for (int half = 0; half < 2; half++) {
-            const int j = 2 * u + half;                    // keys 16 j .. 16 j + 15: none beyond the wave's own tile
+        for (int j = 0; j < 4; j++) {                      // keys 16 j .. 16 j + 15: zeros beyond the wave's own tile
             ls_f32x4 acc = {0.f, 0.f, 0.f, 0.f};
             if (j <= wave) {
 #pragma unroll
@@ -315,46 +314,62 @@ scan_outputs_k(LinearScanArgs x) {
             split_two(w[0], w[1], lo);
             split_two(w[2], w[3], hi);
 #pragma unroll
-            for (int m = 0; m < 3; m++) pf[u][m].half[half] = make_uint2(lo[m], hi[m]);
+            for (int m = 0; m < 3; m++) *reinterpret_cast<uint2*>(P + (m * LC + t) * LCP + j * 16 + g * 4) = make_uint2(lo[m], hi[m]);
         }
-    const float since = pow_s[t + 1];
-    const bf16_t* S = x.starts + ((size_t)blockIdx.x * x.H + h) * 3 * dv * dk;
-    float* yr = x.y + ((size_t)(begin + min(t, n - 1)) * x.H + h) * dv;
+    }
+    __syncthreads();
     const bool quads = dv % 4 == 0;
-    for (int e0 = 0; e0 < dv; e0 += 16) {
-        const bf16_t* Sr = S + (size_t)min(e0 + r, dv - 1) * dk;
+    for (int e0 = wave * 16; e0 < dv; e0 += 64) {
         LFrag sf[KS][3];
 #pragma unroll
-        for (int s = 0; s < KS; s++)
+        for (int s = 0; s < KS; s++) {
+            const float v[8] = {sr[s][0].x, sr[s][0].y, sr[s][0].z, sr[s][0].w, sr[s][1].x, sr[s][1].y, sr[s][1].z, sr[s][1].w};
 #pragma unroll
-            for (int m = 0; m < 3; m++) {
-                const int d = s * 32 + g * 8;
-                sf[s][m].u = *reinterpret_cast<const uint4*>(Sr + (size_t)m * dv * dk + (d < dk ? d : 0));     // (past dk: q's elements are zero)
+            for (int i = 0; i < 4; i++) {
+                uint32_t w[3];
+                split_two(v[2 * i], v[2 * i + 1], w);
+#pragma unroll
+                for (int m = 0; m < 3; m++) sf[s][m].w[i] = w[m];
             }
-        ls_f32x4 in = {0.f, 0.f, 0.f, 0.f}, own = {0.f, 0.f, 0.f, 0.f};
+        }
+        if (e0 + 64 < dv) rows_of(e0 + 64);
+        LFrag vf[2];
 #pragma unroll
-        for (int u = 0; u < 2; u++)
-            if (u == 0 || wave >= 2) {
-                LFrag vf;
-                const bf16_t* vr = Vt + (e0 + r) * LCP + u * 32 + g * 4;
-                vf.half[0] = *reinterpret_cast<const uint2*>(vr);
-                vf.half[1] = *reinterpret_cast<const uint2*>(vr + 16);
+        for (int u = 0; u < 2; u++) vf[u].u = *reinterpret_cast<const uint4*>(Vt + (e0 + r) * LCP + u * 32 + g * 8);
 #pragma unroll
-                for (int m = 2; m >= 0; m--) own = mma(vf, pf[u][m], own);
+        for (int tt = 0; tt < 4; tt++) {                   // 16 tokens, a lane one of them
+            ls_f32x4 in = {0.f, 0.f, 0.f, 0.f}, in1 = in, own = in;
+#pragma unroll
+            for (int s = 0; s < KS; s++) {
+                LFrag qf;
+                qf.u = *reinterpret_cast<const uint4*>(Qr + (tt * 16 + r) * KP + s * 32 + g * 8);
+                in1 = mma(sf[s][2], qf, in1);
+                in = mma(sf[s][0], qf, in);
+                in1 = mma(sf[s][1], qf, in1);
             }
 #pragma unroll
-        for (int m = 2; m >= 0; m--)
+            for (int u = 0; u < 2; u++)
+                if (u == 0 || tt >= 2) {                   // (the lower half's tokens see no key of the upper half)
 #pragma unroll
-            for (int s = 0; s < KS; s++) in = mma(sf[s][m], qf[s], in);
-        const int e = e0 + g * 4;
-        if (t < n) {
-            if (quads) {
-                if (e < dv)
-                    *reinterpret_cast<float4*>(yr + e) = make_float4(__builtin_fmaf(since, in[0], own[0]), __builtin_fmaf(since, in[1], own[1]),
-                                                                     __builtin_fmaf(since, in[2], own[2]), __builtin_fmaf(since, in[3], own[3]));
-            } else {
+                    for (int m = 2; m >= 0; m--) {
+                        LFrag pf;
+                        pf.u = *reinterpret_cast<const uint4*>(P + (m * LC + tt * 16 + r) * LCP + u * 32 + g * 8);
+                        own = mma(vf[u], pf, own);
+                    }
+                }
+            in = in + in1;
+            const int t = tt * 16 + r, e = e0 + g * 4;
+            const float since = pow_s[t + 1];
+            if (t < n) {
+                float* yr = x.y + ((size_t)(begin + t) * x.H + h) * dv;
+                if (quads) {
+                    if (e < dv)
+                        *reinterpret_cast<float4*>(yr + e) = make_float4(__builtin_fmaf(since, in[0], own[0]), __builtin_fmaf(since, in[1], own[1]),
+                                                                         __builtin_fmaf(since, in[2], own[2]), __builtin_fmaf(since, in[3], own[3]));
+                } else {
 #pragma unroll
-                for (int i = 0; i < 4; i++) if (e + i < dv) yr[e + i] = __builtin_fmaf(since, in[i], own[i]);
+                    for (int i = 0; i < 4; i++) if (e + i < dv) yr[e + i] = __builtin_fmaf(since, in[i], own[i]);
+                }
             }
         }
     }
@@ -364,7 +379,7 @@ static size_t ls_align(size_t n) { return (n + 255) / 256 * 256; }
 
 extern "C" long tp_linear_scan_workspace_bytes(int n_seq, int n_chunks, int H, int dk, int dv) {
     const size_t el = (size_t)n_seq * n_chunks * H * dk * dv;
-    return (long)(ls_align(el * sizeof(float)) + ls_align(el * 3 * sizeof(bf16_t)));
+    return (long)ls_align(el * sizeof(float));
 }
 
 // q, k [M, H dk], v [M, H dv] as views of wider rows of one dtype; decay float32 [H]; state [slots, H, dv, dk] float32, left
@@ -373,23 +388,22 @@ extern "C" int tp_linear_scan(const void* q, long q_stride, const void* k, long 
                               const float* decay, float* state, const int* slot_ids, const int* cu_rows, float* y, int n_seq, int H,
                               int dk, int dv, int n_chunks, void* workspace, long workspace_bytes, void* stream) {
     TP_REQUIRE(n_seq > 0 && H > 0 && dk > 0 && dv > 0, "linear_scan: empty shape sequences=%d heads=%d key=%d value=%d", n_seq, H, dk, dv);
-    TP_REQUIRE(dk <= 256 && dv <= 512, "linear_scan: heads of %d x %d exceed 256 x 512", dk, dv);
+    TP_REQUIRE(dk <= 256 && dv <= 256, "linear_scan: heads of %d x %d exceed 256 x 256", dk, dv);
     TP_REQUIRE(H <= 65535, "linear_scan: %d heads exceed one launch", H);
     TP_REQUIRE(q && k && v && decay && state && slot_ids && cu_rows && y, "linear_scan: null operand");
     TP_REQUIRE(dtype == TP_BF16 || dtype == TP_F32, "linear_scan: unknown dtype %d", dtype);
     hipStream_t s = (hipStream_t)stream;
-    LinearScanArgs x{q, q_stride, k, k_stride, v, v_stride, decay, state, slot_ids, cu_rows, y, n_seq, H, dk, dv, n_chunks, nullptr, nullptr};
+    LinearScanArgs x{q, q_stride, k, k_stride, v, v_stride, decay, state, slot_ids, cu_rows, y, n_seq, H, dk, dv, n_chunks, nullptr};
     if (n_chunks > 0) {
         TP_REQUIRE(dtype == TP_BF16 && dk % 8 == 0 && dv % 8 == 0 && q_stride % 8 == 0 && k_stride % 8 == 0 && v_stride % 8 == 0 &&
                    (uintptr_t)q % 16 == 0 && (uintptr_t)k % 16 == 0 && (uintptr_t)v % 16 == 0, "linear_scan: chunks need bfloat16 rows of whole 16-byte pieces");
         TP_REQUIRE((long)n_seq * n_chunks <= 0x7fffffffL, "linear_scan: %d chunks of %d sequences exceed one launch", n_chunks, n_seq);
         TP_REQUIRE(workspace && (uintptr_t)workspace % 16 == 0 && workspace_bytes >= tp_linear_scan_workspace_bytes(n_seq, n_chunks, H, dk, dv),
                    "linear_scan: a workspace of %ld bytes is too small", workspace_bytes);
-        x.ends = (float*)workspace;
-        x.starts = (bf16_t*)((char*)workspace + ls_align((size_t)n_seq * n_chunks * H * dk * dv * sizeof(float)));
+        x.chunks = (float*)workspace;
         const int units = n_seq * n_chunks, ks = tp_cdiv(dk, 32), ksr = ks <= 4 ? ks : (ks <= 6 ? 6 : 8);
         const size_t lds_ends = (size_t)(3 * EB + (dk + 15) / 16 * 16) * LCP * sizeof(bf16_t);
-        const size_t lds_out = ((size_t)LC * (ksr * 32 + 8) + (size_t)((dv + 15) / 16 * 16) * LCP) * sizeof(bf16_t);
+        const size_t lds_out = ((size_t)2 * LC * (ksr * 32 + 8) + 3 * LC * LCP + (size_t)((dv + 15) / 16 * 16) * LCP) * sizeof(bf16_t);
         auto room = [](const void* kernel, size_t bytes) {       // more LDS than a kernel gets without asking
             return bytes <= 65536 || hipFuncSetAttribute(kernel, hipFuncAttributeMaxDynamicSharedMemorySize, (int)bytes) == hipSuccess;
         };

@@ -797,7 +797,6 @@ class HipOps:
 
     LINEAR_CHUNK = 64              # tokens of a chunk (the kernel library's)
     LINEAR_CHUNKS_FROM = 16        # rows of the longest sequence from which a bfloat16 step runs in chunks
-    MAX_LINEAR_VALUES = 512
 
     def linear_scan(self, q, k, v, decay, state, slot_ids, cu_rows, max_count, heads, dk, dv, chunks=None):
         """S <- decay S + v k^T, o = S q, row after row of every sequence from state[slot] (float32 [slots, heads, dv, dk]),
@@ -808,8 +807,8 @@ class HipOps:
         qs, ks, vs = self._rows(q, "linear_scan q"), self._rows(k, "linear_scan k"), self._rows(v, "linear_scan v")
         if tuple(q.shape) != (m, heads * dk) or tuple(k.shape) != (m, heads * dk) or tuple(v.shape) != (m, heads * dv) or not (q.dtype == k.dtype == v.dtype):
             raise KernelError(f"linear_scan: q, k {(m, heads * dk)} and v {(m, heads * dv)} of one dtype")
-        if dk > self.MAX_SCAN_DIM or dv > self.MAX_LINEAR_VALUES:
-            raise KernelError(f"linear_scan: heads of {dk} x {dv} exceed {self.MAX_SCAN_DIM} x {self.MAX_LINEAR_VALUES}")
+        if dk > self.MAX_SCAN_DIM or dv > self.MAX_SCAN_DIM:
+            raise KernelError(f"linear_scan: heads of {dk} x {dv} exceed {self.MAX_SCAN_DIM} x {self.MAX_SCAN_DIM}")
         if decay.dtype != torch.float32 or decay.numel() != heads or not decay.is_contiguous():
             raise KernelError(f"linear_scan: the decays must be contiguous float32 [{heads}]")
         if state.dtype != torch.float32 or state.dim() != 4 or tuple(state.shape[1:]) != (heads, dv, dk) or not state.is_contiguous():
