@@ -308,7 +308,9 @@ attn_decode_k(DecodeArgs a) {
         for (int i = 0; i < 4; i++) {
             const int u = tb + g * 4 + i, t = u < kept_al ? u : u + gap;
             const bool ok = (t >= lo || t < a.keep) && u < t_end;
-            s[i] = ok ? score_of(s[i], scale_c, a.cap, soc) + (BY_POSITION ? bs[i] : 0.f) : -INFINITY;
+            float score = score_of(s[i], scale_c, a.cap, soc);
+            if constexpr (BY_POSITION) score += bs[i];
+            s[i] = ok ? score : -INFINITY;
             mx = fmaxf(mx, s[i]);
         }
         mx = fmaxf(mx, __shfl_xor(mx, 16, 64));

@@ -33,6 +33,7 @@ static inline float4 epi_constants(const GemmArgs& a) {
 // gate), or SiLU where n is one of the first `units` columns (below 2^24: exact as a float) and as summed elsewhere
 __device__ __forceinline__ float squared_relu_f(float o) { o = fmaxf(o, 0.f); return o * o; }
 __device__ __forceinline__ float plain_epilogue(int epilogue, float o, float4 epi, int n) {
+    if (epilogue == TP_EPI_NONE) return o;
     if (epilogue == TP_EPI_SILU) return (float)n < epi.z ? gate_act_fast(o, epi) : o;
     return epilogue == TP_EPI_SOFTCAP ? softcap_f(o, epi.x) : (epilogue == TP_EPI_RELU2 ? squared_relu_f(o) : o);
 }
